@@ -48,6 +48,7 @@ MODULES = {
             "ssm_scan.hip",
             "linear_scan.hip",
             "attention_f32.hip",
+            "talk_attention.hip",
             "latent_attention.hip",
             "moe_route.hip",
             "activation.hip",
@@ -58,7 +59,7 @@ MODULES = {
     },
 }
 
-HEADERS = ["common.h", "mfma_layouts.h", "dtype_io.h"]
+HEADERS = ["common.h", "mfma_layouts.h", "dtype_io.h", "cache_chunk.h"]
 # hipcc makes packed-fp32 instructions on its own from plain float code; keep
 # them off for every kernel of this package
 DEVICE_FLAGS = ["-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]

@@ -249,20 +249,26 @@ class DeltaMixerSpec:
     """Gated delta rule: ``heads`` value heads of ``vdim`` columns, ``kv_heads``
     query/key heads of ``dim`` columns shared by groups of value heads, a
     causal convolution of ``conv`` taps + silu on q, k and v, unit-norm q/k, a
-    data-dependent decay and write strength per head."""
+    data-dependent decay and write strength per head. ``channel_decay``: one
+    decay per head AND key channel, from a projection through ``a_rank``
+    columns, and an output gate through ``g_rank`` columns (0: one head's
+    size until a checkpoint's tensor shapes say otherwise)."""
 
     heads: int
     kv_heads: int
     dim: int
     vdim: int
     conv: int = 4
+    channel_decay: bool = False
+    a_rank: int = 0
+    g_rank: int = 0
 
     @property
     def conv_channels(self) -> int:
         return 2 * self.kv_heads * self.dim + self.heads * self.vdim
 
     @classmethod
-    def from_dict(cls, d: dict) -> "DeltaMixerSpec":
+    def from_dict(cls, d: dict, channel_decay: bool = False) -> "DeltaMixerSpec":
         heads = int(d["heads"])
         kv = int(d.get("kv_heads", heads))
         if kv < 1 or heads % kv:
@@ -273,7 +279,109 @@ class DeltaMixerSpec:
             dim=int(d["dim"]),
             vdim=int(d.get("vdim", d["dim"])),
             conv=int(d.get("conv", 4)),
+            channel_decay=channel_decay,
         )
+
+
+@dataclass
+class DifferentialMixerSpec:
+    """Differential attention: every query head has two score maps of ``dim``
+    columns each over the same values; head output = first - lambda * second,
+    RMS-normed, times (1 - ``diff``). A causal convolution of ``conv`` taps on
+    q, k and v (0: none), per-head q/k norm, rotation in pairs (2i, 2i+1) of
+    the first ``rot_dims`` columns with optional YaRN scaling, scores times
+    ``scale`` then soft-capped (0: no cap), sliding window (0: none)."""
+
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    diff: float
+    conv: int = 0
+    softcap: float = 0.0
+    window: int = 0
+    rot_dims: int = 0
+    rot_base: float = 10000.0
+    # {"factor", "original", "fast", "slow"} or None
+    rot_scaling: Optional[dict] = None
+
+    @property
+    def conv_channels(self) -> int:
+        return 2 * (self.heads + self.kv_heads) * self.dim + self.kv_heads * self.vdim
+
+    @classmethod
+    def from_dict(cls, d: dict) -> "DifferentialMixerSpec":
+        heads = int(d["heads"])
+        kv = int(d.get("kv_heads", heads))
+        if kv < 1 or heads % kv:
+            raise ValueError("heads must be a multiple of kv_heads")
+        rot = d.get("rot") or {}
+        sc = rot.get("scaling")
+        return cls(
+            heads=heads,
+            kv_heads=kv,
+            dim=int(d["dim"]),
+            vdim=int(d.get("vdim", d["dim"])),
+            scale=float(d["scale"]),
+            diff=float(d["diff"]),
+            conv=int(d.get("conv") or 0),
+            softcap=float(d.get("softcap") or 0.0),
+            window=int((d.get("mask") or {}).get("size", 0)),
+            rot_dims=int(rot.get("dims", 0)),
+            rot_base=float(rot.get("base", 10000.0)),
+            rot_scaling={k: float(sc[k]) for k in ("factor", "original", "fast", "slow")}
+            if sc else None,
+        )
+
+
+@dataclass
+class TalkingMixerSpec:
+    """Attention whose heads' scores are mixed by a learned matrix before the
+    softmax: scores times ``scale`` plus a learned bias by distance bucket
+    (logarithmic up to ``bias_max``), sliding window (0: none), one added to
+    the softmax denominator, values that are the un-normed keys, an
+    element-wise output gate. ``buckets``: rows of the bias table (taken from
+    the checkpoint's tensor when weights are loaded)."""
+
+    heads: int
+    kv_heads: int
+    dim: int
+    scale: float
+    bias_max: float
+    window: int = 0
+    buckets: int = 32
+
+    @classmethod
+    def from_dict(cls, d: dict) -> "TalkingMixerSpec":
+        heads = int(d["heads"])
+        kv = int(d.get("kv_heads", heads))
+        if kv < 1 or heads % kv:
+            raise ValueError("heads must be a multiple of kv_heads")
+        if int(d.get("vdim", d["dim"])) != int(d["dim"]):
+            raise ValueError("the values are the keys: vdim must equal dim")
+        return cls(
+            heads=heads,
+            kv_heads=kv,
+            dim=int(d["dim"]),
+            scale=float(d["scale"]),
+            bias_max=float(d["bias_max"]),
+            window=int((d.get("mask") or {}).get("size", 0)),
+        )
+
+
+@dataclass
+class SiluGLUSpec:
+    """Dense gated feed-forward down(silu(gate h) * (up h))."""
+
+    ff: int
+
+    @classmethod
+    def from_dict(cls, d: dict) -> "SiluGLUSpec":
+        kind = d.get("kind", "dense")
+        if kind != "dense":
+            raise ValueError(f"unsupported feed-forward kind {kind!r}")
+        return cls(ff=int(d["ff"]))
 
 
 @dataclass
@@ -514,6 +622,24 @@ def laperax_layer_spec(kind: str, mixer: dict, mlp: Optional[dict]):
     raise ValueError(f"unknown layer type {kind!r}")
 
 
+def mededra_layer_spec(kind: str, mixer: dict, mlp: Optional[dict]):
+    """One Mededra layer: differential attention, or talking-heads attention
+    beside a channel-decay delta rule, and an optional dense feed-forward."""
+    ff = SiluGLUSpec.from_dict(mlp) if mlp else None
+    if kind == "attention":
+        return HybridLayerSpec(
+            kind, differential=DifferentialMixerSpec.from_dict(mixer), mlp=ff
+        )
+    if kind == "parallel":
+        return HybridLayerSpec(
+            kind,
+            talking=TalkingMixerSpec.from_dict(mixer["left"]),
+            delta=DeltaMixerSpec.from_dict(mixer["right"], channel_decay=True),
+            attention_scale=0.5, ssm_scale=0.5, mlp=ff,
+        )
+    raise ValueError(f"unknown layer type {kind!r}")
+
+
 @dataclass
 class LoopSpec:
     """Layers ``start .. stop-1`` run ``times`` times in a row with the same
@@ -536,9 +662,12 @@ class HybridLayerSpec:
     latent: Optional[LatentAttentionSpec] = None
     retention: Optional[RetentionMixerSpec] = None
     delta: Optional[DeltaMixerSpec] = None
+    differential: Optional[DifferentialMixerSpec] = None
+    talking: Optional[TalkingMixerSpec] = None
     attention_scale: float = 1.0
     ssm_scale: float = 1.0
-    # GLUSpec, MoESpec, MLPSpec, SoftmaxMoESpec or SquaredReluMoESpec
+    # GLUSpec, SiluGLUSpec, MoESpec, MLPSpec, SoftmaxMoESpec or
+    # SquaredReluMoESpec
     mlp: Optional[object] = None
 
 
@@ -551,6 +680,8 @@ class HybridModelConfig:
     hidden_size: int
     layers: list
     rms_norm_eps: float = 1e-5
+    # residual-stream norms work on this many equal parts of a row
+    norm_groups: int = 1
     embedding_scale: float = 1.0
     dtype: str = "bfloat16"
     model_name: str = "merulorn"
@@ -586,19 +717,29 @@ class HybridModelConfig:
     def has_recurrent_state(self) -> bool:
         return any(
             l.ssm is not None or l.retention is not None or l.delta is not None
+            or (l.differential is not None and l.differential.conv > 1)
             for l in self.layers
         )
 
     def kv_bytes_per_block(self, block_size: int, itemsize: int) -> int:
         per_token = 0
+        scales = 0
         for i, _ in self.layer_runs():
             a, lt = self.layers[i].attention, self.layers[i].latent
+            df, tk = self.layers[i].differential, self.layers[i].talking
+            if df is not None:
+                per_token += df.kv_heads * (2 * df.dim + df.vdim)
+            if tk is not None:
+                # un-normed keys, which are the values too, and their fp32
+                # inverse RMS
+                per_token += tk.kv_heads * tk.dim
+                scales += 4
             if a is not None:
                 per_token += a.kv_heads * (a.dim + a.vdim)
             if lt is not None and lt.kv_from is None:
                 # one row per token: latent + shared rotated key part
                 per_token += lt.cache_dim
-        return per_token * block_size * itemsize
+        return (per_token * itemsize + scales) * block_size
 
     @classmethod
     def from_dict(cls, cfg: dict, model_name: str = "merulorn") -> "HybridModelConfig":
@@ -607,6 +748,9 @@ class HybridModelConfig:
         for entry in cfg["layers"]:
             kind = entry["type"]
             mixer = entry["mixer"]
+            if arch == "Mededra":
+                layers.append(mededra_layer_spec(kind, mixer, entry.get("mlp")))
+                continue
             if arch == "Laperax":
                 layers.append(laperax_layer_spec(kind, mixer, entry.get("mlp")))
                 continue
@@ -653,6 +797,7 @@ class HybridModelConfig:
             hidden_size=int(cfg["width"]),
             layers=layers,
             rms_norm_eps=float(cfg.get("norm", {}).get("eps", 1e-5)),
+            norm_groups=int(cfg.get("norm", {}).get("groups", 1)),
             embedding_scale=float(cfg.get("embedding", {}).get("scale", 1.0)),
             model_name=model_name,
             architecture=cfg.get("architecture", "Merulorn"),

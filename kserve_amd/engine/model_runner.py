@@ -151,7 +151,7 @@ class ModelRunner:
         caches = []
         kv_bytes = state_bytes = 0
         for kv, state in self._layout:
-            k = v = conv = ssm = None
+            k = v = conv = ssm = k_scale = None
             if kv is not None:
                 g, d, dv = kv
                 k = alloc((num_blocks, g, bs, d), dtype=dtype, device=self.device)
@@ -159,6 +159,10 @@ class ModelRunner:
                 if dv:  # dv 0: the values are columns of the key rows
                     v = alloc((num_blocks, g, bs, dv), dtype=dtype, device=self.device)
                     kv_bytes += v.numel() * v.itemsize
+            if state.get("k_scale"):
+                # one fp32 factor per cached key row
+                k_scale = alloc((num_blocks, bs), dtype=torch.float32, device=self.device)
+                kv_bytes += k_scale.numel() * k_scale.itemsize
             # a recurrent layer keeps a convolution history, a matrix state
             # or both
             if state.get("conv"):
@@ -169,7 +173,7 @@ class ModelRunner:
                 shape, dt = state["ssm"]
                 ssm = alloc((slots, *shape), dtype=dt, device=self.device)
                 state_bytes += ssm.numel() * ssm.itemsize
-            caches.append(LayerCache(k, v, conv, ssm))
+            caches.append(LayerCache(k, v, conv, ssm, k_scale))
         self.kv_caches = caches
         self.num_gpu_blocks = num_blocks
         self.num_state_slots = slots if state_bytes else 0

@@ -14,6 +14,7 @@ they need ``cu_seqlens`` / ``seq_of_token`` (flat-batch layout) and
 
 from __future__ import annotations
 
+import math
 from typing import NamedTuple, Optional
 
 import torch
@@ -24,6 +25,7 @@ from kserve_amd import ops
 from kserve_amd.engine.config import (
     AttentionMixerSpec,
     DeltaMixerSpec,
+    DifferentialMixerSpec,
     GLUSpec,
     LatentAttentionSpec,
     MLPSpec,
@@ -32,8 +34,13 @@ from kserve_amd.engine.config import (
     SoftmaxMoESpec,
     SquaredReluMoESpec,
     SSMMixerSpec,
+    TalkingMixerSpec,
 )
-from kserve_amd.ops.torch_ref import rotary_inv_freq
+from kserve_amd.ops.torch_ref import (
+    distance_buckets,
+    rotary_inv_freq,
+    yarn_inv_freq,
+)
 
 
 class LayerCache(NamedTuple):
@@ -46,6 +53,8 @@ class LayerCache(NamedTuple):
     # matrix state of a recurrent layer, fp32: [slots, heads, vdim, state]
     # (state-space scan) or [slots, heads, vdim, dim] (linear attention)
     ssm: Optional[torch.Tensor] = None
+    k_scale: Optional[torch.Tensor] = None  # [blocks, block] fp32: a factor
+    #                                         per cached key row
 
 
 def _param(*shape, dtype):
@@ -933,3 +942,313 @@ class SquaredReluMoE(nn.Module):
         if dense:
             return self._dense(h, dense_w, extra)
         return self._sorted(h, idx, w, extra)
+
+
+class DifferentialAttention(nn.Module):
+    """Softmax attention with two score maps per head over the same values:
+    the head's output is map 1's minus lambda times map 2's, divided by its
+    RMS, times (1 - diff), with lambda = exp(lq1 . lk1) - exp(lq2 . lk2) +
+    diff, one number for the layer. q, k and v pass a short causal convolution
+    (no activation; history kept per sequence), q and k a per-head-and-map RMS
+    norm and a rotation in pairs (2i, 2i+1) with optional YaRN frequencies;
+    scores are scaled and soft-capped; sliding window.
+
+    A cached key row holds both maps side by side ([kv_heads, 2 dim]); the
+    attention kernel takes 2 x heads query heads of ``dim`` columns, in
+    storage order (head, map), and reads a map as a column range of the row.
+    q|k|v are one fused GEMM."""
+
+    MAPS = 2
+
+    def __init__(self, width: int, spec: DifferentialMixerSpec, eps: float, dtype):
+        super().__init__()
+        s = spec
+        self.spec = s
+        self.eps = eps
+        self.dtype = dtype
+        if s.rot_dims % 2 or s.rot_dims > s.dim:
+            raise ValueError("rot dims must be even and at most the head size")
+        self.q_w = s.heads * self.MAPS * s.dim
+        self.k_w = s.kv_heads * self.MAPS * s.dim
+        self.v_w = s.kv_heads * s.vdim
+        self.qkv = _param(self.q_w + self.k_w + self.v_w, width, dtype=dtype)
+        self.conv_w = (
+            _param(s.conv_channels, s.conv, dtype=torch.float32) if s.conv else None
+        )
+        self.q_norm = _param(s.dim, dtype=torch.float32)
+        self.k_norm = _param(s.dim, dtype=torch.float32)
+        # lq1, lk1, lq2, lk2
+        self.lambda_vecs = _param(4, s.dim, dtype=torch.float32)
+        self.o_proj = _param(width, s.heads * s.vdim, dtype=dtype)
+        inv_freq, self.rot_mult = None, 1.0
+        if s.rot_dims:
+            inv_freq, self.rot_mult = yarn_inv_freq(s.rot_dims, s.rot_base, s.rot_scaling)
+        self.register_buffer("inv_freq", inv_freq, persistent=False)
+        self.register_buffer("lam", torch.zeros(1, dtype=torch.float32), persistent=False)
+
+    def kv_shape(self):
+        s = self.spec
+        return (s.kv_heads, self.MAPS * s.dim, s.vdim)
+
+    def state_shapes(self):
+        s = self.spec
+        if s.conv > 1:
+            return {"conv": ((s.conv - 1, s.conv_channels), self.dtype)}
+        return {}
+
+    def load(self, get, prefix: str):
+        dt = self.dtype
+        self.qkv.copy_(
+            torch.cat([get(prefix + n).to(dt) for n in ("q", "k", "v")], dim=0)
+        )
+        if self.conv_w is not None:
+            self.conv_w.copy_(
+                torch.cat(
+                    [get(prefix + n + ".conv").float() for n in ("q", "k", "v")], dim=0
+                )
+            )
+        self.q_norm.copy_(get(prefix + "q.norm").float())
+        self.k_norm.copy_(get(prefix + "k.norm").float())
+        for i, n in enumerate(("lq1", "lk1", "lq2", "lk2")):
+            self.lambda_vecs[i].copy_(get(prefix + n).float())
+        self.o_proj.copy_(get(prefix + "o").to(dt))
+        self.finish_load()
+
+    def finish_load(self):
+        v = self.lambda_vecs
+        self.lam.copy_(
+            torch.exp((v[0] * v[1]).sum()) - torch.exp((v[2] * v[3]).sum())
+            + self.spec.diff
+        )
+
+    def forward(self, h, positions, cache: LayerCache, meta):
+        s = self.spec
+        x = F.linear(h, self.qkv)
+        if s.conv > 1:
+            x = ops.causal_conv_silu(
+                x, self.conv_w, None, cache.conv, positions, meta.seq_of_token,
+                meta.cu_seqlens, meta.state_slots, silu=False,
+            )
+        elif s.conv:
+            x = x.float() * self.conv_w[:, 0]
+        a, b = self.q_w, self.q_w + self.k_w
+        heads = self.MAPS * s.heads
+        qn = ops.qk_headnorm_rope_cache(
+            x[:, :a], x[:, a:b], x[:, b:], self.q_norm, self.k_norm, positions,
+            meta.slot_mapping, cache.k, cache.v, self.eps, heads, self.inv_freq,
+            pairs=True, rot_mult=self.rot_mult, maps=self.MAPS,
+        )
+        o = ops.ctx_attention_f32(
+            qn, cache.k, cache.v, meta.block_tables, meta.cu_seqlens,
+            meta.context_lens, s.scale, meta.max_seqlen, heads,
+            out_dtype=torch.float32, window=s.window, maps=self.MAPS,
+            softcap=s.softcap,
+        )
+        o = ops.diff_combine(o, self.lam, s.heads, self.eps, 1.0 - s.diff, self.dtype)
+        return F.linear(o, self.o_proj)
+
+
+class TalkingHeadsAttention(nn.Module):
+    """Softmax attention whose heads' scores are mixed by a learned matrix
+    before the softmax. q and k are RMS-normed over the whole projection;
+    values are the keys before that norm. score_g = q_g . k * scale + a learned
+    bias by distance bucket; s_h = sum_g talk[h, g] score_g; sliding window;
+    one more term exp(0) in the softmax denominator; every output element
+    times the sigmoid of a projection of the sublayer input.
+
+    Pages hold the un-normed keys only (they are the values as well) and one
+    fp32 1/rms per row, which the kernel multiplies the scores by; the key
+    norm's weight is folded into the query. The bias is mixed over the heads
+    and laid out per distance once, when weights are loaded. q|k|gate rows
+    are the mixer's share of a fused projection (``mix``)."""
+
+    def __init__(self, width: int, spec: TalkingMixerSpec, eps: float, dtype):
+        super().__init__()
+        s = spec
+        self.spec = s
+        self.eps = eps
+        self.dtype = dtype
+        self.width = width
+        self.q_w = s.heads * s.dim
+        self.k_w = s.kv_heads * s.dim
+        self.proj_width = 2 * self.q_w + self.k_w
+        self.qkg = _param(self.proj_width, width, dtype=dtype)
+        self.q_norm = _param(self.q_w, dtype=torch.float32)
+        self.k_norm = _param(self.k_w, dtype=torch.float32)
+        self.rel = _param(s.buckets, s.heads, dtype=torch.float32)
+        self.talk = _param(s.heads, s.heads, dtype=torch.float32)
+        self.o_proj = _param(width, self.q_w, dtype=dtype)
+        # distances with a bias of their own: up to the window's edge, or up
+        # to where the last bucket starts
+        n = int(math.ceil(s.bias_max)) + 1
+        if s.window:
+            n = min(n, s.window)
+        self.register_buffer(
+            "bias", torch.zeros(s.heads, n, dtype=torch.float32), persistent=False
+        )
+        # q norm's weight times the k norm's of the head's group
+        self.register_buffer(
+            "q_weight", torch.ones(self.q_w, dtype=torch.float32), persistent=False
+        )
+
+    def kv_shape(self):
+        # vdim 0: the values are the key rows
+        return (self.spec.kv_heads, self.spec.dim, 0)
+
+    def state_shapes(self):
+        return {"k_scale": True}
+
+    def load(self, get, prefix: str):
+        dt = self.dtype
+        rel = get(prefix + "rel").float()
+        if rel.shape != self.rel.shape:
+            self.rel = _param(*rel.shape, dtype=torch.float32).to(self.qkg.device)
+        self.rel.copy_(rel)
+        self.qkg.copy_(
+            torch.cat([get(prefix + n).to(dt) for n in ("q", "k", "g")], dim=0)
+        )
+        self.q_norm.copy_(get(prefix + "q.norm").float())
+        self.k_norm.copy_(get(prefix + "k.norm").float())
+        self.talk.copy_(get(prefix + "talk").float())
+        self.o_proj.copy_(get(prefix + "o").to(dt))
+        self.finish_load()
+
+    def finish_load(self):
+        row = distance_buckets(
+            self.bias.shape[1], self.rel.shape[0], self.spec.bias_max
+        ).to(self.rel.device)
+        # sum_g talk[h, g] rel[bucket(n), g]
+        mixed = self.talk.double() @ self.rel.double().t()[:, row]
+        self.bias.copy_(mixed.float())
+        s = self.spec
+        kw = self.k_norm.view(s.kv_heads, s.dim)
+        kw = kw.repeat_interleave(s.heads // s.kv_heads, dim=0)
+        self.q_weight.copy_(self.q_norm * kw.reshape(-1))
+
+    def mix(self, proj, positions, cache: LayerCache, meta):
+        s = self.spec
+        a, b = self.q_w, self.q_w + self.k_w
+        qn = ops.talk_prep_cache(
+            proj[:, :a], proj[:, a:b], self.q_weight, meta.slot_mapping,
+            cache.k, cache.k_scale, self.eps,
+        )
+        o = ops.talk_attention(
+            qn, cache.k, cache.k_scale, meta.block_tables, meta.cu_seqlens,
+            meta.context_lens, s.scale, meta.max_seqlen, s.heads, self.talk,
+            self.bias, s.window, gate=proj[:, b:], out_dtype=self.dtype,
+        )
+        return F.linear(o, self.o_proj)
+
+    def forward(self, h, positions, cache: LayerCache, meta):
+        return self.mix(F.linear(h, self.qkg), positions, cache, meta)
+
+
+class ChannelDeltaMixer(nn.Module):
+    """Gated delta rule with one decay per head and key channel: q, k, v
+    through a short causal convolution + silu, unit-norm q/k (q also times
+    dim^-1/2), g = exp(-exp(A_log_h) softplus(a2 (a1 h) + dt_bias)) acting on
+    the state's key rows, write strength sigmoid(b h), read-out after the
+    write. Head outputs are RMS-normed with one weight vector shared by the
+    heads and gated by sigmoid(g2 (g1 h)). q|k|v|a1|g1|b rows are the mixer's
+    share of a fused projection (``mix``); the two second factors are one
+    block-diagonal GEMM on the adjacent a1|g1 columns."""
+
+    UNIT_EPS = GatedDeltaMixer.UNIT_EPS
+
+    def __init__(self, width: int, spec: DeltaMixerSpec, eps: float, dtype):
+        super().__init__()
+        s = spec
+        self.spec = s
+        self.eps = eps
+        self.dtype = dtype
+        self.width = width
+        self.qk_w = s.kv_heads * s.dim
+        self.v_w = s.heads * s.vdim
+        self.decay_w = s.heads * s.dim
+        self.conv_w = _param(s.conv_channels, s.conv, dtype=torch.float32)
+        self.a_log = _param(s.heads, dtype=torch.float32)
+        self.dt_bias = _param(self.decay_w, dtype=torch.float32)
+        self.norm_w = _param(s.vdim, dtype=torch.float32)
+        self.o_proj = _param(width, self.v_w, dtype=dtype)
+        self._make_projections(s.a_rank or s.dim, s.g_rank or s.vdim, None)
+
+    def _make_projections(self, a_rank: int, g_rank: int, device):
+        s = self.spec
+        self.a_rank, self.g_rank = a_rank, g_rank
+        self.low_at = s.conv_channels
+        self.b_at = self.low_at + a_rank + g_rank
+        # rows padded to whole 16-byte units so that every token's row of the
+        # projection starts aligned
+        self.proj_width = -(-(self.b_at + s.heads) // 8) * 8
+        self.proj = _param(self.proj_width, self.width, dtype=self.dtype)
+        self.low2 = _param(
+            self.decay_w + self.v_w, a_rank + g_rank, dtype=self.dtype
+        )
+        if device is not None:
+            self.proj.data = self.proj.data.to(device)
+            self.low2.data = self.low2.data.to(device)
+
+    def state_shapes(self):
+        s = self.spec
+        out = {"ssm": ((s.heads, s.vdim, s.dim), torch.float32)}
+        if s.conv > 1:
+            out["conv"] = ((s.conv - 1, s.conv_channels), self.dtype)
+        return out
+
+    def load(self, get, prefix: str):
+        dt = self.dtype
+        a1, g1 = get(prefix + "a1"), get(prefix + "g1")
+        if (a1.shape[0], g1.shape[0]) != (self.a_rank, self.g_rank):
+            self._make_projections(a1.shape[0], g1.shape[0], self.o_proj.device)
+        self.proj.zero_()
+        self.proj[: self.b_at + self.spec.heads].copy_(
+            torch.cat(
+                [get(prefix + n).to(dt) for n in ("q", "k", "v")]
+                + [a1.to(dt), g1.to(dt), get(prefix + "b").to(dt)], dim=0,
+            )
+        )
+        self.low2.zero_()
+        self.low2[: self.decay_w, : self.a_rank].copy_(get(prefix + "a2").to(dt))
+        self.low2[self.decay_w :, self.a_rank :].copy_(get(prefix + "g2").to(dt))
+        self.conv_w.copy_(
+            torch.cat([get(prefix + n + ".conv").float() for n in ("q", "k", "v")], dim=0)
+        )
+        self.a_log.copy_(get(prefix + "A_log").float())
+        self.dt_bias.copy_(get(prefix + "dt_bias").float())
+        self.norm_w.copy_(get(prefix + "norm").float())
+        self.o_proj.copy_(get(prefix + "o").to(dt))
+
+    def finish_load(self):
+        """After a random fill: the block-diagonal's off blocks are zero."""
+        self.low2[: self.decay_w, self.a_rank :].zero_()
+        self.low2[self.decay_w :, : self.a_rank].zero_()
+
+    def mix(self, proj, positions, cache: LayerCache, meta):
+        s = self.spec
+        low = F.linear(proj[:, self.low_at : self.b_at], self.low2)
+        if s.conv > 1:
+            qkv = ops.causal_conv_silu(
+                proj[:, : self.low_at], self.conv_w, None, cache.conv, positions,
+                meta.seq_of_token, meta.cu_seqlens, meta.state_slots,
+            )
+        else:
+            x = proj[:, : self.low_at].float() * self.conv_w[:, 0]
+            qkv = x * torch.sigmoid(x)
+        g = ops.delta_unit_decay(
+            qkv, s.kv_heads, s.dim, s.dim ** -0.5, self.UNIT_EPS,
+            low[:, : self.decay_w], self.a_log, self.dt_bias,
+        )
+        a = self.qk_w
+        o = ops.linear_scan(
+            qkv[:, :a], qkv[:, a : 2 * a], qkv[:, 2 * a :], cache.ssm, positions,
+            meta.cu_seqlens, meta.state_slots, s.kv_heads,
+            b_raw=proj[:, self.b_at : self.b_at + s.heads], channel_decay=g,
+        )
+        on = ops.gated_group_rms_norm(
+            o, low[:, self.decay_w :], self.norm_w, self.eps, s.heads, self.dtype,
+            gate_after=True, gate_sigmoid=True,
+        )
+        return F.linear(on, self.o_proj)
+
+    def forward(self, h, positions, cache: LayerCache, meta):
+        return self.mix(F.linear(h, self.proj), positions, cache, meta)

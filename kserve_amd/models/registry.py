@@ -62,6 +62,12 @@ register(
     "kserve_amd.models.laperax.LaperaxForCausalLM",
     ("kserve_amd_seq_C",),
 )
+register(
+    "Mededra",
+    "kserve_amd.engine.config.HybridModelConfig",
+    "kserve_amd.models.mededra.MededraForCausalLM",
+    ("kserve_amd_seq_C",),
+)
 
 
 def architecture_of(config_json: dict) -> str:

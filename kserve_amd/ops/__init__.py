@@ -365,37 +365,41 @@ def add_rms_norm_f32res(
 
 
 def gated_group_rms_norm(
-    y, z, weight, eps: float, groups: int, out_dtype, gate_after: bool = False
+    y, z, weight, eps: float, groups: int, out_dtype, gate_after: bool = False,
+    gate_sigmoid: bool = False,
 ):
-    """RMS norm of fp32 ``y`` in ``groups`` equal parts with a silu(z) gate:
-    on the input of the norm, or (``gate_after``) on its output. ``weight``
+    """RMS norm of fp32 ``y`` in ``groups`` equal parts with a silu(z) gate
+    (``gate_sigmoid``: sigmoid(z)): on the input of the norm, or
+    (``gate_after``) on its output. ``weight``
     may be shorter than a row (it repeats: one vector shared by the groups)
     or None."""
     if y.is_cuda:
         out = torch.empty(y.shape, dtype=out_dtype, device=y.device)
         _native_seq("gated_group_rms_norm").gated_group_rms_norm(
-            out, y, z, weight, float(eps), int(groups), bool(gate_after)
+            out, y, z, weight, float(eps), int(groups), bool(gate_after),
+            bool(gate_sigmoid),
         )
         return out
     return torch_ref.gated_group_rms_norm(
-        y, z, weight, eps, groups, out_dtype, gate_after
+        y, z, weight, eps, groups, out_dtype, gate_after, gate_sigmoid
     )
 
 
 def causal_conv_silu(
-    x_in, w, bias, conv_state, positions, seq_of_token, cu_seqlens, slots
+    x_in, w, bias, conv_state, positions, seq_of_token, cu_seqlens, slots,
+    silu: bool = True,
 ):
-    """Depthwise causal conv + silu over a flat varlen batch; reads and then
+    """Depthwise causal conv (+ silu) over a flat varlen batch; reads and then
     advances each sequence's conv history in ``conv_state[slot]``."""
     if x_in.is_cuda:
         out = _f32_like(x_in.shape[0], x_in.shape[1], x_in)
         _native_seq("causal_conv_silu").causal_conv_silu(
             out, x_in, w, bias, conv_state, positions, seq_of_token,
-            cu_seqlens, slots,
+            cu_seqlens, slots, bool(silu),
         )
         return out
     return torch_ref.causal_conv_silu(
-        x_in, w, bias, conv_state, positions, cu_seqlens, slots
+        x_in, w, bias, conv_state, positions, cu_seqlens, slots, silu
     )
 
 
@@ -439,6 +443,7 @@ def ctx_attention_f32(
     q, k_cache, v_cache, block_tables, cu_q, ctx_lens, scale: float,
     max_q_len: int, heads: int, gate=None, out_dtype=torch.float32,
     sink=None, chunk: int = 0, out_inv_freq=None, window: int = 0,
+    maps: int = 1, softcap: float = 0.0,
 ):
     """Paged causal attention with fp32 scores and weights. Optional parts:
     ``gate`` [T, heads] (output times sigmoid), ``sink`` [heads] fp32 (one
@@ -447,7 +452,11 @@ def ctx_attention_f32(
     sees itself and the window-1 positions before it), ``out_inv_freq``
     [vdim/2] fp32 (each head output turned back by its query position).
     ``v_cache`` may be a view of the leading columns of ``k_cache`` (values
-    that are a prefix of the keys are stored once)."""
+    that are a prefix of the keys are stored once). ``maps``: every cached key
+    row holds that many keys side by side, and query head h reads number
+    h % maps of its group's (all of them share the group's values); ``softcap``:
+    scores become softcap * tanh(score / softcap). With bf16 pages the output
+    may be bf16 or fp32."""
     if q.is_cuda:
         out = torch.empty(
             (q.shape[0], heads * v_cache.shape[3]), dtype=out_dtype,
@@ -456,31 +465,36 @@ def ctx_attention_f32(
         _native_seq("ctx_attention_f32").ctx_attention_f32(
             out, q, k_cache, v_cache, block_tables, cu_q, ctx_lens, gate,
             float(scale), int(max_q_len), int(heads), sink, int(chunk),
-            out_inv_freq, int(window),
+            out_inv_freq, int(window), int(maps), float(softcap),
         )
         return out
     return torch_ref.ctx_attention_f32(
         q, k_cache, v_cache, block_tables, cu_q, ctx_lens, scale, heads,
-        gate, out_dtype, sink, chunk, out_inv_freq, window,
+        gate, out_dtype, sink, chunk, out_inv_freq, window, maps, softcap,
     )
 
 
 def qk_headnorm_rope_cache(
     q, k, v, qw, kw, positions, slot_mapping, k_cache, v_cache, eps: float,
     heads: int, qk_inv_freq=None, v_unit_norm: bool = False, v_inv_freq=None,
+    pairs: bool = False, rot_mult: float = 1.0, maps: int = 1,
 ):
-    """Per-head q/k RMS norm (weights [dim]) + rotary positions, optional
-    unit-norm and rotation of the values, KV page scatter; returns q fp32."""
+    """Per-head q/k RMS norm (weights [dim]) + rotary positions (``pairs``:
+    coordinate 2i turns with 2i+1 instead of i with i + half; turned
+    coordinates times ``rot_mult``), optional unit-norm and rotation of the
+    values, KV page scatter (``maps`` k heads share a cached row and a value
+    head); returns q fp32. q, k, v may be fp32 beside bf16 pages."""
     if q.is_cuda:
         q_out = _f32_like(q.shape[0], q.shape[1], q)
         _native_seq("qk_headnorm_rope_cache").qk_headnorm_rope_cache(
             q_out, q, k, v, qw, kw, positions, slot_mapping, k_cache, v_cache,
             float(eps), int(heads), qk_inv_freq, bool(v_unit_norm), v_inv_freq,
+            bool(pairs), float(rot_mult), int(maps),
         )
         return q_out
     return torch_ref.qk_headnorm_rope_cache(
         q, k, v, qw, kw, positions, slot_mapping, k_cache, v_cache, eps,
-        heads, qk_inv_freq, v_unit_norm, v_inv_freq,
+        heads, qk_inv_freq, v_unit_norm, v_inv_freq, pairs, rot_mult, maps,
     )
 
 
@@ -726,24 +740,27 @@ def unit_norm_heads(
 def linear_scan(
     q, k, v, state, positions, cu_seqlens, slots, qk_heads: int,
     decay=None, a_raw=None, b_raw=None, a_log=None, dt_bias=None,
+    channel_decay=None,
 ):
     """Linear-attention recurrence over a flat varlen batch; carries
     ``state[slot]`` ([heads, V, K] fp32). q, k [T, qk_heads*K] and
     v [T, heads*V] are fp32 (rows may be strided). With ``decay`` [heads]:
     S <- d S + k v^T. Without: the gated delta rule with
     g = exp(-exp(a_log) softplus(a_raw + dt_bias)), b = sigmoid(b_raw):
-    S <- g S; S <- S + k (b (v - S^T k))^T. Output o = S^T q, fp32."""
+    S <- g S; S <- S + k (b (v - S^T k))^T; ``channel_decay`` [T, heads*K] fp32
+    gives g per head and key channel (then a_raw, a_log, dt_bias are not
+    used). Output o = S^T q, fp32."""
     if q.is_cuda:
         heads, V = state.shape[1], state.shape[2]
         o = _f32_like(q.shape[0], heads * V, q)
         _native_seq("linear_scan").linear_scan(
-            o, q, k, v, decay, a_raw, b_raw, a_log, dt_bias, state, positions,
-            cu_seqlens, slots, int(qk_heads),
+            o, q, k, v, decay, a_raw, b_raw, a_log, dt_bias, channel_decay,
+            state, positions, cu_seqlens, slots, int(qk_heads),
         )
         return o
     return torch_ref.linear_scan(
         q, k, v, state, positions, cu_seqlens, slots, qk_heads, decay, a_raw,
-        b_raw, a_log, dt_bias,
+        b_raw, a_log, dt_bias, channel_decay,
     )
 
 
@@ -763,3 +780,108 @@ def scale_softcap(x, scale: float, cap: float):
         _native_seq("scale_softcap").scale_softcap(out, x, float(scale), float(cap))
         return out
     return torch_ref.scale_softcap(x, scale, cap)
+
+
+# -- two score maps, mixed score heads, per-channel decays, grouped norms -----
+
+def post_group_norm_add(
+    residual, delta, weight, groups: int, eps: float, out_dtype, delta2=None,
+    pre_w=None, pre_w2=None, next_weight=None, want_out: bool = True,
+):
+    """fp32 residual (in place) += GroupRMS(d) * weight, where d is ``delta``
+    or, with ``delta2``, half of rms(delta) * pre_w + rms(delta2) * pre_w2;
+    returns the new residual in ``out_dtype`` or, with ``next_weight``, its
+    group RMS norm times that weight."""
+    if residual.is_cuda:
+        out = (
+            torch.empty(residual.shape, dtype=out_dtype, device=residual.device)
+            if want_out else None
+        )
+        _native_seq("post_group_norm_add").post_group_norm_add(
+            residual, delta, weight, delta2, pre_w, pre_w2, int(groups),
+            float(eps), out, next_weight,
+        )
+        return out
+    return torch_ref.post_group_norm_add(
+        residual, delta, weight, groups, eps, out_dtype, delta2, pre_w,
+        pre_w2, next_weight, want_out,
+    )
+
+
+def diff_combine(o, lam, heads: int, eps: float, mult: float, out_dtype):
+    """fp32 rows with two outputs per head side by side -> their difference
+    first - lam * second (lam: fp32 tensor of one element), divided by its RMS
+    over the head, times ``mult``."""
+    if o.is_cuda:
+        out = torch.empty(
+            (o.shape[0], o.shape[1] // 2), dtype=out_dtype, device=o.device
+        )
+        _native_seq("diff_combine").diff_combine(
+            out, o, lam, int(heads), float(eps), float(mult)
+        )
+        return out
+    return torch_ref.diff_combine(o, lam, heads, eps, mult, out_dtype)
+
+
+def talk_prep_cache(
+    q, k, w, slot_mapping, k_cache, k_scale, eps: float,
+):
+    """Whole-row RMS norm of q times ``w`` (fp32, returned); the un-normed
+    keys to the pages, 1 / rms of every key row to ``k_scale`` [blocks, block]
+    (a weight of the key norm belongs into ``w``: it commutes into the
+    query)."""
+    if q.is_cuda:
+        q_out = _f32_like(q.shape[0], q.shape[1], q)
+        _native_seq("talk_prep_cache").talk_prep_cache(
+            q_out, q, k, w, slot_mapping, k_cache, k_scale, float(eps)
+        )
+        return q_out
+    return torch_ref.talk_prep_cache(
+        q, k, w, slot_mapping, k_cache, k_scale, eps
+    )
+
+
+def talk_attention(
+    q, k_cache, k_scale, block_tables, cu_q, ctx_lens, scale: float,
+    max_q_len: int, heads: int, talk, bias, window: int = 0, gate=None,
+    out_dtype=torch.float32,
+):
+    """Paged causal attention whose scores are mixed over the heads before
+    the softmax: s_h = sum_g talk[h, g] (q_g . k) k_scale scale +
+    bias[h, distance] (``bias`` [heads, n] fp32, constant past distance
+    n - 1), one added to the softmax denominator, the cached keys as values,
+    ``gate`` [T, heads*dim]: output times its sigmoid per element."""
+    if q.is_cuda:
+        out = torch.empty(
+            (q.shape[0], heads * k_cache.shape[3]), dtype=out_dtype,
+            device=q.device,
+        )
+        _native_seq("talk_attention").talk_attention(
+            out, q, k_cache, k_scale, block_tables, cu_q, ctx_lens, talk, bias,
+            gate, float(scale), int(max_q_len), int(heads), int(window),
+        )
+        return out
+    return torch_ref.talk_attention(
+        q, k_cache, k_scale, block_tables, cu_q, ctx_lens, scale, heads, talk,
+        bias, window, gate, out_dtype,
+    )
+
+
+def delta_unit_decay(
+    qkv, qk_heads: int, dim: int, q_scale: float, eps: float, a_raw, a_log,
+    dt_bias,
+):
+    """What the channel-decay delta rule reads, in one pass per token: fp32
+    rows [q | k | v] get unit-norm q and k heads in place (q times
+    ``q_scale``); returns exp(-exp(a_log) softplus(a_raw + dt_bias)) per head
+    and key channel, fp32 [T, heads*dim]."""
+    if qkv.is_cuda:
+        g = _f32_like(qkv.shape[0], a_raw.shape[1], qkv)
+        _native_seq("delta_unit_decay").delta_unit_decay(
+            qkv, g, a_raw, a_log, dt_bias, int(qk_heads), int(dim),
+            float(q_scale), float(eps),
+        )
+        return g
+    return torch_ref.delta_unit_decay(
+        qkv, qk_heads, dim, q_scale, eps, a_raw, a_log, dt_bias
+    )

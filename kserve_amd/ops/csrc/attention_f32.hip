@@ -38,17 +38,20 @@
 //    partial (max, sum, O) through LDS at the end, so the group's K/V is read
 //    once. Head sizes are padded up to 64/128/256 with zeros. An optional
 //    per-(token, head) gate multiplies the result by sigmoid(gate).
+//    Optional: scores soft-capped with cap * tanh(score / cap); and `maps` keys
+//    side by side in one cached row, query head h reading number h % maps.
+//    Prefill reads the map's columns of the row as a head of its own; decode
+//    keeps all maps of a group in one block, reads the whole row once and
+//    pads every query with zeros outside its map's columns.
 #include <type_traits>
 
-#include "dtype_io.h"
+#include "cache_chunk.h"
 
 namespace {
 
 constexpr int NT = 256;
 constexpr int NW = NT / WAVE_SIZE;
 constexpr int BK = 64;  // keys per staged tile
-
-typedef float f32x4 __attribute__((ext_vector_type(4)));
 
 template <typename T>
 __global__ void qk_norm_temp_cache_kernel(
@@ -103,8 +106,11 @@ __global__ void qk_norm_temp_cache_kernel(
 // then [v_half] pairs) and shared by every head. Then one wave per head
 // job: jobs 0..heads-1 are q heads, then kv_heads k heads, then kv_heads v
 // heads. x_n[j] = x[j] * inv_rms * w[j]; coordinate i < half pairs with
-// i + half. VEC = 2: a lane owns two neighbouring coordinates (4- and 8-byte
-// accesses); needs even head sizes, halves and row stride.
+// i + half, or with `pairs` 2i with 2i + 1; the qk angles' sines and cosines
+// are multiplied by rot_mult. `maps` k heads share one cached row (map m at
+// columns m D ..). VEC = 2: a lane owns two neighbouring coordinates (4- and
+// 8-byte accesses); needs even head sizes, halves (unless `pairs`) and row
+// stride. TI: dtype of q, k, v (fp32 beside bf16 pages is allowed).
 template <int VEC>
 __device__ __forceinline__ void ld_vec(const short* p, float* v) {
   if (VEC == 2) {
@@ -143,15 +149,16 @@ __device__ __forceinline__ void st_vec(float* p, const float* v) {
     p[0] = v[0];
 }
 
-template <typename T, int VEC>
+template <typename TI, typename T, int VEC>
 __global__ void qk_headnorm_rope_cache_kernel(
-    float* __restrict__ q_out, const T* __restrict__ q, const T* __restrict__ k,
-    const T* __restrict__ v, long row_stride, const float* __restrict__ qw,
+    float* __restrict__ q_out, const TI* __restrict__ q,
+    const TI* __restrict__ k, const TI* __restrict__ v, long row_stride, const float* __restrict__ qw,
     const float* __restrict__ kw, const long* __restrict__ positions,
     const int* __restrict__ slot_mapping, T* __restrict__ k_cache,
     T* __restrict__ v_cache, float eps, int heads, int kv_heads, int D, int DV,
     int block_size, const float* __restrict__ qk_inv_freq, int qk_half,
-    int v_unit_norm, const float* __restrict__ v_inv_freq, int v_half) {
+    int v_unit_norm, const float* __restrict__ v_inv_freq, int v_half,
+    int pairs, float rot_mult, int maps) {
   extern __shared__ float lds[];
   if (!qk_inv_freq) qk_half = 0;
   if (!v_inv_freq) v_half = 0;
@@ -165,16 +172,18 @@ __global__ void qk_headnorm_rope_cache_kernel(
     const float f = i < qk_half ? qk_inv_freq[i] : v_inv_freq[i - qk_half];
     float sn, cs;
     sincosf(pos * f, &sn, &cs);
-    lds[2 * i] = cs;
-    lds[2 * i + 1] = sn;
+    const float m = i < qk_half ? rot_mult : 1.0f;
+    lds[2 * i] = cs * m;
+    lds[2 * i + 1] = sn * m;
   }
   __syncthreads();
   const long slot = slot_mapping[t];
   const long blk = slot >= 0 ? slot / block_size : 0;
   const long off = slot >= 0 ? slot % block_size : 0;
-  const int jobs = heads + 2 * kv_heads;
+  const int k_heads = kv_heads * maps;
+  const int jobs = heads + k_heads + kv_heads;
   for (int job = wave; job < jobs; job += NW) {
-    const T* src;
+    const TI* src;
     const float* w = nullptr;
     const float* cs;
     int width, half;
@@ -188,7 +197,7 @@ __global__ void qk_headnorm_rope_cache_kernel(
       cs = cs_qk;
       half = qk_half;
       dst_f = q_out + (t * heads + job) * D;
-    } else if (job < heads + kv_heads) {
+    } else if (job < heads + k_heads) {
       const int g = job - heads;
       src = k + t * row_stride + (long)g * D;
       w = kw;
@@ -196,9 +205,10 @@ __global__ void qk_headnorm_rope_cache_kernel(
       cs = cs_qk;
       half = qk_half;
       if (slot < 0) continue;
-      dst_c = k_cache + ((blk * kv_heads + g) * block_size + off) * D;
+      dst_c = k_cache +
+              (((blk * kv_heads + g / maps) * block_size + off) * maps + g % maps) * D;
     } else {
-      const int g = job - heads - kv_heads;
+      const int g = job - heads - k_heads;
       src = v + t * row_stride + (long)g * DV;
       width = DV;
       cs = cs_v;
@@ -227,7 +237,19 @@ __global__ void qk_headnorm_rope_cache_kernel(
         if (norm) x[c] = w ? x[c] * inv * w[i + c] : x[c] * inv;
         r[c] = x[c];
       }
-      if (i < 2 * half) {  // i and i + VEC - 1 lie in the same half
+      if (pairs && i < 2 * half) {
+        if (VEC == 2) {
+          const float co = cs[i], sn = cs[i + 1];
+          r[0] = x[0] * co - x[VEC - 1] * sn;
+          r[VEC - 1] = x[VEC - 1] * co + x[0] * sn;
+        } else {
+          float y[VEC];
+          ld_vec<VEC>(src + (i ^ 1), y);
+          if (norm) y[0] = w ? y[0] * inv * w[i ^ 1] : y[0] * inv;
+          const float co = cs[i & ~1], sn = cs[i | 1];
+          r[0] = (i & 1) ? x[0] * co + y[0] * sn : x[0] * co - y[0] * sn;
+        }
+      } else if (i < 2 * half) {  // i and i + VEC - 1 lie in the same half
         const int pi = i < half ? i + half : i - half;  // partner
         const int fi = i < half ? i : i - half;
         float y[VEC];
@@ -244,50 +266,6 @@ __global__ void qk_headnorm_rope_cache_kernel(
     }
   }
 }
-
-// 8 consecutive elements of a cache row, kept in the cache dtype while the
-// load is in flight (a bf16 chunk costs 4 registers) and widened on the way
-// into LDS
-template <typename T>
-struct Chunk8;
-template <>
-struct Chunk8<short> {
-  short8_t x;
-  __device__ __forceinline__ void load(const short* p, bool vec, int valid) {
-    if (vec && valid >= 8) {
-      x = *reinterpret_cast<const short8_t*>(p);
-    } else {
-#pragma unroll
-      for (int i = 0; i < 8; ++i) x[i] = i < valid ? p[i] : (short)0;
-    }
-  }
-  __device__ __forceinline__ void zero() {
-#pragma unroll
-    for (int i = 0; i < 8; ++i) x[i] = 0;
-  }
-  __device__ __forceinline__ float get(int i) const { return bf16_bits_to_float(x[i]); }
-};
-template <>
-struct Chunk8<float> {
-  f32x4 a, b;
-  __device__ __forceinline__ void load(const float* p, bool vec, int valid) {
-    if (vec && valid >= 8) {
-      a = *reinterpret_cast<const f32x4*>(p);
-      b = *reinterpret_cast<const f32x4*>(p + 4);
-    } else {
-#pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        a[i] = i < valid ? p[i] : 0.f;
-        b[i] = 4 + i < valid ? p[4 + i] : 0.f;
-      }
-    }
-  }
-  __device__ __forceinline__ void zero() {
-    a = f32x4{0.f, 0.f, 0.f, 0.f};
-    b = a;
-  }
-  __device__ __forceinline__ float get(int i) const { return i < 4 ? a[i] : b[i - 4]; }
-};
 
 // rows [k0, k0 + nk) of one kv head, WP (padded width) columns: each thread
 // owns WP / 32 chunks of 8; fetch() issues the global loads, store() writes
@@ -356,6 +334,19 @@ __device__ __forceinline__ f32x4 lds4(const short* p) {
                bf16_bits_to_float(x[2]), bf16_bits_to_float(x[3])};
 }
 
+// tanh to fp32 accuracy in absolute terms: 1 - 2 / (exp(2x) + 1)
+__device__ __forceinline__ float tanh_exp2(float x) {
+  const float e = exp2f(x * 2.88539008177792681472f);
+  return 1.0f - 2.0f * __builtin_amdgcn_rcpf(e + 1.0f);
+}
+
+// an output element in the cache dtype, or in fp32
+template <typename T>
+__device__ __forceinline__ void st_out(T* out, long i, float v, int f32) {
+  if (f32) reinterpret_cast<float*>(out)[i] = v;
+  else st_f32(out, i, v);
+}
+
 template <typename T, int DP, int DVP, bool SPLITK, bool VK>
 __global__ void __launch_bounds__(NT) ctx_attention_f32_kernel(
     T* __restrict__ out, const float* __restrict__ q,
@@ -366,7 +357,9 @@ __global__ void __launch_bounds__(NT) ctx_attention_f32_kernel(
     int kv_heads, int D, int DV, int block_size, int hpb,
     const float* __restrict__ sink, int chunk,
     const float* __restrict__ out_inv_freq, int window, long v_row_stride,
-    float* __restrict__ ws) {
+    float* __restrict__ ws, int maps, float softcap, int out_f32) {
+  // D: columns of a key row this launch reads per query (decode: all maps of
+  // a row; prefill: one map, at columns (head % maps) D of rows of maps * D)
   extern __shared__ float lds[];
   constexpr int KS = DP + 4;   // K row stride: lanes of one MFMA read hit 64 banks
   // V row stride: likewise for the 4-key-apart rows. VK: the values are the
@@ -443,7 +436,10 @@ __global__ void __launch_bounds__(NT) ctx_attention_f32_kernel(
   // the last row), where the K tile is staged afterwards: a lane's own
   // values are 64 floats apart from its neighbour's, which global memory
   // serves badly.
-  const float qscale = scale * 1.44269504088896340736f;
+  const float qscale =
+      softcap > 0.f ? scale / softcap : scale * 1.44269504088896340736f;
+  const float capl = softcap * 1.44269504088896340736f;
+  const int dq = SPLITK ? D / maps : D;  // columns of a query
   float qf[DP / 4];
   {
     float* Qs = lds;  // [ROWS][KS] floats
@@ -451,14 +447,15 @@ __global__ void __launch_bounds__(NT) ctx_attention_f32_kernel(
       const int rr = e / (DP / 4), d = (e % (DP / 4)) * 4;
       f32x4 v = f32x4{0.f, 0.f, 0.f, 0.f};
       if (rr < nrows) {
-        const float* src =
-            q + ((long)(q0 + tok0 + rr / hpb) * heads + head0 + rr % hpb) * D;
-        if ((D % 4) == 0 && d + 3 < D) {
-          v = *reinterpret_cast<const f32x4*>(src + d);
+        const int h2 = head0 + rr % hpb;
+        const float* src = q + ((long)(q0 + tok0 + rr / hpb) * heads + h2) * dq;
+        const int d1 = SPLITK ? d - (h2 % maps) * dq : d;
+        if ((dq % 4) == 0) {
+          if (d1 >= 0 && d1 < dq) v = *reinterpret_cast<const f32x4*>(src + d1);
         } else {
 #pragma unroll
           for (int c = 0; c < 4; ++c)
-            if (d + c < D) v[c] = src[d + c];
+            if (d1 + c >= 0 && d1 + c < dq) v[c] = src[d1 + c];
         }
       }
       *reinterpret_cast<f32x4*>(Qs + rr * KS + d) = v * qscale;
@@ -479,6 +476,8 @@ __global__ void __launch_bounds__(NT) ctx_attention_f32_kernel(
   float m = -INFINITY, l = 0.f;
 
   const int* bt = block_tables + (long)s * bt_stride;
+  const long k_row_stride = SPLITK ? D : (long)maps * D;
+  const T* kc = SPLITK ? k_cache : k_cache + (head0 % maps) * D;
   const bool kvec = (D % 8) == 0;
   const bool vvec = (DV % 8) == 0 && (v_row_stride % 8) == 0 &&
                     ((uintptr_t)v_cache % 32) == 0;
@@ -490,7 +489,7 @@ __global__ void __launch_bounds__(NT) ctx_attention_f32_kernel(
   TileStage<T, DP> kst;
   TileStage<T, DVP> vst;
   const int kfirst = kbeg + split * BK;
-  kst.fetch(k_cache, bt, kfirst, min(BK, last_pos + 1 - kfirst), g, kv_heads, D, D, block_size, bs_shift, kvec);
+  kst.fetch(kc, bt, kfirst, min(BK, last_pos + 1 - kfirst), g, kv_heads, D, k_row_stride, block_size, bs_shift, kvec);
   if (!VK)
     vst.fetch(v_cache, bt, kfirst, min(BK, last_pos + 1 - kfirst), g, kv_heads, DV, v_row_stride, block_size, bs_shift, vvec);
   for (int k0 = kfirst; k0 <= last_pos; k0 += kstep) {
@@ -500,7 +499,7 @@ __global__ void __launch_bounds__(NT) ctx_attention_f32_kernel(
     __syncthreads();
     if (k0 + kstep <= last_pos) {
       const int nn = min(BK, last_pos + 1 - (k0 + kstep));
-      kst.fetch(k_cache, bt, k0 + kstep, nn, g, kv_heads, D, D, block_size, bs_shift, kvec);
+      kst.fetch(kc, bt, k0 + kstep, nn, g, kv_heads, D, k_row_stride, block_size, bs_shift, kvec);
       if (!VK)
         vst.fetch(v_cache, bt, k0 + kstep, nn, g, kv_heads, DV, v_row_stride, block_size, bs_shift, vvec);
     }
@@ -529,6 +528,12 @@ __global__ void __launch_bounds__(NT) ctx_attention_f32_kernel(
     }
 #pragma unroll
     for (int t = 0; t < KT; ++t) sc[t] += sc2[t];
+    if (softcap > 0.f) {
+#pragma unroll
+      for (int t = 0; t < KT; ++t)
+#pragma unroll
+        for (int v = 0; v < 4; ++v) sc[t][v] = capl * tanh_exp2(sc[t][v]);
+    }
     float mt = -INFINITY;
 #pragma unroll
     for (int t = 0; t < KT; ++t) {
@@ -670,10 +675,10 @@ __global__ void __launch_bounds__(NT) ctx_attention_f32_kernel(
           O2 *= f;
           float sn, cs;
           sincosf((float)(base_pos + row / hpb) * out_inv_freq[dv], &sn, &cs);
-          st_f32(out, ((long)tk * heads + h2) * DV + dv, O * cs + O2 * sn);
-          st_f32(out, ((long)tk * heads + h2) * DV + dv + ohalf, O2 * cs - O * sn);
+          st_out(out, ((long)tk * heads + h2) * DV + dv, O * cs + O2 * sn, out_f32);
+          st_out(out, ((long)tk * heads + h2) * DV + dv + ohalf, O2 * cs - O * sn, out_f32);
         } else {
-          st_f32(out, ((long)tk * heads + h2) * DV + dv, O);
+          st_out(out, ((long)tk * heads + h2) * DV + dv, O, out_f32);
         }
       }
     }
@@ -713,8 +718,8 @@ __global__ void __launch_bounds__(NT) ctx_attention_f32_kernel(
       const float a = Os[row * OS + dv], b = Os[row * OS + dv + ohalf];
       float sn, cs;
       sincosf((float)(base_pos + row / hpb) * out_inv_freq[dv], &sn, &cs);
-      st_f32(out, ((long)tk * heads + h2) * DV + dv, a * cs + b * sn);
-      st_f32(out, ((long)tk * heads + h2) * DV + dv + ohalf, b * cs - a * sn);
+      st_out(out, ((long)tk * heads + h2) * DV + dv, a * cs + b * sn, out_f32);
+      st_out(out, ((long)tk * heads + h2) * DV + dv + ohalf, b * cs - a * sn, out_f32);
     }
     return;
   }
@@ -724,7 +729,7 @@ __global__ void __launch_bounds__(NT) ctx_attention_f32_kernel(
 #pragma unroll
     for (int v = 0; v < 4; ++v) {
       const int dv = 64 * (i / 4) + 4 * (4 * lg + v) + i % 4;
-      if (dv < DV) st_f32(out, ((long)tok * heads + hd) * DV + dv, o[i][v] * f);
+      if (dv < DV) st_out(out, ((long)tok * heads + hd) * DV + dv, o[i][v] * f, out_f32);
     }
 }
 
@@ -734,7 +739,7 @@ template <typename T>
 __global__ void ctx_attention_merge_kernel(
     T* __restrict__ out, const float* __restrict__ ws,
     const int* __restrict__ cu_q, const T* __restrict__ gate, long gate_stride,
-    const float* __restrict__ sink, int heads, int DV, int nsplit) {
+    const float* __restrict__ sink, int heads, int DV, int nsplit, int out_f32) {
   const int s = blockIdx.x / heads, h = blockIdx.x % heads;
   const int tok = cu_q[s];
   if (cu_q[s + 1] - tok < 1) return;
@@ -762,7 +767,7 @@ __global__ void ctx_attention_merge_kernel(
       const float mi = wr[i * (DV + 2) + DV];
       if (mi != -INFINITY) O += wr[i * (DV + 2) + dv] * exp2f(mi - M);
     }
-    st_f32(out, ((long)tok * heads + h) * DV + dv, O * f);
+    st_out(out, ((long)tok * heads + h) * DV + dv, O * f, out_f32);
   }
 }
 
@@ -801,37 +806,40 @@ extern "C" hipError_t ks_qk_headnorm_rope_cache(
     const void* slot_mapping, void* k_cache, void* v_cache, float eps,
     int tokens, int heads, int kv_heads, int D, int DV, int block_size,
     const void* qk_inv_freq, int qk_half, int v_unit_norm,
-    const void* v_inv_freq, int v_half, int is_f32, hipStream_t stream) {
+    const void* v_inv_freq, int v_half, int pairs, float rot_mult, int maps,
+    int in_f32, int is_f32, hipStream_t stream) {
   if (tokens == 0) return hipSuccess;
-  if (2 * qk_half > D || 2 * v_half > DV) return hipErrorInvalidValue;
-#define HN_ARGS(TT)                                                          \
-  (float*)q_out, (const TT*)q, (const TT*)k, (const TT*)v, row_stride,       \
+  if (2 * qk_half > D || 2 * v_half > DV || maps < 1 ||
+      (pairs && v_inv_freq) || (is_f32 && !in_f32))
+    return hipErrorInvalidValue;
+#define HN_ARGS(TI, TT)                                                      \
+  (float*)q_out, (const TI*)q, (const TI*)k, (const TI*)v, row_stride,       \
       (const float*)qw, (const float*)kw, (const long*)positions,            \
       (const int*)slot_mapping, (TT*)k_cache, (TT*)v_cache, eps, heads,      \
       kv_heads, D, DV, block_size, (const float*)qk_inv_freq, qk_half,       \
-      v_unit_norm, (const float*)v_inv_freq, v_half
+      v_unit_norm, (const float*)v_inv_freq, v_half, pairs, rot_mult, maps
+#define HN_LAUNCH(TI, TT)                                                    \
+  do {                                                                       \
+    if (vec)                                                                 \
+      hipLaunchKernelGGL((qk_headnorm_rope_cache_kernel<TI, TT, 2>),         \
+                         dim3(tokens), dim3(NT), smem, stream,               \
+                         HN_ARGS(TI, TT));                                   \
+    else                                                                     \
+      hipLaunchKernelGGL((qk_headnorm_rope_cache_kernel<TI, TT, 1>),         \
+                         dim3(tokens), dim3(NT), smem, stream,               \
+                         HN_ARGS(TI, TT));                                   \
+  } while (0)
   const size_t smem = sizeof(float) * 2 * (size_t)(qk_half + v_half);
-  const int esz = is_f32 ? 4 : 2;
-  auto al = [&](const void* p) { return ((uintptr_t)p % (2 * esz)) == 0; };
-  const bool vec = D % 2 == 0 && DV % 2 == 0 && qk_half % 2 == 0 &&
-                   v_half % 2 == 0 && row_stride % 2 == 0 && al(q) && al(k) &&
-                   al(v) && al(k_cache) && al(v_cache) &&
-                   ((uintptr_t)q_out % 8) == 0;
-  if (is_f32) {
-    if (vec)
-      hipLaunchKernelGGL((qk_headnorm_rope_cache_kernel<float, 2>), dim3(tokens),
-                         dim3(NT), smem, stream, HN_ARGS(float));
-    else
-      hipLaunchKernelGGL((qk_headnorm_rope_cache_kernel<float, 1>), dim3(tokens),
-                         dim3(NT), smem, stream, HN_ARGS(float));
-  } else {
-    if (vec)
-      hipLaunchKernelGGL((qk_headnorm_rope_cache_kernel<short, 2>), dim3(tokens),
-                         dim3(NT), smem, stream, HN_ARGS(short));
-    else
-      hipLaunchKernelGGL((qk_headnorm_rope_cache_kernel<short, 1>), dim3(tokens),
-                         dim3(NT), smem, stream, HN_ARGS(short));
-  }
+  auto al = [](const void* p, int f32) {
+    return ((uintptr_t)p % (f32 ? 8 : 4)) == 0;
+  };
+  const bool vec = D % 2 == 0 && DV % 2 == 0 && (pairs || qk_half % 2 == 0) &&
+                   v_half % 2 == 0 && row_stride % 2 == 0 && al(q, in_f32) &&
+                   al(k, in_f32) && al(v, in_f32) && al(k_cache, is_f32) &&
+                   al(v_cache, is_f32) && ((uintptr_t)q_out % 8) == 0;
+  if (is_f32) HN_LAUNCH(float, float);
+  else if (in_f32) HN_LAUNCH(float, short);
+  else HN_LAUNCH(short, short);
   HIP_CHECK_KERNEL();
   return hipSuccess;
 }
@@ -877,6 +885,10 @@ struct CtxArgs {
   void* ws;
   int nsplit;
   hipStream_t stream;
+  int maps;
+  float softcap;
+  int out_f32;
+  bool decode;  // one token per sequence, in the split-key form
 };
 
 template <typename T, int DP, int DVP, bool VK>
@@ -884,7 +896,7 @@ hipError_t launch_ctx_attention(const CtxArgs& a) {
   // the staged tiles are fp32 in prefill and in the cache dtype in decode;
   // the other uses of the same LDS (query rows; decode: cross-wave merge;
   // prefill: rows to turn back) are fp32
-  const bool decode = a.max_q_len == 1;
+  const bool decode = a.decode;
   size_t smem = (decode ? sizeof(T) : sizeof(float)) * (size_t)BK *
                 (DP + 4 + (VK ? 0 : DVP + 4));
   int hpb = 1;
@@ -918,21 +930,22 @@ hipError_t launch_ctx_attention(const CtxArgs& a) {
                      a.kv_heads, a.D, a.DV, a.block_size, hpb,
                      (const float*)a.sink, a.chunk,
                      (const float*)a.out_inv_freq, a.window, a.v_row_stride,
-                     (float*)a.ws);
+                     (float*)a.ws, a.maps, a.softcap, a.out_f32);
   hipError_t e = hipGetLastError();
   if (e != hipSuccess || nsplit <= 1) return e;
   hipLaunchKernelGGL(ctx_attention_merge_kernel<T>,
                      dim3(a.num_seqs * a.heads), dim3(64), 0, a.stream,
                      (T*)a.out, (const float*)a.ws, (const int*)a.cu_q,
                      (const T*)a.gate, a.gate_stride, (const float*)a.sink,
-                     a.heads, a.DV, nsplit);
+                     a.heads, a.DV, nsplit, a.out_f32);
   return hipGetLastError();
 }
 
 template <typename T, int DP, int DVP>
 hipError_t dispatch_vk(const CtxArgs& a) {
   // the values are the leading columns of the key rows themselves
-  const bool vk = a.v_cache == a.k_cache && a.v_row_stride == a.D && DVP <= DP;
+  const bool vk = a.v_cache == a.k_cache && a.v_row_stride == a.D && DVP <= DP &&
+                  a.maps == 1;
   if constexpr (DVP <= DP) {
     if (vk) return launch_ctx_attention<T, DP, DVP, true>(a);
   }
@@ -961,8 +974,15 @@ extern "C" hipError_t ks_ctx_attention_f32(
     int num_seqs, int max_q_len, int heads, int kv_heads, int D, int DV,
     int block_size, int is_f32, const void* sink, int chunk,
     const void* out_inv_freq, int window, long v_row_stride, void* ws,
-    int nsplit, hipStream_t stream) {
+    int nsplit, int maps, float softcap, int out_f32, hipStream_t stream) {
   if (num_seqs == 0 || max_q_len == 0) return hipSuccess;
+  // D: columns of one key (a cached row holds maps of them)
+  if (maps < 1 || heads % (kv_heads > 0 ? kv_heads * maps : 1) != 0)
+    return hipErrorInvalidValue;
+  // rows too wide for the split-key form take the prefill form
+  const bool decode = max_q_len == 1 && maps * D <= 256;
+  if (decode) D *= maps;
+  else if (maps > 1) nsplit = 1;
   if (D < 1 || D > 256 || DV < 1 || DV > 256 || kv_heads < 1 ||
       heads % kv_heads != 0 || chunk < 0 || window < 0 ||
       (chunk > 0 && window > 0) || v_row_stride < DV ||
@@ -972,6 +992,7 @@ extern "C" hipError_t ks_ctx_attention_f32(
   const CtxArgs a{out, q, k_cache, v_cache, block_tables, bt_stride, cu_q,
                   ctx_lens, gate, gate_stride, scale, num_seqs, max_q_len,
                   heads, kv_heads, D, DV, block_size, sink, chunk,
-                  out_inv_freq, window, v_row_stride, ws, nsplit, stream};
+                  out_inv_freq, window, v_row_stride, ws, nsplit, stream,
+                  maps, softcap, out_f32, decode};
   return is_f32 ? dispatch_d<float>(a) : dispatch_d<short>(a);
 }

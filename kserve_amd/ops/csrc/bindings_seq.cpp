@@ -13,11 +13,11 @@ hipError_t ks_add_rms_norm_f32res(void*, const void*, long, float, const void*,
                                   void*, int, int, int, int, hipStream_t);
 hipError_t ks_gated_group_rms_norm(void*, const void*, const void*, long,
                                    const void*, int, float, int, int, int, int,
-                                   int, hipStream_t);
+                                   int, int, hipStream_t);
 hipError_t ks_causal_conv_silu(void*, const void*, long, const void*,
                                const void*, void*, const void*, const void*,
                                const void*, const void*, int, int, int, int,
-                               int, hipStream_t);
+                               int, int, hipStream_t);
 hipError_t ks_ssd_scan(void*, const void*, const void*, long, int, const void*,
                        const void*, const void*, void*, const void*,
                        const void*, const void*, int, int, int, int, int,
@@ -31,15 +31,16 @@ hipError_t ks_ctx_attention_f32(void*, const void*, const void*, const void*,
                                 const void*, int, const void*, const void*,
                                 const void*, long, float, int, int, int, int,
                                 int, int, int, int, const void*, int,
-                                const void*, int, long, void*, int,
-                                hipStream_t);
+                                const void*, int, long, void*, int, int, float,
+                                int, hipStream_t);
 int ks_ctx_attention_decode_splits(int, int, int, int, int);
 hipError_t ks_qk_headnorm_rope_cache(void*, const void*, const void*,
                                      const void*, long, const void*,
                                      const void*, const void*, const void*,
                                      void*, void*, float, int, int, int, int,
                                      int, int, const void*, int, int,
-                                     const void*, int, int, hipStream_t);
+                                     const void*, int, int, float, int, int,
+                                     int, hipStream_t);
 hipError_t ks_post_norm_add_rms_norm(void*, const void*, long, int, float,
                                      const void*, const void*, const void*,
                                      float, float, void*, int, int, int,
@@ -82,8 +83,26 @@ hipError_t ks_unit_norm_heads(void*, long, int, int, float, int, float, int,
 hipError_t ks_linear_scan(void*, const void*, long, const void*, long,
                           const void*, long, const void*, const void*,
                           const void*, long, int, const void*, const void*,
-                          void*, const void*, const void*, const void*, int,
-                          int, int, int, int, hipStream_t);
+                          const void*, void*, const void*, const void*,
+                          const void*, int, int, int, int, int, hipStream_t);
+hipError_t ks_delta_unit_decay(void*, long, void*, const void*, long,
+                               const void*, const void*, int, int, int, float,
+                               float, int, int, hipStream_t);
+hipError_t ks_post_group_norm_add(void*, const void*, long, const void*, long,
+                                  int, const void*, const void*, const void*,
+                                  int, float, void*, int, const void*, int, int,
+                                  hipStream_t);
+hipError_t ks_diff_combine(void*, const void*, const void*, int, int, int,
+                           float, float, int, hipStream_t);
+hipError_t ks_talk_prep_cache(void*, const void*, long, const void*, long,
+                              const void*, const void*, void*, void*, float,
+                              int, int, int, int, int, int, hipStream_t);
+int ks_talk_decode_splits(int, int);
+hipError_t ks_talk_attention(void*, const void*, const void*, const void*,
+                             const void*, int, const void*, const void*,
+                             const void*, const void*, int, const void*, long,
+                             float, int, int, int, int, int, int, int, int,
+                             void*, int, hipStream_t);
 }
 
 namespace {
@@ -184,7 +203,8 @@ void add_rms_norm_f32res(at::Tensor& residual,
 
 void gated_group_rms_norm(at::Tensor& out, at::Tensor& y, at::Tensor& z,
                           const c10::optional<at::Tensor>& weight_opt,
-                          double eps, int64_t groups, bool gate_after) {
+                          double eps, int64_t groups, bool gate_after,
+                          bool gate_sigmoid) {
   CHECK_F32(y);
   const void* wp = nullptr;
   int64_t wn = y.size(1);
@@ -205,7 +225,7 @@ void gated_group_rms_norm(at::Tensor& out, at::Tensor& y, at::Tensor& z,
   check_hip(ks_gated_group_rms_norm(out.data_ptr(), y.data_ptr(), z.data_ptr(),
                                     z.stride(0), wp, (int)wn, (float)eps, rows,
                                     inner, (int)groups, gate_after ? 1 : 0,
-                                    f32, current_stream()),
+                                    gate_sigmoid ? 1 : 0, f32, current_stream()),
             "gated_group_rms_norm");
 }
 
@@ -213,7 +233,7 @@ void causal_conv_silu(at::Tensor& out, at::Tensor& in, at::Tensor& w,
                       const c10::optional<at::Tensor>& bias_opt,
                       at::Tensor& conv_state,
                       at::Tensor& positions, at::Tensor& seq_of_token,
-                      at::Tensor& cu_seqlens, at::Tensor& slots) {
+                      at::Tensor& cu_seqlens, at::Tensor& slots, bool silu) {
   CHECK_F32(out);
   CHECK_F32(w);
   const void* bias_ptr = nullptr;
@@ -246,7 +266,7 @@ void causal_conv_silu(at::Tensor& out, at::Tensor& in, at::Tensor& w,
                                 conv_state.data_ptr(), positions.data_ptr(),
                                 seq_of_token.data_ptr(), cu_seqlens.data_ptr(),
                                 slots.data_ptr(), tokens, num_seqs, channels,
-                                taps, f32, current_stream()),
+                                taps, silu ? 1 : 0, f32, current_stream()),
             "causal_conv_silu");
 }
 
@@ -335,7 +355,7 @@ void ctx_attention_f32(at::Tensor& out, at::Tensor& q, at::Tensor& k_cache,
                        int64_t max_q_len, int64_t heads,
                        const c10::optional<at::Tensor>& sink, int64_t chunk,
                        const c10::optional<at::Tensor>& out_inv_freq,
-                       int64_t window) {
+                       int64_t window, int64_t maps, double softcap) {
   CHECK_F32(q);
   CHECK_I32(cu_q);
   CHECK_I32(ctx_lens);
@@ -345,8 +365,14 @@ void ctx_attention_f32(at::Tensor& out, at::Tensor& q, at::Tensor& k_cache,
   TORCH_CHECK(k_cache.dim() == 4 && v_cache.dim() == 4 &&
                   k_cache.is_contiguous() && out.is_contiguous(),
               "caches [blocks, kv_heads, block, dim]");
-  const int f32 = act_is_f32(out, "out");
-  const int G = k_cache.size(1), bs = k_cache.size(2), D = k_cache.size(3);
+  // the output may be fp32 beside bf16 pages
+  const int out_f32 = act_is_f32(out, "out");
+  const int f32 = act_is_f32(k_cache, "k_cache");
+  const int G = k_cache.size(1), bs = k_cache.size(2);
+  TORCH_CHECK(maps >= 1 && k_cache.size(3) % maps == 0 &&
+                  heads % (G * maps) == 0 && (out_f32 || !f32) && softcap >= 0,
+              "ctx_attention_f32: heads / key maps / output dtype");
+  const int D = k_cache.size(3) / maps;
   const int DV = v_cache.size(3);
   // the values may be a column range of wider rows (a view of the key pool)
   const int64_t vrs = v_cache.stride(2);
@@ -356,8 +382,7 @@ void ctx_attention_f32(at::Tensor& out, at::Tensor& q, at::Tensor& k_cache,
               "v_cache: dense pages of rows with one common stride");
   const int num_seqs = ctx_lens.numel();
   const int64_t tokens = q.numel() / (heads * D);
-  TORCH_CHECK(act_is_f32(k_cache, "k_cache") == f32 &&
-                  act_is_f32(v_cache, "v_cache") == f32 &&
+  TORCH_CHECK(act_is_f32(v_cache, "v_cache") == f32 &&
                   q.numel() == tokens * heads * D &&
                   out.numel() == tokens * heads * DV &&
                   cu_q.numel() == num_seqs + 1 &&
@@ -392,7 +417,7 @@ void ctx_attention_f32(at::Tensor& out, at::Tensor& q, at::Tensor& k_cache,
   // leave partial results in a scratch tensor for a merge pass
   int nsplit = 1;
   at::Tensor ws;
-  if (max_q_len == 1) {
+  if (max_q_len == 1 && maps * D <= 256) {
     nsplit = ks_ctx_attention_decode_splits(num_seqs, (int)heads, G,
                                             (int)window, fp != nullptr);
     if (nsplit > 1)
@@ -406,8 +431,8 @@ void ctx_attention_f32(at::Tensor& out, at::Tensor& q, at::Tensor& k_cache,
                 ctx_lens.data_ptr(), gp, gst, (float)scale, num_seqs,
                 (int)max_q_len, (int)heads, G, D, DV, bs, f32, sp, (int)chunk,
                 fp, (int)window, (long)vrs,
-                nsplit > 1 ? ws.data_ptr() : nullptr, nsplit,
-                current_stream()),
+                nsplit > 1 ? ws.data_ptr() : nullptr, nsplit, (int)maps,
+                (float)softcap, out_f32, current_stream()),
             "ctx_attention_f32");
 }
 
@@ -420,18 +445,23 @@ void qk_headnorm_rope_cache(at::Tensor& q_out, at::Tensor& q, at::Tensor& k,
                             double eps, int64_t heads,
                             const c10::optional<at::Tensor>& qk_inv_freq,
                             bool v_unit_norm,
-                            const c10::optional<at::Tensor>& v_inv_freq) {
+                            const c10::optional<at::Tensor>& v_inv_freq,
+                            bool pairs, double rot_mult, int64_t maps) {
   CHECK_F32(q_out);
+  TORCH_CHECK(maps >= 1 && k_cache.size(3) % maps == 0 &&
+                  !(pairs && v_inv_freq.has_value()),
+              "qk_headnorm_rope_cache: key maps / rotation");
+  const int D = k_cache.size(3) / maps;
   // without weights the norm is plain x / rms(x)
   const void *qwp = nullptr, *kwp = nullptr;
   if (qw_opt.has_value()) {
     CHECK_F32(*qw_opt);
-    TORCH_CHECK(qw_opt->numel() == k_cache.size(3), "qw [dim]");
+    TORCH_CHECK(qw_opt->numel() == D, "qw [dim]");
     qwp = qw_opt->data_ptr();
   }
   if (kw_opt.has_value()) {
     CHECK_F32(*kw_opt);
-    TORCH_CHECK(kw_opt->numel() == k_cache.size(3), "kw [dim]");
+    TORCH_CHECK(kw_opt->numel() == D, "kw [dim]");
     kwp = kw_opt->data_ptr();
   }
   CHECK_ROWS(q);
@@ -442,15 +472,16 @@ void qk_headnorm_rope_cache(at::Tensor& q_out, at::Tensor& q, at::Tensor& k,
   TORCH_CHECK(k_cache.dim() == 4 && v_cache.dim() == 4 &&
                   k_cache.is_contiguous() && v_cache.is_contiguous(),
               "caches [blocks, kv_heads, block, dim]");
-  const int f32 = act_is_f32(q, "q");
+  // inputs in the cache dtype, or fp32 beside bf16 pages
+  const int in_f32 = act_is_f32(q, "q");
+  const int f32 = act_is_f32(k_cache, "k_cache");
   const int tokens = q.size(0);
-  const int G = k_cache.size(1), bs = k_cache.size(2), D = k_cache.size(3);
+  const int G = k_cache.size(1), bs = k_cache.size(2);
   const int DV = v_cache.size(3);
-  TORCH_CHECK(act_is_f32(k, "k") == f32 && act_is_f32(v, "v") == f32 &&
-                  act_is_f32(k_cache, "k_cache") == f32 &&
-                  act_is_f32(v_cache, "v_cache") == f32,
+  TORCH_CHECK(act_is_f32(k, "k") == in_f32 && act_is_f32(v, "v") == in_f32 &&
+                  act_is_f32(v_cache, "v_cache") == f32 && (in_f32 || !f32),
               "qk_headnorm_rope_cache: dtype mismatch");
-  TORCH_CHECK(q.size(1) == heads * D && k.size(1) == G * D &&
+  TORCH_CHECK(q.size(1) == heads * D && k.size(1) == G * maps * D &&
                   v.size(1) == G * DV && k.size(0) == tokens &&
                   v.size(0) == tokens && q.stride(0) == k.stride(0) &&
                   q.stride(0) == v.stride(0) && v_cache.size(1) == G &&
@@ -478,7 +509,8 @@ void qk_headnorm_rope_cache(at::Tensor& q_out, at::Tensor& q, at::Tensor& k,
                 positions.data_ptr(), slot_mapping.data_ptr(),
                 k_cache.data_ptr(), v_cache.data_ptr(), (float)eps, tokens,
                 (int)heads, G, D, DV, bs, qf, qh, v_unit_norm ? 1 : 0, vf, vh,
-                f32, current_stream()),
+                pairs ? 1 : 0, (float)rot_mult, (int)maps, in_f32, f32,
+                current_stream()),
             "qk_headnorm_rope_cache");
 }
 
@@ -910,8 +942,9 @@ void linear_scan(at::Tensor& o, at::Tensor& q, at::Tensor& k, at::Tensor& v,
                  const c10::optional<at::Tensor>& a_raw,
                  const c10::optional<at::Tensor>& b_raw,
                  const c10::optional<at::Tensor>& a_log,
-                 const c10::optional<at::Tensor>& dt_bias, at::Tensor& state,
-                 at::Tensor& positions, at::Tensor& cu_seqlens,
+                 const c10::optional<at::Tensor>& dt_bias,
+                 const c10::optional<at::Tensor>& channel_decay,
+                 at::Tensor& state, at::Tensor& positions, at::Tensor& cu_seqlens,
                  at::Tensor& slots, int64_t qk_heads) {
   CHECK_F32(o);
   CHECK_F32(state);
@@ -937,13 +970,25 @@ void linear_scan(at::Tensor& o, at::Tensor& q, at::Tensor& k, at::Tensor& v,
                   cu_seqlens.numel() == num_seqs + 1,
               "linear_scan: shape mismatch");
   const void *dp = nullptr, *ap = nullptr, *bp = nullptr, *alp = nullptr,
-             *dtp = nullptr;
+             *dtp = nullptr, *cdp = nullptr;
   long ab_stride = 0;
   int ab_f32 = 1;
   if (decay.has_value()) {
     CHECK_F32(*decay);
     TORCH_CHECK(decay->numel() == heads, "decay [heads]");
     dp = decay->data_ptr();
+  } else if (channel_decay.has_value()) {
+    CHECK_F32(*channel_decay);
+    TORCH_CHECK(b_raw.has_value() &&
+                    channel_decay->numel() == (int64_t)tokens * heads * K,
+                "the channel-decay form needs decays [T, heads*K] and b_raw");
+    CHECK_ROWS(*b_raw);
+    ab_f32 = act_is_f32(*b_raw, "b_raw");
+    TORCH_CHECK(b_raw->size(0) == tokens && b_raw->size(1) == heads,
+                "b_raw [T, heads]");
+    bp = b_raw->data_ptr();
+    ab_stride = b_raw->stride(0);
+    cdp = channel_decay->data_ptr();
   } else {
     TORCH_CHECK(a_raw.has_value() && b_raw.has_value() && a_log.has_value() &&
                     dt_bias.has_value(),
@@ -967,11 +1012,197 @@ void linear_scan(at::Tensor& o, at::Tensor& q, at::Tensor& k, at::Tensor& v,
   }
   check_hip(ks_linear_scan(o.data_ptr(), q.data_ptr(), q.stride(0),
                            k.data_ptr(), k.stride(0), v.data_ptr(),
-                           v.stride(0), dp, ap, bp, ab_stride, ab_f32, alp, dtp,
+                           v.stride(0), dp, ap, bp, ab_stride, ab_f32, alp, dtp, cdp,
                            state.data_ptr(), positions.data_ptr(),
                            cu_seqlens.data_ptr(), slots.data_ptr(), num_seqs,
                            heads, (int)qk_heads, V, K, current_stream()),
             "linear_scan");
+}
+
+void delta_unit_decay(at::Tensor& x, at::Tensor& g, at::Tensor& a_raw,
+                      at::Tensor& a_log, at::Tensor& dt_bias, int64_t qk_heads,
+                      int64_t dim, double q_scale, double eps) {
+  TORCH_CHECK(x.is_cuda() && x.scalar_type() == at::kFloat, "x must be fp32");
+  CHECK_ROWS(x);
+  CHECK_ROWS(a_raw);
+  CHECK_F32(g);
+  CHECK_F32(a_log);
+  CHECK_F32(dt_bias);
+  const int f32 = act_is_f32(a_raw, "a_raw");
+  const int64_t decays = a_raw.size(1);
+  TORCH_CHECK(qk_heads > 0 && dim > 0 && 2 * qk_heads * dim <= x.size(1) &&
+                  a_raw.size(0) == x.size(0) && dt_bias.numel() == decays &&
+                  a_log.numel() * dim == decays &&
+                  g.numel() == x.size(0) * decays,
+              "delta_unit_decay: shape mismatch");
+  check_hip(ks_delta_unit_decay(x.data_ptr(), x.stride(0), g.data_ptr(),
+                                a_raw.data_ptr(), a_raw.stride(0),
+                                a_log.data_ptr(), dt_bias.data_ptr(),
+                                (int)x.size(0), (int)qk_heads, (int)dim,
+                                (float)q_scale, (float)eps, (int)decays, f32,
+                                current_stream()),
+            "delta_unit_decay");
+}
+
+void post_group_norm_add(at::Tensor& residual,
+                         const c10::optional<at::Tensor>& delta,
+                         const c10::optional<at::Tensor>& weight,
+                         const c10::optional<at::Tensor>& delta2,
+                         const c10::optional<at::Tensor>& pre_w,
+                         const c10::optional<at::Tensor>& pre_w2,
+                         int64_t groups, double eps,
+                         const c10::optional<at::Tensor>& out,
+                         const c10::optional<at::Tensor>& next_weight) {
+  CHECK_F32(residual);
+  TORCH_CHECK(residual.dim() == 2, "residual [T, W]");
+  const int rows = residual.size(0), width = residual.size(1);
+  TORCH_CHECK(groups > 0 && width % groups == 0, "groups must divide the width");
+  auto vec = [&](const c10::optional<at::Tensor>& t) -> const void* {
+    if (!t.has_value()) return nullptr;
+    CHECK_F32(*t);
+    TORCH_CHECK(t->numel() == width, "norm weights [W]");
+    return t->data_ptr();
+  };
+  const void *d0 = nullptr, *d1 = nullptr;
+  long s0 = 0, s1 = 0;
+  int df32 = 0;
+  if (delta.has_value()) {
+    CHECK_ROWS(*delta);
+    df32 = act_is_f32(*delta, "delta");
+    TORCH_CHECK(delta->size(0) == rows && delta->size(1) == width &&
+                    weight.has_value(),
+                "delta [T, W] with a weight");
+    d0 = delta->data_ptr();
+    s0 = delta->stride(0);
+    if (delta2.has_value()) {
+      CHECK_ROWS(*delta2);
+      TORCH_CHECK(act_is_f32(*delta2, "delta2") == df32 &&
+                      delta2->size(0) == rows && delta2->size(1) == width &&
+                      pre_w.has_value() && pre_w2.has_value(),
+                  "delta2 [T, W] with both weights");
+      d1 = delta2->data_ptr();
+      s1 = delta2->stride(0);
+    }
+  }
+  void* op = nullptr;
+  int of32 = 1;
+  if (out.has_value()) {
+    of32 = act_is_f32(*out, "out");
+    TORCH_CHECK(out->is_contiguous() && out->numel() == residual.numel(),
+                "out [T, W]");
+    op = out->data_ptr();
+  }
+  check_hip(ks_post_group_norm_add(residual.data_ptr(), d0, s0, d1, s1, df32,
+                                   vec(weight), vec(pre_w), vec(pre_w2),
+                                   (int)groups, (float)eps, op, of32,
+                                   vec(next_weight), rows, width,
+                                   current_stream()),
+            "post_group_norm_add");
+}
+
+void diff_combine(at::Tensor& out, at::Tensor& o, at::Tensor& lam,
+                  int64_t heads, double eps, double mult) {
+  CHECK_F32(o);
+  CHECK_F32(lam);
+  const int f32 = act_is_f32(out, "out");
+  TORCH_CHECK(o.dim() == 2 && heads > 0 && o.size(1) % (2 * heads) == 0 &&
+                  out.is_contiguous() && out.numel() * 2 == o.numel() &&
+                  lam.numel() == 1,
+              "diff_combine: shape mismatch");
+  check_hip(ks_diff_combine(out.data_ptr(), o.data_ptr(), lam.data_ptr(),
+                            (int)o.size(0), (int)heads,
+                            (int)(o.size(1) / (2 * heads)), (float)eps,
+                            (float)mult, f32, current_stream()),
+            "diff_combine");
+}
+
+void talk_prep_cache(at::Tensor& q_out, at::Tensor& q, at::Tensor& k,
+                     at::Tensor& w, at::Tensor& slot_mapping,
+                     at::Tensor& k_cache, at::Tensor& k_scale, double eps) {
+  CHECK_F32(q_out);
+  CHECK_F32(w);
+  CHECK_F32(k_scale);
+  CHECK_ROWS(q);
+  CHECK_ROWS(k);
+  CHECK_I32(slot_mapping);
+  const int f32 = act_is_f32(k_cache, "k_cache");
+  TORCH_CHECK(k_cache.dim() == 4 && k_cache.is_contiguous(),
+              "k_cache [blocks, kv_heads, block, dim]");
+  const int tokens = q.size(0);
+  const int G = k_cache.size(1), bs = k_cache.size(2), D = k_cache.size(3);
+  TORCH_CHECK(act_is_f32(q, "q") == f32 && act_is_f32(k, "k") == f32 &&
+                  k.size(0) == tokens && k.size(1) == G * D &&
+                  w.numel() == q.size(1) && q_out.numel() == q.numel() &&
+                  slot_mapping.numel() >= tokens &&
+                  k_scale.numel() == k_cache.size(0) * bs,
+              "talk_prep_cache: dtype/shape mismatch");
+  check_hip(ks_talk_prep_cache(q_out.data_ptr(), q.data_ptr(), q.stride(0),
+                               k.data_ptr(), k.stride(0), w.data_ptr(),
+                               slot_mapping.data_ptr(), k_cache.data_ptr(),
+                               k_scale.data_ptr(), (float)eps, tokens,
+                               (int)q.size(1), G, D, bs, f32, current_stream()),
+            "talk_prep_cache");
+}
+
+void talk_attention(at::Tensor& out, at::Tensor& q, at::Tensor& k_cache,
+                    at::Tensor& k_scale, at::Tensor& block_tables,
+                    at::Tensor& cu_q, at::Tensor& ctx_lens, at::Tensor& talk,
+                    at::Tensor& bias, const c10::optional<at::Tensor>& gate,
+                    double scale, int64_t max_q_len, int64_t heads,
+                    int64_t window) {
+  CHECK_F32(q);
+  CHECK_F32(k_scale);
+  CHECK_F32(talk);
+  CHECK_F32(bias);
+  CHECK_I32(cu_q);
+  CHECK_I32(ctx_lens);
+  TORCH_CHECK(block_tables.is_cuda() && block_tables.scalar_type() == at::kInt &&
+                  block_tables.dim() == 2 && block_tables.stride(1) == 1,
+              "block_tables [seqs, blocks] int32");
+  TORCH_CHECK(k_cache.dim() == 4 && k_cache.is_contiguous() && out.is_contiguous(),
+              "k_cache [blocks, kv_heads, block, dim]");
+  const int f32 = act_is_f32(out, "out");
+  const int G = k_cache.size(1), bs = k_cache.size(2), D = k_cache.size(3);
+  const int num_seqs = ctx_lens.numel();
+  TORCH_CHECK(heads > 0 && heads % G == 0 && heads <= 96 && D <= 256,
+              "talk_attention: at most 96 heads of at most 256 columns");
+  const int64_t tokens = q.numel() / (heads * D);
+  TORCH_CHECK(act_is_f32(k_cache, "k_cache") == f32 &&
+                  q.numel() == tokens * heads * D &&
+                  out.numel() == q.numel() && cu_q.numel() == num_seqs + 1 &&
+                  block_tables.size(0) >= num_seqs &&
+                  k_scale.numel() == k_cache.size(0) * bs &&
+                  k_cache.size(0) * G * bs < (int64_t(1) << 31) &&
+                  talk.numel() == heads * heads && bias.dim() == 2 &&
+                  bias.size(0) == heads && window >= 0,
+              "talk_attention: dtype/shape mismatch");
+  const void* gp = nullptr;
+  long gst = 0;
+  if (gate.has_value()) {
+    CHECK_ROWS(*gate);
+    TORCH_CHECK(act_is_f32(*gate, "gate") == f32 && gate->size(0) == tokens &&
+                    gate->size(1) == heads * D,
+                "gate [T, heads*dim] in the activation dtype");
+    gp = gate->data_ptr();
+    gst = gate->stride(0);
+  }
+  int nsplit = 1;
+  at::Tensor ws;
+  if (max_q_len == 1) {
+    nsplit = ks_talk_decode_splits(num_seqs, (int)window);
+    ws = at::empty({(int64_t)num_seqs * heads * nsplit * (D + 2)},
+                   q.options().dtype(at::kFloat));
+  }
+  check_hip(ks_talk_attention(
+                out.data_ptr(), q.data_ptr(), k_cache.data_ptr(),
+                k_scale.data_ptr(), block_tables.data_ptr(),
+                (int)block_tables.stride(0), cu_q.data_ptr(),
+                ctx_lens.data_ptr(), talk.data_ptr(), bias.data_ptr(),
+                (int)bias.size(1), gp, gst, (float)scale, num_seqs,
+                (int)max_q_len, (int)heads, G, D, bs, (int)window, f32,
+                max_q_len == 1 ? ws.data_ptr() : nullptr, nsplit,
+                current_stream()),
+            "talk_attention");
 }
 
 void bias_gelu_tanh(at::Tensor& out, at::Tensor& input, at::Tensor& bias) {
@@ -1028,6 +1259,15 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
         "rotary positions on projection heads, times a constant, fp32 out");
   m.def("unit_norm_heads", &unit_norm_heads,
         "per-head unit vectors times a constant, in place");
+  m.def("delta_unit_decay", &delta_unit_decay,
+        "unit-norm q/k heads and per-channel decays");
+  m.def("post_group_norm_add", &post_group_norm_add,
+        "group RMS norm of a sublayer output, fp32 residual add, next input");
+  m.def("diff_combine", &diff_combine, "normed difference of two head outputs");
+  m.def("talk_prep_cache", &talk_prep_cache,
+        "whole-row query norm, key pages and their 1/rms");
+  m.def("talk_attention", &talk_attention,
+        "paged fp32 attention with scores mixed over the heads");
   m.def("linear_scan", &linear_scan,
         "decay / gated-delta linear-attention recurrence, per-slot fp32 state");
   def_sampling(m);

@@ -11,6 +11,10 @@
 //   delta form (gated delta): S <- g S;  u = b (v - S^T k);
 //                             S <- S + k u^T                   o = S^T q
 //
+// A third form has one decay per head AND key channel, read per token from
+// fp32 rows: S <- diag(g) S first (one multiplication per state element), then
+// the delta form with g = 1.
+//
 // d is a constant per head; g = exp(-exp(A_log) softplus(a + dt_bias)) and
 // b = sigmoid(beta_raw) are computed here in fp32 from raw per-token, per-head
 // projection columns. Both forms are evaluated from the OLD state with two
@@ -33,6 +37,8 @@
 //    after them are only widened to fp32 (values).
 //  * unit_norm_heads: x / sqrt(sum(x^2) + eps) * scale per head, in place on
 //    fp32 rows; two runs of heads with a scale each (queries, keys).
+//  * delta_unit_decay: the unit norms, and for the third form the decays
+//    g = exp(-exp(A_log) softplus(a + dt_bias)) per head and key channel.
 #include "dtype_io.h"
 
 #include <type_traits>
@@ -106,11 +112,41 @@ __global__ void unit_norm_heads_kernel(float* __restrict__ x, long stride,
   }
 }
 
+// unit norms of q and k heads in place (as above, scale 1 for k), and the
+// decay of every head and key channel
+template <typename T>
+__global__ void delta_unit_decay_kernel(
+    float* __restrict__ x, long stride, float* __restrict__ g,
+    const T* __restrict__ a_raw, long a_stride, const float* __restrict__ a_log,
+    const float* __restrict__ dt_bias, int qk_heads, int dim, float q_scale,
+    float eps, int decays) {
+  const long t = blockIdx.x;
+  const int lane = threadIdx.x & 63;
+  const int wave = threadIdx.x >> 6;
+  for (int job = wave; job < 2 * qk_heads; job += NW) {
+    float* p = x + t * stride + (long)job * dim;
+    float ss = 0.f;
+    for (int i = lane; i < dim; i += WAVE_SIZE) ss += p[i] * p[i];
+    ss = wave_reduce_sum(ss);
+    const float m = (job < qk_heads ? q_scale : 1.0f) / sqrtf(ss + eps);
+    for (int i = lane; i < dim; i += WAVE_SIZE) p[i] *= m;
+  }
+  for (int e = threadIdx.x; e < decays; e += NT) {
+    const float z = ld_f32(a_raw, t * a_stride + e) + dt_bias[e];
+    // softplus without a clamp; log1p(exp(z)) is z itself past z ~ 30
+    const float sp = z > 30.f ? z : log1pf(expf(z));
+    g[t * decays + e] = expf(-expf(a_log[e / dim]) * sp);
+  }
+}
+
 constexpr int SCAN_TC = 16;  // tokens per chunk
+
+// recurrence forms
+constexpr int DECAY = 0, HEAD_DELTA = 1, CHANNEL_DELTA = 2;
 
 // R = state rows per lane (K <= 16 R), PC = columns per lane (a block covers
 // 16 PC value columns of one head).
-template <int R, int PC, bool DELTA>
+template <int R, int PC, int FORM>
 __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(4)))
 linear_scan_kernel(
     float* __restrict__ o, const float* __restrict__ q, long q_stride,
@@ -119,10 +155,13 @@ linear_scan_kernel(
     const float* __restrict__ a_f32, const short* __restrict__ a_bf16,
     const float* __restrict__ b_f32, const short* __restrict__ b_bf16,
     long ab_stride, const float* __restrict__ a_log,
-    const float* __restrict__ dt_bias, float* __restrict__ state,
+    const float* __restrict__ dt_bias, const float* __restrict__ channel_decay,
+    float* __restrict__ state,
     const long* __restrict__ positions, const int* __restrict__ cu_seqlens,
     const int* __restrict__ slots, int heads, int qk_heads, int V, int K) {
   extern __shared__ float lds[];
+  constexpr bool DELTA = FORM != DECAY;
+  constexpr bool CHAN = FORM == CHANNEL_DELTA;
   constexpr int tc = SCAN_TC;
   constexpr int XS = 16 * PC;
   const int s = blockIdx.z;
@@ -139,10 +178,11 @@ linear_scan_kernel(
   const long slot = slots[s];
   const bool fresh = positions[first] == 0;
   const float fixed = DELTA ? 1.f : decay[h];
-  const float A = DELTA ? -expf(a_log[h]) : 0.f;
-  const float bias = DELTA ? dt_bias[h] : 0.f;
+  const float A = FORM == HEAD_DELTA ? -expf(a_log[h]) : 0.f;
+  const float bias = FORM == HEAD_DELTA ? dt_bias[h] : 0.f;
 
   // LDS: k[tc][K] | q[tc][K] | v[tc][XS] | g[tc] | beta[tc] | k.q[tc] | o[tc][XS]
+  //      | channel decays [tc][K]
   float* Ks = lds;
   float* Qs = Ks + tc * K;
   float* Vs = Qs + tc * K;
@@ -150,6 +190,7 @@ linear_scan_kernel(
   float* Bs = Gs + tc;
   float* Ds = Bs + tc;
   float* Os = Ds + tc;
+  float* Cs = Os + tc * XS;
   float S[R][PC];
   float* sp = state + ((slot * heads + h) * (long)V) * K;
 #pragma unroll
@@ -166,7 +207,7 @@ linear_scan_kernel(
   // element of the token's k, q and v rows
   const int stk = threadIdx.x >> 4;
   const int sl = threadIdx.x & 15;
-  float sK[R], sQ[R], sV[PC], sa = 0.f, sb = 0.f;
+  float sK[R], sQ[R], sC[CHAN ? R : 1], sV[PC], sa = 0.f, sb = 0.f;
   auto prefetch = [&](int t0, int cnt) {
     const bool on = stk < cnt;
     const long t = first + t0 + (on ? stk : 0);
@@ -179,6 +220,7 @@ linear_scan_kernel(
       const bool ok = on && n < K;
       sK[r] = ok ? krow[n] : 0.f;
       sQ[r] = ok ? qrow[n] : 0.f;
+      if (CHAN) sC[r] = ok ? channel_decay[(t * heads + h) * K + n] : 0.f;
     }
 #pragma unroll
     for (int c = 0; c < PC; ++c) {
@@ -187,7 +229,7 @@ linear_scan_kernel(
     }
     if (DELTA && on && sl == 0) {
       const long i = t * ab_stride + h;
-      sa = (a_f32 ? a_f32[i] : bf16_bits_to_float(a_bf16[i])) + bias;
+      if (!CHAN) sa = (a_f32 ? a_f32[i] : bf16_bits_to_float(a_bf16[i])) + bias;
       sb = b_f32 ? b_f32[i] : bf16_bits_to_float(b_bf16[i]);
     }
   };
@@ -203,6 +245,7 @@ linear_scan_kernel(
         if (n < K) {
           Ks[stk * K + n] = sK[r];
           Qs[stk * K + n] = sQ[r];
+          if (CHAN) Cs[stk * K + n] = sC[r];
         }
       }
 #pragma unroll
@@ -212,7 +255,7 @@ linear_scan_kernel(
         if (DELTA) {
           // softplus without a clamp; log1p(exp(x)) is x itself past x ~ 30
           const float sp_ = sa > 30.f ? sa : log1pf(expf(sa));
-          Gs[stk] = expf(A * sp_);
+          Gs[stk] = CHAN ? 1.f : expf(A * sp_);
           Bs[stk] = 1.0f / (1.0f + expf(-sb));
         } else {
           Gs[stk] = fixed;
@@ -238,6 +281,11 @@ linear_scan_kernel(
         const bool ok = n < K;
         kk[r] = ok ? Ks[tk * K + n] : 0.f;
         qq[r] = ok ? Qs[tk * K + n] : 0.f;
+        if (CHAN) {
+          const float gc = ok ? Cs[tk * K + n] : 0.f;
+#pragma unroll
+          for (int c = 0; c < PC; ++c) S[r][c] *= gc;
+        }
       }
 #pragma unroll
       for (int c = 0; c < PC; ++c) {
@@ -253,11 +301,11 @@ linear_scan_kernel(
         float u = vv;
         if (DELTA) {
           p1 = row16_sum(p1);
-          u = bt * (vv - g * p1);
+          u = bt * (vv - (CHAN ? p1 : g * p1));
         }
 #pragma unroll
-        for (int r = 0; r < R; ++r) S[r][c] = g * S[r][c] + kk[r] * u;
-        if (ns == 0) Os[tk * XS + col] = g * p2 + u * kq;
+        for (int r = 0; r < R; ++r) S[r][c] = (CHAN ? S[r][c] : g * S[r][c]) + kk[r] * u;
+        if (ns == 0) Os[tk * XS + col] = (CHAN ? p2 : g * p2) + u * kq;
       }
     }
     __syncthreads();
@@ -317,6 +365,26 @@ extern "C" hipError_t ks_unit_norm_heads(void* x, long stride, int tokens,
   return hipSuccess;
 }
 
+extern "C" hipError_t ks_delta_unit_decay(
+    void* x, long stride, void* g, const void* a_raw, long a_stride,
+    const void* a_log, const void* dt_bias, int tokens, int qk_heads, int dim,
+    float q_scale, float eps, int decays, int is_f32, hipStream_t stream) {
+  if (tokens == 0) return hipSuccess;
+  if (dim < 1 || decays % dim != 0) return hipErrorInvalidValue;
+  if (is_f32)
+    hipLaunchKernelGGL(delta_unit_decay_kernel<float>, dim3(tokens), dim3(NT), 0,
+                       stream, (float*)x, stride, (float*)g, (const float*)a_raw,
+                       a_stride, (const float*)a_log, (const float*)dt_bias,
+                       qk_heads, dim, q_scale, eps, decays);
+  else
+    hipLaunchKernelGGL(delta_unit_decay_kernel<short>, dim3(tokens), dim3(NT), 0,
+                       stream, (float*)x, stride, (float*)g, (const short*)a_raw,
+                       a_stride, (const float*)a_log, (const float*)dt_bias,
+                       qk_heads, dim, q_scale, eps, decays);
+  HIP_CHECK_KERNEL();
+  return hipSuccess;
+}
+
 #define LSCAN_LAUNCH(RR, PCC, DD)                                             \
   hipLaunchKernelGGL((linear_scan_kernel<RR, PCC, DD>), grid, dim3(256), smem, \
                      stream, (float*)o, (const float*)q, q_stride,            \
@@ -327,7 +395,7 @@ extern "C" hipError_t ks_unit_norm_heads(void* x, long stride, int tokens,
                      ab_is_f32 ? (const float*)b_raw : nullptr,               \
                      ab_is_f32 ? nullptr : (const short*)b_raw, ab_stride,    \
                      (const float*)a_log, (const float*)dt_bias,              \
-                     (float*)state, (const long*)positions,                   \
+                     (const float*)channel_decay, (float*)state, (const long*)positions,                   \
                      (const int*)cu_seqlens, (const int*)slots, heads,        \
                      qk_heads, V, K)
 
@@ -348,20 +416,20 @@ extern "C" hipError_t ks_unit_norm_heads(void* x, long stride, int tokens,
     else LSCAN_LAUNCH(16, 2, DD);                                             \
   } while (0)
 
-// decay != null: decay form; otherwise the delta form, which reads a_raw /
-// b_raw [T, heads] (two column ranges of rows with one stride), a_log and
-// dt_bias.
+// decay != null: decay form; otherwise a delta form, which reads b_raw
+// [T, heads] and either channel_decay [T, heads*K] or a_raw [T, heads] (a and
+// b: two column ranges of rows with one stride), a_log and dt_bias.
 extern "C" hipError_t ks_linear_scan(
     void* o, const void* q, long q_stride, const void* k, long k_stride,
     const void* v, long v_stride, const void* decay, const void* a_raw,
     const void* b_raw, long ab_stride, int ab_is_f32, const void* a_log,
-    const void* dt_bias, void* state, const void* positions,
-    const void* cu_seqlens, const void* slots, int num_seqs, int heads,
-    int qk_heads, int V, int K, hipStream_t stream) {
+    const void* dt_bias, const void* channel_decay, void* state,
+    const void* positions, const void* cu_seqlens, const void* slots,
+    int num_seqs, int heads, int qk_heads, int V, int K, hipStream_t stream) {
   if (num_seqs == 0) return hipSuccess;
   if (qk_heads <= 0 || heads % qk_heads != 0 || K < 1 || K > 256 || V < 1)
     return hipErrorInvalidValue;
-  if (!decay && (!a_raw || !b_raw || !a_log || !dt_bias))
+  if (!decay && (!b_raw || (!channel_decay && (!a_raw || !a_log || !dt_bias))))
     return hipErrorInvalidValue;
   const int R = cdiv(K, 16);
   int pc = V > 32 ? 4 : (V > 16 ? 2 : 1);
@@ -370,10 +438,11 @@ extern "C" hipError_t ks_linear_scan(
   // (sequence, head) pairs takes narrower tiles to put more blocks on the chip
   while (pc > 1 && (long)cdiv(V, 16 * pc) * heads * num_seqs < 1024) pc >>= 1;
   const int xs = 16 * pc;
-  const size_t smem = sizeof(float) * ((size_t)SCAN_TC * (2 * K + 2 * xs + 3));
+  const size_t smem = sizeof(float) * ((size_t)SCAN_TC * ((channel_decay ? 3 : 2) * K + 2 * xs + 3));
   dim3 grid(cdiv(V, xs), heads, num_seqs);
-  if (decay) LSCAN_LAUNCH_R(false);
-  else LSCAN_LAUNCH_R(true);
+  if (decay) LSCAN_LAUNCH_R(DECAY);
+  else if (channel_decay) LSCAN_LAUNCH_R(CHANNEL_DELTA);
+  else LSCAN_LAUNCH_R(HEAD_DELTA);
   HIP_CHECK_KERNEL();
   return hipSuccess;
 }

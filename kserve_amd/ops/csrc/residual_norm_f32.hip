@@ -20,6 +20,15 @@
 //    the normed value; a weight shorter than the row repeats; no weight = 1)
 //    otherwise: v = y * silu(z), normalised separately in equal
 //    contiguous groups of the row, times a weight (gate before the norm).
+//    gate_sigmoid: the gate is sigmoid(z) instead of silu(z).
+//  * post_group_norm_add: residual += GroupRMS(d) * weight, every one of
+//    `groups` equal parts of the row divided by its own RMS; d is a sublayer
+//    output or half the sum of two, each first RMS-normed over the row with a
+//    weight of its own. out = the new residual in the activation dtype or its
+//    group norm times next_weight. One pass closes a sublayer and hands the
+//    stream to the next.
+//  * diff_combine: per head, first - lambda * second of two fp32 outputs,
+//    divided by its RMS over the head, times a constant.
 //
 // Everything is accumulated in fp32 with exact (non-approximate) sqrt and
 // division: these ops sit on the 32-bit path of the models that use them.
@@ -417,6 +426,11 @@ __global__ void post_norm_add_rms_norm_vec4_kernel(
   }
 }
 
+// silu(z), or sigmoid(z)
+__device__ __forceinline__ float gate_of(float z, int sigmoid) {
+  return (sigmoid ? 1.0f : z) / (1.0f + expf(-z));
+}
+
 template <typename TZ, typename TO>
 __global__ void gated_group_rms_norm_kernel(TO* __restrict__ out,
                                             const float* __restrict__ y,
@@ -424,7 +438,8 @@ __global__ void gated_group_rms_norm_kernel(TO* __restrict__ out,
                                             long z_stride,
                                             const float* __restrict__ weight,
                                             int weight_n, float eps, int inner,
-                                            int group_size, int gate_after) {
+                                            int group_size, int gate_after,
+    int sigmoid) {
   __shared__ float scratch[NW];
   const long row = blockIdx.x;
   const int g0 = blockIdx.y * group_size;
@@ -432,14 +447,14 @@ __global__ void gated_group_rms_norm_kernel(TO* __restrict__ out,
   for (int i = threadIdx.x; i < group_size; i += NT) {
     const float zf = ld_f32(z, row * z_stride + g0 + i);
     const float yv = y[row * inner + g0 + i];
-    const float v = gate_after ? yv : yv * (zf / (1.0f + expf(-zf)));
+    const float v = gate_after ? yv : yv * gate_of(zf, sigmoid);
     ss += v * v;
   }
   ss = block_sum_sync<NW>(ss, scratch);
   const float inv = 1.0f / sqrtf(ss / (float)group_size + eps);
   for (int i = threadIdx.x; i < group_size; i += NT) {
     const float zf = ld_f32(z, row * z_stride + g0 + i);
-    const float gate = zf / (1.0f + expf(-zf));
+    const float gate = gate_of(zf, sigmoid);
     const float yv = y[row * inner + g0 + i];
     const float w = weight ? weight[(g0 + i) % weight_n] : 1.0f;
     st_f32(out, row * inner + g0 + i,
@@ -451,7 +466,8 @@ template <typename TZ, typename TO>
 __global__ void gated_group_rms_norm_vec4_kernel(
     TO* __restrict__ out, const float* __restrict__ y, const TZ* __restrict__ z,
     long z_stride, const float* __restrict__ weight, int weight_n, float eps,
-    int inner, int group_size, int gate_after) {
+    int inner, int group_size, int gate_after,
+    int sigmoid) {
   __shared__ float scratch[NW];
   const long row = blockIdx.x;
   const int g0 = blockIdx.y * group_size;
@@ -466,7 +482,7 @@ __global__ void gated_group_rms_norm_vec4_kernel(
       ld4<TZ>(z + row * z_stride + g0 + i, zv);
 #pragma unroll
       for (int j = 0; j < 4; ++j) {
-        const float sg = zv[j] / (1.0f + expf(-zv[j]));
+        const float sg = gate_of(zv[j], sigmoid);
         const float v = gate_after ? yv[j] : yv[j] * sg;
         gate[k][j] = gate_after ? sg : 1.0f;
         keep[k][j] = v;
@@ -496,7 +512,8 @@ template <typename TZ, typename TO>
 __global__ void __launch_bounds__(NT) gated_group_rms_norm_wave_kernel(
     TO* __restrict__ out, const float* __restrict__ y, const TZ* __restrict__ z,
     long z_stride, const float* __restrict__ weight, int weight_n, float eps,
-    int inner, int group_size, int groups, int gate_after) {
+    int inner, int group_size, int groups, int gate_after,
+    int sigmoid) {
   const long row = blockIdx.x;
   const int lane = threadIdx.x & 63;
   const int i = lane * 4;
@@ -511,7 +528,7 @@ __global__ void __launch_bounds__(NT) gated_group_rms_norm_wave_kernel(
       ld4<TZ>(z + row * z_stride + g0 + i, zv);
 #pragma unroll
       for (int j = 0; j < 4; ++j) {
-        const float sg = zv[j] / (1.0f + expf(-zv[j]));
+        const float sg = gate_of(zv[j], sigmoid);
         if (gate_after) gate[j] = sg;
         else v[j] *= sg;
         ss += v[j] * v[j];
@@ -527,6 +544,156 @@ __global__ void __launch_bounds__(NT) gated_group_rms_norm_wave_kernel(
       st4<TO>(out + row * inner + g0 + i, o);
     }
   }
+}
+
+// 1/rms of every group of a row of `width` floats in LDS, into inv[groups].
+// With fewer groups than waves several waves share a group (part[NW] holds
+// their sums); starts and ends with a barrier.
+__device__ __forceinline__ void group_inv_rms(const float* row, float* inv,
+                                              float* part, int groups, int gs,
+                                              float eps) {
+  const int lane = threadIdx.x & 63;
+  const int wave = threadIdx.x >> 6;
+  const int wpg = groups < NW ? NW / groups : 1;  // waves per group
+  __syncthreads();
+  if (wpg == 1) {
+    for (int g = wave; g < groups; g += NW) {
+      float ss = 0.f;
+      for (int i = lane; i < gs; i += WAVE_SIZE) {
+        const float v = row[g * gs + i];
+        ss += v * v;
+      }
+      ss = wave_reduce_sum(ss);
+      if (lane == 0) inv[g] = 1.0f / sqrtf(ss / (float)gs + eps);
+    }
+    __syncthreads();
+    return;
+  }
+  const int g = wave / wpg;
+  float ss = 0.f;
+  if (g < groups)
+    for (int i = (wave % wpg) * WAVE_SIZE + lane; i < gs; i += wpg * WAVE_SIZE) {
+      const float v = row[g * gs + i];
+      ss += v * v;
+    }
+  ss = wave_reduce_sum(ss);
+  if (lane == 0) part[wave] = ss;
+  __syncthreads();
+  if (threadIdx.x < groups) {
+    float t = 0.f;
+    for (int w = 0; w < wpg; ++w) t += part[threadIdx.x * wpg + w];
+    inv[threadIdx.x] = 1.0f / sqrtf(t / (float)gs + eps);
+  }
+  __syncthreads();
+}
+
+// VEC = 4 elements per lane and step (widths, group sizes, strides and
+// pointers aligned), or 1. The row passes through LDS once.
+template <typename TD, typename TO, int VEC>
+__global__ void __launch_bounds__(NT) post_group_norm_add_kernel(
+    float* __restrict__ residual, const TD* __restrict__ d0, long d0_stride,
+    const TD* __restrict__ d1, long d1_stride, const float* __restrict__ weight,
+    const float* __restrict__ pre_w0, const float* __restrict__ pre_w1,
+    int groups, float eps, TO* __restrict__ out,
+    const float* __restrict__ next_weight, int width) {
+  extern __shared__ float rows[];  // [width] | inv [groups]
+  __shared__ float part[NW];
+  float* inv = rows + width;
+  const long row = blockIdx.x;
+  float* r = residual + row * width;
+  const int gs = width / groups;
+  auto load = [&](const auto* p, float* v) {
+    if constexpr (VEC == 4) ld4(p, v);
+    else v[0] = ld_f32(p, 0);
+  };
+  auto store = [&](auto* p, const float* v) {
+    if constexpr (VEC == 4) st4(p, v);
+    else st_f32(p, 0, v[0]);
+  };
+  if (d0) {
+    if (d1) {
+      float s0 = 0.f, s1 = 0.f;
+      for (int i = threadIdx.x * VEC; i < width; i += NT * VEC) {
+        float a[VEC], b[VEC];
+        load(d0 + row * d0_stride + i, a);
+        load(d1 + row * d1_stride + i, b);
+#pragma unroll
+        for (int c = 0; c < VEC; ++c) {
+          s0 += a[c] * a[c];
+          s1 += b[c] * b[c];
+        }
+      }
+      s0 = block_sum_sync<NW>(s0, part);
+      s1 = block_sum_sync<NW>(s1, part);
+      const float i0 = 0.5f / sqrtf(s0 / (float)width + eps);
+      const float i1 = 0.5f / sqrtf(s1 / (float)width + eps);
+      for (int i = threadIdx.x * VEC; i < width; i += NT * VEC) {
+        float a[VEC], b[VEC], w0[VEC], w1[VEC];
+        load(d0 + row * d0_stride + i, a);
+        load(d1 + row * d1_stride + i, b);
+        load(pre_w0 + i, w0);
+        load(pre_w1 + i, w1);
+#pragma unroll
+        for (int c = 0; c < VEC; ++c) a[c] = a[c] * i0 * w0[c] + b[c] * i1 * w1[c];
+        store(rows + i, a);
+      }
+    } else {
+      for (int i = threadIdx.x * VEC; i < width; i += NT * VEC) {
+        float a[VEC];
+        load(d0 + row * d0_stride + i, a);
+        store(rows + i, a);
+      }
+    }
+    group_inv_rms(rows, inv, part, groups, gs, eps);
+  }
+  for (int i = threadIdx.x * VEC; i < width; i += NT * VEC) {
+    float v[VEC];
+    load(r + i, v);
+    if (d0) {
+      float a[VEC], w[VEC];
+      load(rows + i, a);
+      load(weight + i, w);
+      const float m = inv[i / gs];
+#pragma unroll
+      for (int c = 0; c < VEC; ++c) v[c] += a[c] * m * w[c];
+      store(r + i, v);
+    }
+    // each thread overwrites only what it has just read itself
+    if (next_weight) store(rows + i, v);
+    else if (out) store(out + row * width + i, v);
+  }
+  if (!out || !next_weight) return;
+  group_inv_rms(rows, inv, part, groups, gs, eps);
+  for (int i = threadIdx.x * VEC; i < width; i += NT * VEC) {
+    float v[VEC], w[VEC];
+    load(rows + i, v);
+    load(next_weight + i, w);
+    const float m = inv[i / gs];
+#pragma unroll
+    for (int c = 0; c < VEC; ++c) v[c] *= m * w[c];
+    store(out + row * width + i, v);
+  }
+}
+
+// A wave per (token, head).
+template <typename TO>
+__global__ void __launch_bounds__(NT) diff_combine_kernel(
+    TO* __restrict__ out, const float* __restrict__ o,
+    const float* __restrict__ lam, long items, int V, float eps, float mult) {
+  const long item = (long)blockIdx.x * NW + (threadIdx.x >> 6);
+  if (item >= items) return;
+  const int lane = threadIdx.x & 63;
+  const float l = lam[0];
+  const float* a = o + item * 2 * V;
+  float ss = 0.f;
+  for (int i = lane; i < V; i += WAVE_SIZE) {
+    const float d = a[i] - l * a[V + i];
+    ss += d * d;
+  }
+  ss = wave_reduce_sum(ss);
+  const float m = mult / sqrtf(ss / (float)V + eps);
+  for (int i = lane; i < V; i += WAVE_SIZE)
+    st_f32(out, item * V + i, (a[i] - l * a[V + i]) * m);
 }
 
 }  // namespace
@@ -681,7 +848,7 @@ extern "C" hipError_t ks_gated_group_rms_norm(void* out, const void* y,
                                               const void* weight, int weight_n,
                                               float eps, int rows, int inner,
                                               int groups, int gate_after,
-                                              int is_f32,
+                                              int gate_sigmoid, int is_f32,
                                               hipStream_t stream) {
   if (rows == 0) return hipSuccess;
   if (groups <= 0 || inner % groups != 0) return hipErrorInvalidValue;
@@ -703,11 +870,11 @@ extern "C" hipError_t ks_gated_group_rms_norm(void* out, const void* y,
     if (is_f32)
       hipLaunchKernelGGL((gated_group_rms_norm_wave_kernel<float, float>),
                          dim3(rows), dim3(NT), 0, stream, GNORM_ARGS(float),
-                         groups, gate_after);
+                         groups, gate_after, gate_sigmoid);
     else
       hipLaunchKernelGGL((gated_group_rms_norm_wave_kernel<short, short>),
                          dim3(rows), dim3(NT), 0, stream, GNORM_ARGS(short),
-                         groups, gate_after);
+                         groups, gate_after, gate_sigmoid);
     HIP_CHECK_KERNEL();
     return hipSuccess;
   }
@@ -715,21 +882,87 @@ extern "C" hipError_t ks_gated_group_rms_norm(void* out, const void* y,
     if (vec)
       hipLaunchKernelGGL((gated_group_rms_norm_vec4_kernel<float, float>),
                          dim3(rows, groups), dim3(NT), 0, stream,
-                         GNORM_ARGS(float), gate_after);
+                         GNORM_ARGS(float), gate_after, gate_sigmoid);
     else
       hipLaunchKernelGGL((gated_group_rms_norm_kernel<float, float>),
                          dim3(rows, groups), dim3(NT), 0, stream,
-                         GNORM_ARGS(float), gate_after);
+                         GNORM_ARGS(float), gate_after, gate_sigmoid);
   } else {
     if (vec)
       hipLaunchKernelGGL((gated_group_rms_norm_vec4_kernel<short, short>),
                          dim3(rows, groups), dim3(NT), 0, stream,
-                         GNORM_ARGS(short), gate_after);
+                         GNORM_ARGS(short), gate_after, gate_sigmoid);
     else
       hipLaunchKernelGGL((gated_group_rms_norm_kernel<short, short>),
                          dim3(rows, groups), dim3(NT), 0, stream,
-                         GNORM_ARGS(short), gate_after);
+                         GNORM_ARGS(short), gate_after, gate_sigmoid);
   }
+  HIP_CHECK_KERNEL();
+  return hipSuccess;
+}
+
+template <typename TD, typename TO>
+static void launch_post_group_norm(bool vec, void* residual, const void* d0,
+                                   long d0_stride, const void* d1,
+                                   long d1_stride, const void* weight,
+                                   const void* pre_w0, const void* pre_w1,
+                                   int groups, float eps, void* out,
+                                   const void* next_weight, int rows, int width,
+                                   hipStream_t stream) {
+  auto fn = vec ? post_group_norm_add_kernel<TD, TO, 4>
+                : post_group_norm_add_kernel<TD, TO, 1>;
+  const size_t smem = sizeof(float) * ((size_t)width + groups);
+  hipLaunchKernelGGL(fn, dim3(rows), dim3(NT), smem, stream, (float*)residual,
+                     (const TD*)d0, d0_stride, (const TD*)d1, d1_stride,
+                     (const float*)weight, (const float*)pre_w0,
+                     (const float*)pre_w1, groups, eps, (TO*)out,
+                     (const float*)next_weight, width);
+}
+
+extern "C" hipError_t ks_post_group_norm_add(
+    void* residual, const void* d0, long d0_stride, const void* d1,
+    long d1_stride, int d_is_f32, const void* weight, const void* pre_w0,
+    const void* pre_w1, int groups, float eps, void* out, int out_is_f32,
+    const void* next_weight, int rows, int width, hipStream_t stream) {
+  if (rows == 0 || (!d0 && !out)) return hipSuccess;
+  if (groups < 1 || width % groups != 0 || (d0 && !weight) || (d1 && !d0) ||
+      (d1 && (!pre_w0 || !pre_w1)) || width + groups > 15 * 1024)
+    return hipErrorInvalidValue;
+  auto al = [](const void* p, int bytes) { return ((uintptr_t)p % bytes) == 0; };
+  const int db = d_is_f32 ? 16 : 8;
+  const bool vec = (width / groups) % 4 == 0 && d0_stride % 4 == 0 &&
+                   d1_stride % 4 == 0 && al(residual, 16) && al(weight, 16) &&
+                   al(pre_w0, 16) && al(pre_w1, 16) && al(next_weight, 16) &&
+                   al(d0, db) && al(d1, db) && al(out, out_is_f32 ? 16 : 8);
+#define PGN_ARGS                                                              \
+  vec, residual, d0, d0_stride, d1, d1_stride, weight, pre_w0, pre_w1, groups, \
+      eps, out, next_weight, rows, width, stream
+  if (d_is_f32) {
+    if (out_is_f32) launch_post_group_norm<float, float>(PGN_ARGS);
+    else launch_post_group_norm<float, short>(PGN_ARGS);
+  } else {
+    if (out_is_f32) launch_post_group_norm<short, float>(PGN_ARGS);
+    else launch_post_group_norm<short, short>(PGN_ARGS);
+  }
+  HIP_CHECK_KERNEL();
+  return hipSuccess;
+}
+
+extern "C" hipError_t ks_diff_combine(void* out, const void* o, const void* lam,
+                                      int rows, int heads, int V, float eps,
+                                      float mult, int out_is_f32,
+                                      hipStream_t stream) {
+  const long items = (long)rows * heads;
+  if (items == 0) return hipSuccess;
+  const dim3 grid((unsigned)((items + NW - 1) / NW));
+  if (out_is_f32)
+    hipLaunchKernelGGL(diff_combine_kernel<float>, grid, dim3(NT), 0, stream,
+                       (float*)out, (const float*)o, (const float*)lam, items, V,
+                       eps, mult);
+  else
+    hipLaunchKernelGGL(diff_combine_kernel<short>, grid, dim3(NT), 0, stream,
+                       (short*)out, (const float*)o, (const float*)lam, items, V,
+                       eps, mult);
   HIP_CHECK_KERNEL();
   return hipSuccess;
 }

@@ -8,7 +8,7 @@
 // position 0 ignores whatever its slot held (slots are reused, never cleared).
 //
 //  * causal_conv_silu: depthwise causal convolution over `taps` inputs per
-//    channel + bias (optional) + silu. Inputs before the portion come from the conv
+//    channel + bias (optional) + silu (optional). Inputs before the portion come from the conv
 //    state (the last taps-1 raw inputs of the sequence), zeros before
 //    position 0.
 //  * conv_state_update: runs after the above, shifts the new raw inputs in.
@@ -55,7 +55,7 @@ __global__ void causal_conv_silu_kernel(
     const float* __restrict__ w, const float* __restrict__ bias,
     const T* __restrict__ conv_state, const long* __restrict__ positions,
     const int* __restrict__ seq_of_token, const int* __restrict__ cu_seqlens,
-    const int* __restrict__ slots, int channels, int taps) {
+    const int* __restrict__ slots, int channels, int taps, int silu) {
   const int t = blockIdx.y;
   const int c = blockIdx.x * blockDim.x + threadIdx.x;
   if (c >= channels) return;
@@ -78,7 +78,7 @@ __global__ void causal_conv_silu_kernel(
     }
     acc += w[(long)c * taps + j] * v;
   }
-  out[(long)t * channels + c] = silu_f(acc);
+  out[(long)t * channels + c] = silu ? silu_f(acc) : acc;
 }
 
 // 4 consecutive channels per lane (8- or 16-byte loads, 16-byte stores); the
@@ -106,7 +106,7 @@ __global__ void causal_conv_silu_vec4_kernel(
     const float* __restrict__ w, const float* __restrict__ bias,
     const T* __restrict__ conv_state, const long* __restrict__ positions,
     const int* __restrict__ seq_of_token, const int* __restrict__ cu_seqlens,
-    const int* __restrict__ slots, int tokens, int channels) {
+    const int* __restrict__ slots, int tokens, int channels, int silu) {
   const int c = (blockIdx.x * blockDim.x + threadIdx.x) * 4;
   if (c >= channels) return;
   constexpr int hist = TAPS - 1;
@@ -139,7 +139,7 @@ __global__ void causal_conv_silu_vec4_kernel(
     }
     float4_t o;
 #pragma unroll
-    for (int i = 0; i < 4; ++i) o[i] = silu_f(acc[i]);
+    for (int i = 0; i < 4; ++i) o[i] = silu ? silu_f(acc[i]) : acc[i];
     *reinterpret_cast<float4_t*>(out + (long)t * channels + c) = o;
   }
 }
@@ -336,7 +336,7 @@ extern "C" hipError_t ks_causal_conv_silu(
     void* out, const void* in, long in_stride, const void* w, const void* bias,
     void* conv_state, const void* positions, const void* seq_of_token,
     const void* cu_seqlens, const void* slots, int tokens, int num_seqs,
-    int channels, int taps, int is_f32, hipStream_t stream) {
+    int channels, int taps, int silu, int is_f32, hipStream_t stream) {
   if (tokens == 0) return hipSuccess;
   if (taps < 1 || taps > MAX_TAPS) return hipErrorInvalidValue;
   dim3 grid(cdiv(channels, 256), tokens);
@@ -355,7 +355,7 @@ extern "C" hipError_t ks_causal_conv_silu(
       (const int*)seq_of_token, (const int*)cu_seqlens, (const int*)slots
 #define CONV_VEC_K(TT, K)                                                     \
   hipLaunchKernelGGL((causal_conv_silu_vec4_kernel<TT, K>), grid_v,           \
-                     dim3(256), 0, stream, CONV_ARGS(TT), tokens, channels)
+                     dim3(256), 0, stream, CONV_ARGS(TT), tokens, channels, silu)
 #define CONV_VEC(TT)                                                          \
   do {                                                                        \
     if (taps == 2) CONV_VEC_K(TT, 2);                                         \
@@ -366,7 +366,7 @@ extern "C" hipError_t ks_causal_conv_silu(
     if (vec) CONV_VEC(float);
     else
       hipLaunchKernelGGL(causal_conv_silu_kernel<float>, grid, dim3(256), 0,
-                         stream, CONV_ARGS(float), channels, taps);
+                         stream, CONV_ARGS(float), channels, taps, silu);
     if (taps > 1)
       hipLaunchKernelGGL(conv_state_update_kernel<float>, grid_u, dim3(256), 0,
                          stream, (float*)conv_state, (const float*)in,
@@ -377,7 +377,7 @@ extern "C" hipError_t ks_causal_conv_silu(
     if (vec) CONV_VEC(short);
     else
       hipLaunchKernelGGL(causal_conv_silu_kernel<short>, grid, dim3(256), 0,
-                         stream, CONV_ARGS(short), channels, taps);
+                         stream, CONV_ARGS(short), channels, taps, silu);
     if (taps > 1)
       hipLaunchKernelGGL(conv_state_update_kernel<short>, grid_u, dim3(256), 0,
                          stream, (short*)conv_state, (const short*)in,

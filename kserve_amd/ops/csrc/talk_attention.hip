@@ -1,0 +1,757 @@
+// Softmax attention against the paged cache whose scores are mixed over the
+// heads before the softmax, in fp32 end to end:
+//
+//   score_g(i, j) = q_g(i) . k(j) * k_scale(j) * scale
+//   s_h = sum_g talk[h, g] score_g + bias[h, i - j]
+//   p   = exp(s_h) / (1 + sum exp(s_h))     (keys 0 <= i - j < window)
+//   o_h = sum_j p_j k(j), times sigmoid(gate) per element
+//
+// Pages hold the un-normed keys, which are the values too, and one factor per
+// row (1/rms of the whole key projection). `bias` [heads, n] is already mixed
+// over the heads and constant past distance n - 1.
+//
+//  * talk_prep_cache: whole-row RMS norm of the query projection times a weight
+//    (fp32 out), keys to the pages, 1/rms of the key row to k_scale.
+//  * talk_attention prefill: a block takes 16 consecutive tokens and ALL heads,
+//    8 waves. Per tile of 16 NKT keys: (1) every wave computes its heads'
+//    transposed scores S^T = K Q^T on the fp32 matrix cores
+//    (v_mfma_f32_16x16x4_f32; keys and queries straight from the caches, 64
+//    contiguous bytes per row and load) into LDS [head][key][query];
+//    (2) every wave takes some keys and mixes over the heads, in place: per key
+//    a [heads x heads] x [heads x 16 queries] product, again on the matrix
+//    cores; (3) every wave reads its heads' mixed scores back in accumulator
+//    layout (one query per lane column), adds the bias, masks, updates the
+//    running softmax and multiplies with the keys as values, whose weights
+//    never leave the registers. A wave works on NH heads at once; SHARE: they
+//    belong to one key group, so every key fragment is loaded once for all.
+//    More heads than 8 NH: further blocks (grid z) take the next ones and
+//    recompute the scores of all heads.
+//  * talk_attention decode (one token per sequence): a block takes one split
+//    of the sequence's keys, all heads: the heads of a key group are the
+//    matrix product's columns, 64 keys per tile; the mixed scores go through
+//    a [heads x heads] x [heads x 16 keys] product, the softmax runs with one
+//    key per lane. Partial results go to scratch; talk_merge_kernel combines
+//    the splits, adds the 1 of the denominator and applies the gate.
+#include "cache_chunk.h"
+
+namespace {
+
+constexpr int NT = 512;
+constexpr int NWV = NT / WAVE_SIZE;
+constexpr int QS = 20;  // floats per key row of a score tile (16 queries + pad)
+constexpr float LOG2E = 1.44269504088896340736f;
+
+template <typename T>
+__global__ void __launch_bounds__(256) talk_prep_cache_kernel(
+    float* __restrict__ q_out, const T* __restrict__ q, long q_stride,
+    const T* __restrict__ k, long k_stride, const float* __restrict__ w,
+    const int* __restrict__ slot_mapping, T* __restrict__ k_cache,
+    float* __restrict__ k_scale, float eps, int q_width, int kv_heads, int D,
+    int block_size, int vec) {
+  __shared__ float scratch[4];
+  const long t = blockIdx.x;
+  const T* qr = q + t * q_stride;
+  const T* kr = k + t * k_stride;
+  const int k_width = kv_heads * D;
+  float sq = 0.f, sk = 0.f;
+  for (int i = threadIdx.x * 4; i < q_width; i += 1024) {
+    const f32x4 x = load4_f32(qr + i, vec, q_width - i);
+    sq += x[0] * x[0] + x[1] * x[1] + x[2] * x[2] + x[3] * x[3];
+  }
+  for (int i = threadIdx.x * 4; i < k_width; i += 1024) {
+    const f32x4 x = load4_f32(kr + i, vec, k_width - i);
+    sk += x[0] * x[0] + x[1] * x[1] + x[2] * x[2] + x[3] * x[3];
+  }
+  sq = block_sum_sync<4>(sq, scratch);
+  sk = block_sum_sync<4>(sk, scratch);
+  const float qinv = 1.0f / sqrtf(sq / (float)q_width + eps);
+  for (int i = threadIdx.x * 4; i < q_width; i += 1024) {
+    const f32x4 x = load4_f32(qr + i, vec, q_width - i);
+    const f32x4 ww = load4_f32(w + i, vec, q_width - i);
+    if (vec) {
+      *reinterpret_cast<f32x4*>(q_out + t * q_width + i) = x * ww * qinv;
+    } else {
+      for (int c = 0; c < 4; ++c)
+        if (i + c < q_width) q_out[t * q_width + i + c] = x[c] * ww[c] * qinv;
+    }
+  }
+  const long slot = slot_mapping[t];
+  if (slot < 0) return;
+  const long blk = slot / block_size, off = slot % block_size;
+  if (threadIdx.x == 0)
+    k_scale[blk * block_size + off] = 1.0f / sqrtf(sk / (float)k_width + eps);
+  for (int i = threadIdx.x; i < k_width; i += 256) {
+    const int g = i / D, d = i % D;
+    k_cache[((blk * kv_heads + g) * block_size + off) * D + d] = kr[i];
+  }
+}
+
+// cache row (of kv head 0) and score factor of `count` keys from k0 on; keys
+// past `last` repeat the last one (masked later)
+__device__ __forceinline__ void key_rows(int* rows, float* ksc, int k0, int last,
+                                         int count, const int* bt,
+                                         int block_size, int kv_heads,
+                                         const float* k_scale, float mult) {
+  if ((int)threadIdx.x < count) {
+    const int kp = min(k0 + (int)threadIdx.x, last);
+    const int blk = bt[kp / block_size], po = kp % block_size;
+    rows[threadIdx.x] = blk * kv_heads * block_size + po;
+    ksc[threadIdx.x] = k_scale[(long)blk * block_size + po] * mult;
+  }
+}
+
+// LDS floats of the prefill kernel: scores [H4][16 NKT][QS] | talk^T [H4][16 HT]
+// | rows [2][16 NKT] | factors [2][16 NKT]
+template <typename T, int DP, int NH, int HT, bool SHARE>
+__global__ void __launch_bounds__(NT) talk_prefill_kernel(
+    T* __restrict__ out, const float* __restrict__ q,
+    const T* __restrict__ k_cache, const float* __restrict__ k_scale,
+    const int* __restrict__ block_tables, int bt_stride,
+    const int* __restrict__ cu_q, const int* __restrict__ ctx_lens,
+    const float* __restrict__ talk, const float* __restrict__ bias, int bias_n,
+    const T* __restrict__ gate, long gate_stride, float scale, int heads,
+    int kv_heads, int D, int block_size, int window) {
+  constexpr int NKT = HT <= 2 ? 2 : 1;
+  constexpr int BK = 16 * NKT;
+  extern __shared__ float lds[];
+  const int H4 = (heads + 3) & ~3;
+  float* S = lds;
+  float* Tt = S + H4 * BK * QS;
+  float* Ksc = Tt + H4 * 16 * HT;
+  int* Rows = reinterpret_cast<int*>(Ksc + 2 * BK);
+
+  const int s = blockIdx.y;
+  const int q0 = cu_q[s];
+  const int q_len = cu_q[s + 1] - q0;
+  const int tok0 = blockIdx.x * 16;
+  if (tok0 >= q_len) return;
+  const int nq = min(16, q_len - tok0);
+  const int base_pos = ctx_lens[s] - q_len + tok0;
+  const int last_pos = base_pos + nq - 1;
+  const int kbeg = window > 0 ? max(base_pos - window + 1, 0) : 0;
+  const int lane = threadIdx.x & 63;
+  const int wave = threadIdx.x >> 6;
+  const int li = lane & 15, lg = lane >> 4;
+  const int rep = heads / kv_heads;
+  const int items = (heads + NH - 1) / NH;
+  const int* bt = block_tables + (long)s * bt_stride;
+  const bool vec = (D % 8) == 0;
+  const float mult = scale * LOG2E;
+  const int qpos = li < nq ? base_pos + li : -1;
+  const int qstart = window > 0 ? qpos - window + 1 : 0;
+  const float* qrow = q + (long)(q0 + tok0 + min(li, nq - 1)) * heads * D;
+
+  for (int e = threadIdx.x; e < H4 * 16 * HT; e += NT) {
+    const int g = e / (16 * HT), h = e % (16 * HT);
+    Tt[e] = (g < heads && h < heads) ? talk[h * heads + g] : 0.f;
+  }
+  for (int e = heads * BK * QS + threadIdx.x; e < H4 * BK * QS; e += NT) S[e] = 0.f;
+  key_rows(Rows, Ksc, kbeg, last_pos, BK, bt, block_size, kv_heads, k_scale, mult);
+
+  // this wave's heads in steps (1) and (3) when one block covers all heads;
+  // otherwise step (1) walks all of them and step (3) takes this block's
+  const int item3 = blockIdx.z * NWV + wave;
+  f32x4 o[NH][DP / 16];
+  float m[NH], l[NH];
+#pragma unroll
+  for (int a = 0; a < NH; ++a) {
+    m[a] = -INFINITY;
+    l[a] = 0.f;
+#pragma unroll
+    for (int i = 0; i < DP / 16; ++i) o[a][i] = f32x4{0.f, 0.f, 0.f, 0.f};
+  }
+  __syncthreads();
+
+  int buf = 0;
+  for (int k0 = kbeg; k0 <= last_pos; k0 += BK, buf ^= 1) {
+    const int* rows = Rows + buf * BK;
+    const float* ksc = Ksc + buf * BK;
+    // (1) scores of all heads
+    for (int item = wave; item < items; item += NWV) {
+      int hh[NH];
+#pragma unroll
+      for (int a = 0; a < NH; ++a) hh[a] = min(item * NH + a, heads - 1);
+      f32x4 acc[NH][NKT];
+#pragma unroll
+      for (int a = 0; a < NH; ++a)
+#pragma unroll
+        for (int t = 0; t < NKT; ++t) acc[a][t] = f32x4{0.f, 0.f, 0.f, 0.f};
+      long krow[NKT];
+#pragma unroll
+      for (int t = 0; t < NKT; ++t) krow[t] = rows[16 * t + li];
+#pragma unroll
+      for (int k8 = 0; k8 < DP / 32; ++k8) {
+        // contraction step c of lane group lg stands for d = 32 k8 + 8 lg + c
+        const int d0 = 32 * k8 + 8 * lg;
+        Chunk8<T> kf[NKT];
+#pragma unroll
+        for (int a = 0; a < NH; ++a) {
+          if (a == 0 || !SHARE) {
+            const int g = hh[a] / rep;
+#pragma unroll
+            for (int t = 0; t < NKT; ++t) {
+              if (d0 < D)
+                kf[t].load(k_cache + (krow[t] + (long)g * block_size) * D + d0, vec,
+                           D - d0);
+              else
+                kf[t].zero();
+            }
+          }
+          Chunk8<float> qf;
+          if (d0 < D) qf.load(qrow + hh[a] * D + d0, vec, D - d0);
+          else qf.zero();
+#pragma unroll
+          for (int c = 0; c < 8; ++c)
+#pragma unroll
+            for (int t = 0; t < NKT; ++t)
+              acc[a][t] = __builtin_amdgcn_mfma_f32_16x16x4f32(
+                  kf[t].get(c), qf.get(c), acc[a][t], 0, 0, 0);
+        }
+      }
+#pragma unroll
+      for (int a = 0; a < NH; ++a) {
+        if (item * NH + a < heads) {
+#pragma unroll
+          for (int t = 0; t < NKT; ++t)
+#pragma unroll
+            for (int v = 0; v < 4; ++v) {
+              const int key = 16 * t + 4 * lg + v;
+              S[(hh[a] * BK + key) * QS + li] = acc[a][t][v] * ksc[key];
+            }
+        }
+      }
+    }
+    __syncthreads();
+    // the next tile's rows: every wave is past the previous tile's last use
+    // of the other buffer
+    key_rows(Rows + (buf ^ 1) * BK, Ksc + (buf ^ 1) * BK, k0 + BK, last_pos, BK, bt,
+             block_size, kv_heads, k_scale, mult);
+    // (2) mix over the heads, one key at a time; the wave reads a key's scores
+    // of all heads before it writes any
+    for (int key = wave; key < BK; key += NWV) {
+      f32x4 mx[HT];
+#pragma unroll
+      for (int t = 0; t < HT; ++t) mx[t] = f32x4{0.f, 0.f, 0.f, 0.f};
+      for (int g4 = 0; g4 < H4; g4 += 4) {
+        const float b = S[((g4 + lg) * BK + key) * QS + li];
+#pragma unroll
+        for (int t = 0; t < HT; ++t)
+          mx[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(
+              Tt[(g4 + lg) * 16 * HT + 16 * t + li], b, mx[t], 0, 0, 0);
+      }
+#pragma unroll
+      for (int t = 0; t < HT; ++t)
+#pragma unroll
+        for (int v = 0; v < 4; ++v) {
+          const int h = 16 * t + 4 * lg + v;
+          if (h < heads) S[(h * BK + key) * QS + li] = mx[t][v];
+        }
+    }
+    __syncthreads();
+    // (3) softmax and values of this wave's heads
+    if (item3 < items) {
+      float p[NH][NKT][4];
+#pragma unroll
+      for (int a = 0; a < NH; ++a) {
+        const int h = min(item3 * NH + a, heads - 1);
+        const float* bh = bias + (long)h * bias_n;
+        float mt = -INFINITY;
+#pragma unroll
+        for (int t = 0; t < NKT; ++t)
+#pragma unroll
+          for (int v = 0; v < 4; ++v) {
+            const int key = 16 * t + 4 * lg + v;
+            const int kp = k0 + key;
+            const int n = min(max(qpos - kp, 0), bias_n - 1);
+            const float sc = S[(h * BK + key) * QS + li] + bh[n] * LOG2E;
+            p[a][t][v] = (kp <= qpos && kp >= qstart) ? sc : -INFINITY;
+            mt = fmaxf(mt, p[a][t][v]);
+          }
+        mt = fmaxf(mt, __shfl_xor(mt, 16, WAVE_SIZE));
+        mt = fmaxf(mt, __shfl_xor(mt, 32, WAVE_SIZE));
+        const float mn = fmaxf(m[a], mt);
+        // a column that has seen no visible key yet keeps mn = -inf
+        const float corr = (mn == -INFINITY) ? 1.f : exp2f(m[a] - mn);
+        float ps = 0.f;
+#pragma unroll
+        for (int t = 0; t < NKT; ++t)
+#pragma unroll
+          for (int v = 0; v < 4; ++v) {
+            const float pv = p[a][t][v] == -INFINITY ? 0.f : exp2f(p[a][t][v] - mn);
+            p[a][t][v] = pv;
+            ps += pv;
+          }
+        ps += __shfl_xor(ps, 16, WAVE_SIZE);
+        ps += __shfl_xor(ps, 32, WAVE_SIZE);
+        l[a] = l[a] * corr + ps;
+        m[a] = mn;
+#pragma unroll
+        for (int i = 0; i < DP / 16; ++i) o[a][i] *= corr;
+      }
+#pragma unroll
+      for (int t = 0; t < NKT; ++t)
+#pragma unroll
+        for (int v = 0; v < 4; ++v) {
+          const long vrow = rows[16 * t + 4 * lg + v];
+#pragma unroll
+          for (int j = 0; j < DP / 64; ++j) {
+            // row li of output tile 4 j + c is value column 64 j + 4 li + c
+            const int d0 = 64 * j + 4 * li;
+            f32x4 vv = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (int a = 0; a < NH; ++a) {
+              if (a == 0 || !SHARE) {
+                const int g = min(item3 * NH + a, heads - 1) / rep;
+                if (d0 < D)
+                  vv = load4_f32(k_cache + (vrow + (long)g * block_size) * D + d0,
+                                 vec, D - d0);
+              }
+#pragma unroll
+              for (int c = 0; c < 4; ++c)
+                o[a][4 * j + c] = __builtin_amdgcn_mfma_f32_16x16x4f32(
+                    vv[c], p[a][t][v], o[a][4 * j + c], 0, 0, 0);
+            }
+          }
+        }
+    }
+    // step (1) of the next tile writes other heads' scores than this wave's
+    if (gridDim.z > 1) __syncthreads();
+  }
+
+  if (item3 >= items || li >= nq) return;
+  const long tok = q0 + tok0 + li;
+#pragma unroll
+  for (int a = 0; a < NH; ++a) {
+    const int h = item3 * NH + a;
+    if (h < heads) {
+      // the 1 in the denominator: a key with score 0 and no value
+      const float mn = fmaxf(m[a], 0.f);
+      const float corr = m[a] == -INFINITY ? 0.f : exp2f(m[a] - mn);
+      const float f = corr / (l[a] * corr + exp2f(-mn));
+#pragma unroll
+      for (int j = 0; j < DP / 64; ++j)
+#pragma unroll
+        for (int v = 0; v < 4; ++v) {
+          const int d0 = 64 * j + 4 * (4 * lg + v);
+          if (d0 < D) {
+            const long e = (tok * heads + h) * D + d0;
+            f32x4 gv = f32x4{0.f, 0.f, 0.f, 0.f};
+            if (gate) gv = load4_f32(gate + tok * gate_stride + (long)h * D + d0, false, D - d0);
+#pragma unroll
+            for (int c = 0; c < 4; ++c)
+              if (d0 + c < D) {
+                float r = o[a][4 * j + c][v] * f;
+                if (gate) r *= 1.0f / (1.0f + expf(-gv[c]));
+                st_f32(out, e + c, r);
+              }
+          }
+        }
+    }
+  }
+}
+
+constexpr int DBK = 64;       // keys per decode tile
+constexpr int DS = DBK + 4;   // floats per head row of a decode score tile
+
+// LDS floats of the decode kernel: q [H][DP + 4] | scores [H4][DS] | mixed
+// [H][DS] | talk^T [H4][HP] | max, sum, correction [H] each | factors [2][DBK]
+// | rows [2][DBK]. Value work items: (kv head, 16 query heads, 64 columns).
+template <typename T, int DP, int IPW>
+__global__ void __launch_bounds__(NT) talk_decode_kernel(
+    float* __restrict__ ws, const float* __restrict__ q,
+    const T* __restrict__ k_cache, const float* __restrict__ k_scale,
+    const int* __restrict__ block_tables, int bt_stride,
+    const int* __restrict__ cu_q, const int* __restrict__ ctx_lens,
+    const float* __restrict__ talk, const float* __restrict__ bias, int bias_n,
+    float scale, int heads, int kv_heads, int D, int block_size, int window) {
+  extern __shared__ float lds[];
+  constexpr int QR = DP + 4;
+  const int H4 = (heads + 3) & ~3;
+  const int HP = (heads + 15) & ~15;
+  float* Q = lds;
+  float* S = Q + heads * QR;
+  float* P = S + H4 * DS;
+  float* Tt = P + heads * DS;
+  float* Mx = Tt + H4 * HP;
+  float* Sm = Mx + H4;
+  float* Cr = Sm + H4;
+  float* Ksc = Cr + H4;
+  int* Rows = reinterpret_cast<int*>(Ksc + 2 * DBK);
+
+  const int s = blockIdx.y;
+  const int tok = cu_q[s];
+  if (cu_q[s + 1] - tok < 1) return;
+  const int split = blockIdx.x, nsplit = gridDim.x;
+  const int pos = ctx_lens[s] - 1;
+  const int kbeg = window > 0 ? max(pos - window + 1, 0) : 0;
+  const int lane = threadIdx.x & 63;
+  const int wave = threadIdx.x >> 6;
+  const int li = lane & 15, lg = lane >> 4;
+  const int rep = heads / kv_heads;
+  const int ct = (rep + 15) / 16;  // column tiles of a key group
+  const int nj = (D + 63) / 64;
+  const int* bt = block_tables + (long)s * bt_stride;
+  const bool vec = (D % 8) == 0;
+  const float mult = scale * LOG2E;
+
+  for (int e = threadIdx.x; e < heads * QR; e += NT) {
+    const int h = e / QR, d = e % QR;
+    Q[e] = d < D ? q[((long)tok * heads + h) * D + d] : 0.f;
+  }
+  for (int e = threadIdx.x; e < H4 * HP; e += NT) {
+    const int g = e / HP, h = e % HP;
+    Tt[e] = (g < heads && h < heads) ? talk[h * heads + g] : 0.f;
+  }
+  for (int e = heads * DS + threadIdx.x; e < H4 * DS; e += NT) S[e] = 0.f;
+  for (int e = threadIdx.x; e < heads; e += NT) {
+    Mx[e] = -INFINITY;
+    Sm[e] = 0.f;
+  }
+  const int kfirst = kbeg + split * DBK;
+  const int kstep = nsplit * DBK;
+  key_rows(Rows, Ksc, kfirst, pos, DBK, bt, block_size, kv_heads, k_scale, mult);
+
+  // value items of this wave: kv head, first query head, number of them, columns
+  const int items = kv_heads * ct * nj;
+  f32x4 o[IPW][4];
+#pragma unroll
+  for (int i = 0; i < IPW; ++i)
+#pragma unroll
+    for (int c = 0; c < 4; ++c) o[i][c] = f32x4{0.f, 0.f, 0.f, 0.f};
+  const int item0 = (blockIdx.z * NWV + wave) * IPW;
+  __syncthreads();
+
+  int buf = 0;
+  for (int k0 = kfirst; k0 <= pos; k0 += kstep, buf ^= 1) {
+    const int* rows = Rows + buf * DBK;
+    const float* ksc = Ksc + buf * DBK;
+    // (1) scores: 16 keys x the heads of one key group
+    for (int u = wave; u < kv_heads * ct * 4; u += NWV) {
+      const int kt = u & 3, gc = u >> 2;
+      const int g = gc / ct, c0 = (gc % ct) * 16;
+      const int h = g * rep + min(c0 + li, rep - 1);
+      const long krow = rows[16 * kt + li] + (long)g * block_size;
+      f32x4 acc = f32x4{0.f, 0.f, 0.f, 0.f}, acc2 = acc;
+      Chunk8<T> kf[DP / 32];
+#pragma unroll
+      for (int k8 = 0; k8 < DP / 32; ++k8) {
+        const int d0 = 32 * k8 + 8 * lg;
+        if (d0 < D) kf[k8].load(k_cache + krow * D + d0, vec, D - d0);
+        else kf[k8].zero();
+      }
+#pragma unroll
+      for (int k8 = 0; k8 < DP / 32; ++k8) {
+        const float* qp = Q + h * QR + 32 * k8 + 8 * lg;
+        const f32x4 qa = *reinterpret_cast<const f32x4*>(qp);
+        const f32x4 qb = *reinterpret_cast<const f32x4*>(qp + 4);
+#pragma unroll
+        for (int c = 0; c < 4; ++c) {
+          acc = __builtin_amdgcn_mfma_f32_16x16x4f32(kf[k8].get(c), qa[c], acc, 0, 0, 0);
+          acc2 = __builtin_amdgcn_mfma_f32_16x16x4f32(kf[k8].get(4 + c), qb[c], acc2, 0, 0, 0);
+        }
+      }
+      if (c0 + li < rep) {
+        const f32x4 f = *reinterpret_cast<const f32x4*>(ksc + 16 * kt + 4 * lg);
+        *reinterpret_cast<f32x4*>(S + h * DS + 16 * kt + 4 * lg) = (acc + acc2) * f;
+      }
+    }
+    __syncthreads();
+    key_rows(Rows + (buf ^ 1) * DBK, Ksc + (buf ^ 1) * DBK, k0 + kstep, pos, DBK, bt,
+             block_size, kv_heads, k_scale, mult);
+    // (2) mix over the heads: 16 heads x 16 keys a unit
+    for (int u = wave; u < (HP / 16) * 4; u += NWV) {
+      const int kt = u & 3, ht = u >> 2;
+      f32x4 mx = f32x4{0.f, 0.f, 0.f, 0.f};
+      for (int g4 = 0; g4 < H4; g4 += 4)
+        mx = __builtin_amdgcn_mfma_f32_16x16x4f32(Tt[(g4 + lg) * HP + 16 * ht + li],
+                                                  S[(g4 + lg) * DS + 16 * kt + li],
+                                                  mx, 0, 0, 0);
+#pragma unroll
+      for (int v = 0; v < 4; ++v) {
+        const int h = 16 * ht + 4 * lg + v;
+        if (h < heads) P[h * DS + 16 * kt + li] = mx[v];
+      }
+    }
+    __syncthreads();
+    // (3) softmax, one key per lane
+    for (int h = wave; h < heads; h += NWV) {
+      const int kp = k0 + lane;
+      const int n = min(max(pos - kp, 0), bias_n - 1);
+      const float sc = kp <= pos ? P[h * DS + lane] + bias[(long)h * bias_n + n] * LOG2E
+                                 : -INFINITY;
+      const float m = Mx[h];
+      // the tile's first key is visible, so mn is finite
+      const float mn = fmaxf(m, wave_reduce_max(sc));
+      const float pv = sc == -INFINITY ? 0.f : exp2f(sc - mn);
+      const float ps = wave_reduce_sum(pv);
+      P[h * DS + lane] = pv;
+      if (lane == 0) {
+        const float corr = exp2f(m - mn);
+        Cr[h] = corr;
+        Sm[h] = Sm[h] * corr + ps;
+        Mx[h] = mn;
+      }
+    }
+    __syncthreads();
+    // (4) values
+#pragma unroll
+    for (int i = 0; i < IPW; ++i) {
+      const int item = item0 + i;
+      if (item < items) {
+        const int j = item % nj, gc = item / nj;
+        const int g = gc / ct, c0 = (gc % ct) * 16;
+        const int h = g * rep + min(c0 + li, rep - 1);
+        const int d0 = 64 * j + 4 * li;
+        const float corr = Cr[h];
+#pragma unroll
+        for (int c = 0; c < 4; ++c) o[i][c] *= corr;
+#pragma unroll
+        for (int kt = 0; kt < 4; ++kt) {
+          const f32x4 p = *reinterpret_cast<const f32x4*>(P + h * DS + 16 * kt + 4 * lg);
+          f32x4 vv[4];
+#pragma unroll
+          for (int v = 0; v < 4; ++v) {
+            const long vrow = rows[16 * kt + 4 * lg + v] + (long)g * block_size;
+            vv[v] = f32x4{0.f, 0.f, 0.f, 0.f};
+            if (d0 < D) vv[v] = load4_f32(k_cache + vrow * D + d0, vec, D - d0);
+          }
+#pragma unroll
+          for (int v = 0; v < 4; ++v)
+#pragma unroll
+            for (int c = 0; c < 4; ++c)
+              o[i][c] = __builtin_amdgcn_mfma_f32_16x16x4f32(vv[v][c], p[v], o[i][c], 0, 0, 0);
+        }
+      }
+    }
+  }
+
+  __syncthreads();
+#pragma unroll
+  for (int i = 0; i < IPW; ++i) {
+    const int item = item0 + i;
+    if (item < items) {
+      const int j = item % nj, gc = item / nj;
+      const int g = gc / ct, c0 = (gc % ct) * 16;
+      if (c0 + li < rep) {
+        const int h = g * rep + c0 + li;
+        float* wr = ws + (((long)s * heads + h) * nsplit + split) * (D + 2);
+#pragma unroll
+        for (int v = 0; v < 4; ++v)
+#pragma unroll
+          for (int c = 0; c < 4; ++c) {
+            const int d = 64 * j + 4 * (4 * lg + v) + c;
+            if (d < D) wr[d] = o[i][c][v];
+          }
+      }
+    }
+  }
+  if (blockIdx.z == 0)
+    for (int h = threadIdx.x; h < heads; h += NT) {
+      float* wr = ws + (((long)s * heads + h) * nsplit + split) * (D + 2);
+      wr[D] = Mx[h];
+      wr[D + 1] = Sm[h];
+    }
+}
+
+template <typename T>
+__global__ void talk_merge_kernel(T* __restrict__ out, const float* __restrict__ ws,
+                                  const int* __restrict__ cu_q,
+                                  const T* __restrict__ gate, long gate_stride,
+                                  int heads, int D, int nsplit) {
+  const int s = blockIdx.x / heads, h = blockIdx.x % heads;
+  const long tok = cu_q[s];
+  if (cu_q[s + 1] - tok < 1) return;
+  const float* wr = ws + ((long)s * heads + h) * nsplit * (D + 2);
+  // one more key with score 0 and no value
+  float M = 0.f;
+  for (int i = 0; i < nsplit; ++i) M = fmaxf(M, wr[i * (D + 2) + D]);
+  float L = exp2f(-M);
+  for (int i = 0; i < nsplit; ++i) {
+    const float mi = wr[i * (D + 2) + D];
+    if (mi != -INFINITY) L += wr[i * (D + 2) + D + 1] * exp2f(mi - M);
+  }
+  const float f = 1.0f / L;
+  for (int d = threadIdx.x; d < D; d += blockDim.x) {
+    float O = 0.f;
+    for (int i = 0; i < nsplit; ++i) {
+      const float mi = wr[i * (D + 2) + D];
+      if (mi != -INFINITY) O += wr[i * (D + 2) + d] * exp2f(mi - M);
+    }
+    O *= f;
+    if (gate) {
+      const float gv = ld_f32(gate, tok * gate_stride + (long)h * D + d);
+      O *= 1.0f / (1.0f + expf(-gv));
+    }
+    st_f32(out, (tok * heads + h) * D + d, O);
+  }
+}
+
+struct TalkArgs {
+  void* out;
+  const void *q, *k_cache, *k_scale, *block_tables;
+  int bt_stride;
+  const void *cu_q, *ctx_lens, *talk, *bias;
+  int bias_n;
+  const void* gate;
+  long gate_stride;
+  float scale;
+  int num_seqs, max_q_len, heads, kv_heads, D, block_size, window;
+  void* ws;
+  int nsplit;
+  hipStream_t stream;
+};
+
+constexpr size_t LDS_MAX = 160 * 1024;
+
+template <typename F>
+hipError_t allow_lds(F fn, size_t smem) {
+  if (smem > LDS_MAX) return hipErrorInvalidValue;
+  if (smem <= 48 * 1024) return hipSuccess;
+  return hipFuncSetAttribute((const void*)fn,
+                             hipFuncAttributeMaxDynamicSharedMemorySize, (int)smem);
+}
+
+template <typename T, int DP, int NH, int HT, bool SHARE>
+hipError_t launch_prefill(const TalkArgs& a) {
+  constexpr int BK = HT <= 2 ? 32 : 16;
+  const int H4 = (a.heads + 3) & ~3;
+  const size_t smem =
+      sizeof(float) * ((size_t)H4 * BK * QS + (size_t)H4 * 16 * HT + 4 * BK);
+  auto fn = talk_prefill_kernel<T, DP, NH, HT, SHARE>;
+  hipError_t e = allow_lds(fn, smem);
+  if (e != hipSuccess) return e;
+  dim3 grid(cdiv(a.max_q_len, 16), a.num_seqs, cdiv(cdiv(a.heads, NH), NWV));
+  hipLaunchKernelGGL(fn, grid, dim3(NT), smem, a.stream, (T*)a.out,
+                     (const float*)a.q, (const T*)a.k_cache,
+                     (const float*)a.k_scale, (const int*)a.block_tables,
+                     a.bt_stride, (const int*)a.cu_q, (const int*)a.ctx_lens,
+                     (const float*)a.talk, (const float*)a.bias, a.bias_n,
+                     (const T*)a.gate, a.gate_stride, a.scale, a.heads,
+                     a.kv_heads, a.D, a.block_size, a.window);
+  return hipGetLastError();
+}
+
+// NH heads per wave so that 8 waves cover the heads where that fits the
+// registers; HT: 16-head tiles of the mixing product
+template <typename T, int DP>
+hipError_t dispatch_prefill(const TalkArgs& a) {
+  const int H = a.heads, rep = a.heads / a.kv_heads;
+  if (H <= 8) return launch_prefill<T, DP, 1, 1, true>(a);
+  if constexpr (DP <= 128) {
+    // (fp32 pages: the exact-check dtype, one variant each)
+    constexpr bool fast = sizeof(T) == 2;
+    if (H <= 16)
+      return fast && rep % 2 == 0 ? launch_prefill<T, DP, 2, 1, fast>(a)
+                                  : launch_prefill<T, DP, 2, 1, false>(a);
+    if (H <= 32)
+      return fast && rep % 4 == 0 ? launch_prefill<T, DP, 4, 2, fast>(a)
+                                  : launch_prefill<T, DP, 4, 2, false>(a);
+    return launch_prefill<T, DP, 4, 6, false>(a);
+  } else {
+    if (H <= 16) return launch_prefill<T, DP, 2, 1, false>(a);
+    if (H <= 32) return launch_prefill<T, DP, 2, 2, false>(a);
+    return launch_prefill<T, DP, 2, 6, false>(a);
+  }
+}
+
+template <typename T, int DP, int IPW>
+hipError_t launch_decode(const TalkArgs& a, int items) {
+  const int H4 = (a.heads + 3) & ~3, HP = (a.heads + 15) & ~15;
+  const size_t smem =
+      sizeof(float) * ((size_t)a.heads * (DP + 4) + (size_t)H4 * DS +
+                       (size_t)a.heads * DS + (size_t)H4 * HP + 3 * (size_t)H4 +
+                       4 * DBK);
+  auto fn = talk_decode_kernel<T, DP, IPW>;
+  hipError_t e = allow_lds(fn, smem);
+  if (e != hipSuccess) return e;
+  dim3 grid(a.nsplit, a.num_seqs, cdiv(items, NWV * IPW));
+  hipLaunchKernelGGL(fn, grid, dim3(NT), smem, a.stream, (float*)a.ws,
+                     (const float*)a.q, (const T*)a.k_cache,
+                     (const float*)a.k_scale, (const int*)a.block_tables,
+                     a.bt_stride, (const int*)a.cu_q, (const int*)a.ctx_lens,
+                     (const float*)a.talk, (const float*)a.bias, a.bias_n,
+                     a.scale, a.heads, a.kv_heads, a.D, a.block_size, a.window);
+  e = hipGetLastError();
+  if (e != hipSuccess) return e;
+  hipLaunchKernelGGL(talk_merge_kernel<T>, dim3(a.num_seqs * a.heads), dim3(64),
+                     0, a.stream, (T*)a.out, (const float*)a.ws,
+                     (const int*)a.cu_q, (const T*)a.gate, a.gate_stride,
+                     a.heads, a.D, a.nsplit);
+  return hipGetLastError();
+}
+
+template <typename T, int DP>
+hipError_t dispatch_decode(const TalkArgs& a) {
+  const int ct = cdiv(a.heads / a.kv_heads, 16);
+  const int items = a.kv_heads * ct * cdiv(a.D, 64);
+  if (items <= NWV) return launch_decode<T, DP, 1>(a, items);
+  if (items <= 2 * NWV) return launch_decode<T, DP, 2>(a, items);
+  return launch_decode<T, DP, 4>(a, items);
+}
+
+template <typename T, int DP>
+hipError_t dispatch(const TalkArgs& a) {
+  return a.max_q_len == 1 ? dispatch_decode<T, DP>(a) : dispatch_prefill<T, DP>(a);
+}
+
+template <typename T>
+hipError_t dispatch_d(const TalkArgs& a) {
+  if (a.D <= 64) return dispatch<T, 64>(a);
+  if (a.D <= 128) return dispatch<T, 128>(a);
+  return dispatch<T, 256>(a);
+}
+
+}  // namespace
+
+extern "C" hipError_t ks_talk_prep_cache(
+    void* q_out, const void* q, long q_stride, const void* k, long k_stride,
+    const void* w, const void* slot_mapping, void* k_cache, void* k_scale,
+    float eps, int tokens, int q_width, int kv_heads, int D, int block_size,
+    int is_f32, hipStream_t stream) {
+  if (tokens == 0) return hipSuccess;
+  const int ab = is_f32 ? 16 : 8;
+  auto al = [](const void* p, int bytes) { return ((uintptr_t)p % bytes) == 0; };
+  const int vec = q_width % 4 == 0 && (kv_heads * D) % 4 == 0 &&
+                  q_stride % 4 == 0 && k_stride % 4 == 0 && al(q, ab) &&
+                  al(k, ab) && al(w, 16) && al(q_out, 16);
+#define TP_ARGS(TT)                                                            \
+  (float*)q_out, (const TT*)q, q_stride, (const TT*)k, k_stride,               \
+      (const float*)w, (const int*)slot_mapping, (TT*)k_cache,                 \
+      (float*)k_scale, eps, q_width, kv_heads, D, block_size, vec
+  if (is_f32)
+    hipLaunchKernelGGL(talk_prep_cache_kernel<float>, dim3(tokens), dim3(256), 0,
+                       stream, TP_ARGS(float));
+  else
+    hipLaunchKernelGGL(talk_prep_cache_kernel<short>, dim3(tokens), dim3(256), 0,
+                       stream, TP_ARGS(short));
+  HIP_CHECK_KERNEL();
+  return hipSuccess;
+}
+
+// key splits of a decode launch: enough blocks for two or so on every compute
+// unit, at most 8, with a window no more than it has tiles
+extern "C" int ks_talk_decode_splits(int num_seqs, int window) {
+  int n = cdiv(1024, num_seqs > 0 ? num_seqs : 1);
+  if (n > 8) n = 8;
+  if (window > 0 && n > cdiv(window, DBK)) n = cdiv(window, DBK);
+  return n < 1 ? 1 : n;
+}
+
+extern "C" hipError_t ks_talk_attention(
+    void* out, const void* q, const void* k_cache, const void* k_scale,
+    const void* block_tables, int bt_stride, const void* cu_q,
+    const void* ctx_lens, const void* talk, const void* bias, int bias_n,
+    const void* gate, long gate_stride, float scale, int num_seqs,
+    int max_q_len, int heads, int kv_heads, int D, int block_size, int window,
+    int is_f32, void* ws, int nsplit, hipStream_t stream) {
+  if (num_seqs == 0 || max_q_len == 0) return hipSuccess;
+  if (D < 1 || D > 256 || kv_heads < 1 || heads < 1 || heads % kv_heads != 0 ||
+      heads > 96 || window < 0 || bias_n < 1 ||
+      (max_q_len == 1 && (!ws || nsplit < 1)))
+    return hipErrorInvalidValue;
+  const TalkArgs a{out, q, k_cache, k_scale, block_tables, bt_stride, cu_q,
+                   ctx_lens, talk, bias, bias_n, gate, gate_stride, scale,
+                   num_seqs, max_q_len, heads, kv_heads, D, block_size, window,
+                   ws, nsplit, stream};
+  return is_f32 ? dispatch_d<float>(a) : dispatch_d<short>(a);
+}

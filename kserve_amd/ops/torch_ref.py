@@ -348,10 +348,11 @@ def add_rms_norm_f32res(
 
 
 def gated_group_rms_norm(
-    y, z, weight, eps, groups: int, out_dtype, gate_after: bool = False
+    y, z, weight, eps, groups: int, out_dtype, gate_after: bool = False,
+    gate_sigmoid: bool = False,
 ):
     zf = z.float()
-    gate = zf * torch.sigmoid(zf)
+    gate = torch.sigmoid(zf) if gate_sigmoid else zf * torch.sigmoid(zf)
     v = y if gate_after else y * gate
     vg = v.reshape(v.shape[0], groups, -1)
     vg = vg * torch.rsqrt(vg.pow(2).mean(-1, keepdim=True) + eps)
@@ -363,7 +364,9 @@ def gated_group_rms_norm(
     return out.to(out_dtype)
 
 
-def causal_conv_silu(x_in, w, bias, conv_state, positions, cu_seqlens, slots):
+def causal_conv_silu(
+    x_in, w, bias, conv_state, positions, cu_seqlens, slots, silu: bool = True
+):
     taps = w.shape[1]
     hist = taps - 1
     out = torch.empty(x_in.shape, dtype=torch.float32)
@@ -386,7 +389,7 @@ def causal_conv_silu(x_in, w, bias, conv_state, positions, cu_seqlens, slots):
         )
         for j in range(taps):
             acc = acc + full[j : j + b - a] * w[:, j].unsqueeze(0)
-        out[a:b] = acc * torch.sigmoid(acc)
+        out[a:b] = acc * torch.sigmoid(acc) if silu else acc
         if hist:
             conv_state[slot, :hist] = full[full.shape[0] - hist :].to(
                 conv_state.dtype
@@ -450,9 +453,10 @@ def qk_norm_temp_cache(
 def ctx_attention_f32(
     q, k_cache, v_cache, block_tables, cu_q, ctx_lens, scale: float,
     heads: int, gate=None, out_dtype=torch.float32, sink=None, chunk: int = 0,
-    out_inv_freq=None, window: int = 0,
+    out_inv_freq=None, window: int = 0, maps: int = 1, softcap: float = 0.0,
 ):
     _, G, bs, D = k_cache.shape
+    D //= maps
     DV = v_cache.shape[3]
     T = q.shape[0]
     out = torch.zeros(T, heads, DV, dtype=torch.float32)
@@ -464,12 +468,16 @@ def ctx_attention_f32(
             continue
         nb = -(-ctx // bs)
         blocks = block_tables[s, :nb].long()
-        K = k_cache[blocks].float().permute(1, 0, 2, 3).reshape(G, nb * bs, D)[:, :ctx]
+        K = k_cache[blocks].float().permute(1, 0, 2, 3).reshape(G, nb * bs, maps * D)
         V = v_cache[blocks].float().permute(1, 0, 2, 3).reshape(G, nb * bs, DV)[:, :ctx]
-        K = K.repeat_interleave(rep, dim=0)
+        # query head h reads map h % maps of its group's key rows
+        K = K[:, :ctx].reshape(G, ctx, maps, D).transpose(1, 2)
+        K = K.repeat_interleave(rep // maps, dim=0).reshape(heads, ctx, D)
         V = V.repeat_interleave(rep, dim=0)
         qs = q[a:b].reshape(b - a, heads, D).float().transpose(0, 1)
         sc = torch.matmul(qs, K.transpose(1, 2)) * scale  # [heads, n, ctx]
+        if softcap > 0:
+            sc = softcap * torch.tanh(sc / softcap)
         qpos = torch.arange(ctx - (b - a), ctx).unsqueeze(1)
         kpos = torch.arange(ctx).unsqueeze(0)
         vis = kpos <= qpos
@@ -518,17 +526,22 @@ def rotate_halves(x, positions, inv_freq, sign: float = 1.0):
 def qk_headnorm_rope_cache(
     q, k, v, qw, kw, positions, slot_mapping, k_cache, v_cache, eps,
     heads: int, qk_inv_freq, v_unit_norm: bool, v_inv_freq,
+    pairs: bool = False, rot_mult: float = 1.0, maps: int = 1,
 ):
     """Per-head RMS norm of q and k (weights [dim], shared by the heads),
-    rotary positions on their first 2*len(qk_inv_freq) coordinates; values
+    rotary positions on their first 2*len(qk_inv_freq) coordinates (``pairs``:
+    2i with 2i+1 instead of i with i + half; the turned coordinates times
+    ``rot_mult``). ``maps`` heads of k share one cached row (and one value
+    head). Values
     optionally divided by their per-head RMS and rotated by their position
     over 2*len(v_inv_freq) coordinates; k / v scattered to the pages; q
     returned in fp32."""
     _, G, bs, D = k_cache.shape
+    D //= maps
     DV = v_cache.shape[3]
     T = q.shape[0]
     qf = q.float().reshape(T, heads, D)
-    kf = k.float().reshape(T, G, D)
+    kf = k.float().reshape(T, G * maps, D)
     vf = v.float().reshape(T, G, DV)
     qn = qf * torch.rsqrt(qf.pow(2).mean(-1, keepdim=True) + eps)
     kn = kf * torch.rsqrt(kf.pow(2).mean(-1, keepdim=True) + eps)
@@ -537,8 +550,13 @@ def qk_headnorm_rope_cache(
     if kw is not None:
         kn = kn * kw
     if qk_inv_freq is not None:
-        qn = rotate_halves(qn, positions, qk_inv_freq)
-        kn = rotate_halves(kn, positions, qk_inv_freq)
+        n = 2 * qk_inv_freq.numel()
+        rotate = rotate_pairs if pairs else rotate_halves
+        qn = rotate(qn, positions, qk_inv_freq)
+        kn = rotate(kn, positions, qk_inv_freq)
+        if rot_mult != 1.0:
+            qn = torch.cat([qn[..., :n] * rot_mult, qn[..., n:]], dim=-1)
+            kn = torch.cat([kn[..., :n] * rot_mult, kn[..., n:]], dim=-1)
     if v_unit_norm:
         vf = vf * torch.rsqrt(vf.pow(2).mean(-1, keepdim=True) + eps)
     if v_inv_freq is not None:
@@ -546,7 +564,7 @@ def qk_headnorm_rope_cache(
     slots = slot_mapping.long()
     ok = slots >= 0
     blk, off = slots[ok] // bs, slots[ok] % bs
-    k_cache[blk, :, off] = kn[ok].to(k_cache.dtype)
+    k_cache[blk, :, off] = kn[ok].reshape(-1, G, maps * D).to(k_cache.dtype)
     v_cache[blk, :, off] = vf[ok].to(v_cache.dtype)
     return qn.reshape(T, heads * D)
 
@@ -785,7 +803,7 @@ def unit_norm_heads(x, heads_a, scale_a, heads_b, scale_b, dim, eps):
 
 def linear_scan(
     q, k, v, state, positions, cu_seqlens, slots, qk_heads, decay=None,
-    a_raw=None, b_raw=None, a_log=None, dt_bias=None,
+    a_raw=None, b_raw=None, a_log=None, dt_bias=None, channel_decay=None,
 ):
     """Token-by-token form of the decay / gated-delta recurrences; state
     [slots, heads, V, K] fp32 is read (unless the portion starts at position
@@ -796,9 +814,12 @@ def linear_scan(
     o = torch.empty(T, heads * V, dtype=torch.float32)
     cu = cu_seqlens.tolist()
     if decay is None:
-        sp = a_raw.float() + dt_bias
-        sp = torch.where(sp > 30.0, sp, torch.log1p(torch.exp(sp)))
-        g_all = torch.exp(-torch.exp(a_log) * sp)          # [T, heads]
+        if channel_decay is not None:
+            g_all = channel_decay.reshape(T, heads, 1, K)
+        else:
+            sp = a_raw.float() + dt_bias
+            sp = torch.where(sp > 30.0, sp, torch.log1p(torch.exp(sp)))
+            g_all = torch.exp(-torch.exp(a_log) * sp).reshape(T, heads, 1, 1)
         b_all = torch.sigmoid(b_raw.float())
     for s, slot in enumerate(slots.tolist()):
         a, b = cu[s], cu[s + 1]
@@ -814,7 +835,7 @@ def linear_scan(
             if decay is not None:
                 S = decay[:, None, None] * S + vt[:, :, None] * kt[:, None, :]
             else:
-                S = g_all[t][:, None, None] * S
+                S = g_all[t] * S
                 u = b_all[t][:, None] * (vt - (S * kt[:, None, :]).sum(-1))
                 S = S + u[:, :, None] * kt[:, None, :]
             o[t] = (S * qt[:, None, :]).sum(-1).reshape(-1)
@@ -833,3 +854,163 @@ def relu2_scale(x, scales=None):
 def scale_softcap(x, scale: float, cap: float):
     z = x.float() * scale
     return cap * torch.tanh(z / cap) if cap > 0 else z
+
+
+# -- two score maps, mixed score heads, per-channel decays, grouped norms -----
+
+def yarn_inv_freq(n_rot: int, base: float, scaling=None):
+    """Rotation frequencies base^(-2i/n_rot) and the factor on cos and sin.
+    ``scaling`` (YaRN: factor, original, fast, slow): pairs that turn more
+    than ``fast`` times over ``original`` positions keep their frequency,
+    those that turn less than ``slow`` times get it divided by ``factor``,
+    with a linear ramp over the pair index in between. float64, rounded once."""
+    import math
+
+    i = torch.arange(n_rot // 2, dtype=torch.float64)
+    f = float(base) ** (-2.0 * i / n_rot)
+    if not scaling:
+        return f.to(torch.float32), 1.0
+
+    def pair_of(turns):
+        return (
+            n_rot * math.log(scaling["original"] / (2.0 * math.pi * turns))
+            / (2.0 * math.log(base))
+        )
+
+    lo = max(math.floor(pair_of(scaling["fast"])), 0)
+    hi = min(math.ceil(pair_of(scaling["slow"])), n_rot - 1)
+    ramp = ((i - lo) / max(hi - lo, 0.001)).clamp(0.0, 1.0)
+    f = f / scaling["factor"] * ramp + f * (1.0 - ramp)
+    return f.to(torch.float32), 0.1 * math.log(scaling["factor"]) + 1.0
+
+
+def distance_buckets(count: int, buckets: int, bias_max: float) -> torch.Tensor:
+    """Bucket of every distance 0..count-1: the first half of the buckets one
+    distance each, the rest spaced logarithmically up to ``bias_max``, the
+    last one for everything beyond."""
+    import math
+
+    half = buckets // 2
+    out = []
+    for n in range(count):
+        if n < half:
+            out.append(n)
+        elif n >= bias_max or half == 0:
+            out.append(buckets - 1)
+        else:
+            up = math.log(n / half) / math.log(bias_max / half) * (buckets - half)
+            out.append(min(buckets - 1, half + math.floor(up)))
+    return torch.tensor(out, dtype=torch.int64)
+
+
+def post_group_norm_add(
+    residual, delta, weight, groups: int, eps: float, out_dtype, delta2=None,
+    pre_w=None, pre_w2=None, next_weight=None, want_out: bool = True,
+):
+    """residual (fp32, in place) += GroupRMS(d) * weight, d = ``delta`` or,
+    with ``delta2``, (rms(delta) * pre_w + rms(delta2) * pre_w2) / 2. Returns
+    the new residual in ``out_dtype`` or, with ``next_weight``, its group RMS
+    norm times that weight. GroupRMS: every one of ``groups`` equal parts is
+    divided by its own sqrt(mean(part^2) + eps)."""
+    def grms(x):
+        p = x.reshape(x.shape[0], groups, -1)
+        return (p * torch.rsqrt(p.pow(2).mean(-1, keepdim=True) + eps)).reshape(x.shape)
+
+    def rms(x):
+        return x * torch.rsqrt(x.pow(2).mean(-1, keepdim=True) + eps)
+
+    if delta is not None:
+        d = delta.float()
+        if delta2 is not None:
+            d = 0.5 * (rms(d) * pre_w + rms(delta2.float()) * pre_w2)
+        residual += grms(d) * weight
+    if not want_out:
+        return None
+    if next_weight is None:
+        return residual.to(out_dtype)
+    return (grms(residual) * next_weight).to(out_dtype)
+
+
+def diff_combine(o, lam, heads: int, eps: float, mult: float, out_dtype):
+    """o [T, heads*2*V] fp32 (first and second map of every head side by
+    side) -> (a1 - lam a2) / rms over V, times ``mult``."""
+    T = o.shape[0]
+    a = o.reshape(T, heads, 2, -1)
+    d = a[:, :, 0] - lam * a[:, :, 1]
+    d = d * torch.rsqrt(d.pow(2).mean(-1, keepdim=True) + eps) * mult
+    return d.reshape(T, -1).to(out_dtype)
+
+
+def talk_prep_cache(
+    q, k, w, slot_mapping, k_cache, k_scale, eps: float,
+):
+    """q RMS-normed over the whole row, times ``w``; fp32. The un-normed keys
+    go to the pages and 1 / rms of the whole key row to ``k_scale``."""
+    _, G, bs, D = k_cache.shape
+    T = q.shape[0]
+    qf, kf = q.float(), k.float()
+    qn = qf * torch.rsqrt(qf.pow(2).mean(-1, keepdim=True) + eps) * w
+    slots = slot_mapping.long()[:T]
+    ok = slots >= 0
+    blk, off = slots[ok] // bs, slots[ok] % bs
+    k_cache[blk, :, off] = k[ok].reshape(-1, G, D).to(k_cache.dtype)
+    k_scale[blk, off] = torch.rsqrt(kf.pow(2).mean(-1) + eps)[ok]
+    return qn
+
+
+def talk_attention(
+    q, k_cache, k_scale, block_tables, cu_q, ctx_lens, scale: float,
+    heads: int, talk, bias, window: int, gate, out_dtype,
+):
+    """Paged causal attention with the heads' scores mixed before the softmax:
+    s_h = sum_g talk[h, g] * (q_g . k) * k_scale * scale + bias[h, distance]
+    (``bias`` [heads, n]: the mixed bias per distance, constant past n - 1),
+    one added to the softmax denominator, values = the cached keys, output
+    times sigmoid(gate) per element."""
+    _, G, bs, D = k_cache.shape
+    T = q.shape[0]
+    out = torch.zeros(T, heads, D, dtype=torch.float32)
+    cu = cu_q.tolist()
+    rep = heads // G
+    for s, ctx in enumerate(ctx_lens.tolist()):
+        a, b = cu[s], cu[s + 1]
+        if b <= a:
+            continue
+        nb = -(-ctx // bs)
+        blocks = block_tables[s, :nb].long()
+        K = k_cache[blocks].float().permute(1, 0, 2, 3).reshape(G, nb * bs, D)[:, :ctx]
+        ks = k_scale[blocks].reshape(nb * bs)[:ctx]
+        K = K.repeat_interleave(rep, dim=0)
+        qs = q[a:b].reshape(b - a, heads, D).float().transpose(0, 1)
+        sc = torch.matmul(qs, K.transpose(1, 2)) * (ks * scale)
+        sc = torch.matmul(talk, sc.reshape(heads, -1)).reshape(sc.shape)
+        qpos = torch.arange(ctx - (b - a), ctx).unsqueeze(1)
+        kpos = torch.arange(ctx).unsqueeze(0)
+        dist = (qpos - kpos).clamp(0, bias.shape[1] - 1)
+        sc = sc + bias[:, dist]
+        vis = kpos <= qpos
+        if window > 0:
+            vis = vis & (qpos - kpos < window)
+        sc = sc.masked_fill(~vis.unsqueeze(0), float("-inf"))
+        m = sc.max(-1, keepdim=True).values.clamp(min=0.0)
+        e = torch.exp(sc - m)
+        w = e / (e.sum(-1, keepdim=True) + torch.exp(-m))
+        out[a:b] = torch.matmul(w, K).transpose(0, 1)
+    out = out.reshape(T, heads * D)
+    if gate is not None:
+        out = out * torch.sigmoid(gate.float())
+    return out.to(out_dtype)
+
+
+def delta_unit_decay(
+    qkv, qk_heads: int, dim: int, q_scale: float, eps: float, a_raw, a_log,
+    dt_bias,
+):
+    """In place on fp32 rows [q | k | v]: the q and k heads become unit
+    vectors, q times ``q_scale``. Returns the decay of every head and key
+    channel, exp(-exp(a_log[h]) softplus(a_raw + dt_bias)), fp32 [T, H*dim]."""
+    unit_norm_heads(qkv, qk_heads, q_scale, qk_heads, 1.0, dim, eps)
+    z = a_raw.float() + dt_bias
+    z = torch.where(z > 30.0, z, torch.log1p(torch.exp(z)))
+    A = torch.exp(a_log).repeat_interleave(a_raw.shape[1] // a_log.numel())
+    return torch.exp(-A * z)
