@@ -230,6 +230,55 @@ def _laperax_model_configs(size: dict):
     return laperax, merulorn
 
 
+# layer shapes for --mededra-compare: the widths, head counts, windows and
+# delta sizes of LAPERAX_SIZES; differential heads of two 64-column maps over
+# 128-column values; a dense feed-forward with the arithmetic of the experts
+# one token uses there (three matrices instead of two per expert)
+MEDEDRA_SIZES = {
+    "2k": dict(laperax="2k", ff=5504),
+    "4k": dict(laperax="4k", ff=9600),
+}
+
+
+def _mededra_model_configs(size: dict):
+    """A four-layer Mededra model (differential, parallel, differential,
+    parallel) and the Laperax model that --laperax-compare measures at the
+    same width."""
+    from kserve_amd.engine.config import (
+        DeltaMixerSpec,
+        DifferentialMixerSpec,
+        HybridLayerSpec,
+        HybridModelConfig,
+        SiluGLUSpec,
+        TalkingMixerSpec,
+    )
+
+    base = LAPERAX_SIZES[size["laperax"]]
+    H, G, D = base["heads"], base["kv_heads"], base["head_dim"]
+    mlp = SiluGLUSpec(ff=size["ff"])
+    diff = DifferentialMixerSpec(
+        heads=H, kv_heads=G, dim=D // 2, vdim=D, scale=(D // 2) ** -0.5,
+        diff=0.3, conv=4, softcap=30.0, window=base["window"], rot_dims=D // 2,
+        rot_base=250000.0,
+        rot_scaling={"factor": 4.0, "original": 2048, "fast": 32.0, "slow": 1.0},
+    )
+    talk = TalkingMixerSpec(heads=H, kv_heads=G, dim=D, scale=D ** -0.5,
+                            bias_max=base["window"] - 16, window=base["window"])
+    delta = DeltaMixerSpec(heads=H, kv_heads=H // 2, dim=D, vdim=D, conv=4,
+                           channel_decay=True)
+    layers = [
+        HybridLayerSpec("attention", differential=diff, mlp=mlp),
+        HybridLayerSpec("parallel", talking=talk, delta=delta, mlp=mlp),
+    ] * 2
+    mededra = HybridModelConfig(
+        vocab_size=base["vocab"], hidden_size=base["width"], layers=layers,
+        model_name="mededra-bench", architecture="Mededra", norm_groups=4,
+        embedding_scale=12.0, logit_softcap=30.0,
+    )
+    laperax, _ = _laperax_model_configs(base)
+    return mededra, laperax
+
+
 def _throughput(mcfg, prompt_len, n_prompts, concurrency, steps, warmup, eager):
     """(prefill tok/s, decode tok/s) through the engine's own step()."""
     import torch
@@ -479,6 +528,56 @@ def laperax_compare(args):
     return 0
 
 
+def mededra_compare(args):
+    """Prefill and decode tok/s of the Mededra design next to the Laperax
+    model of equal width and depth (the closest design the engine serves: a
+    delta rule behind short convolutions beside windowed attention), both
+    through LLMEngine.step() on one GPU, bf16, random weights. One JSON line
+    per (size, model), each measured in a process of its own."""
+    import subprocess
+    import sys
+
+    if args.compare_only is None or "," in args.mededra_compare:
+        rc = 0
+        for name in args.mededra_compare.split(","):
+            for label in ("mededra", "laperax"):
+                if args.compare_only and args.compare_only != label:
+                    continue
+                cmd = [sys.executable, "-u", os.path.abspath(__file__),
+                       "--mededra-compare", name, "--compare-only", label,
+                       "--steps", str(args.steps), "--warmup", str(args.warmup),
+                       "--concurrency", str(args.concurrency),
+                       "--prompt-len", str(args.prompt_len)]
+                if args.eager:
+                    cmd.append("--eager")
+                rc = subprocess.call(cmd)
+                if rc != 0:
+                    return rc
+        return rc
+
+    import torch
+
+    assert torch.cuda.is_available(), "--mededra-compare needs a GPU"
+    name, label = args.mededra_compare, args.compare_only
+    mededra, laperax = _mededra_model_configs(MEDEDRA_SIZES[name])
+    mcfg = mededra if label == "mededra" else laperax
+    prefill, decode = _throughput(
+        mcfg, prompt_len=args.prompt_len if args.prompt_len != 512 else 2048,
+        n_prompts=8, concurrency=min(args.concurrency, 256),
+        steps=args.steps, warmup=args.warmup, eager=args.eager,
+    )
+    print(json.dumps({
+        "bench": "mededra-compare", "size": name, "model": mcfg.model_name,
+        "layers": 4, "width": mcfg.hidden_size,
+        "prefill_tok_s": round(prefill, 1),
+        "decode_tok_s": round(decode, 1),
+        "prefill_batch": "8 x prompt", "decode_concurrency":
+            min(args.concurrency, 256),
+        "dtype": "bfloat16", "data": "synthetic, random-init weights",
+    }), flush=True)
+    return 0
+
+
 def main():
     parser = argparse.ArgumentParser()
     parser.add_argument("--gpus", type=int, default=1)
@@ -537,12 +636,18 @@ def main():
                              "decode throughput of a Laperax-design model "
                              "beside the Merulorn model of equal width and "
                              "depth (sizes: " + ", ".join(LAPERAX_SIZES) + ")")
+    parser.add_argument("--mededra-compare", type=str, default=None,
+                        metavar="SIZE[,SIZE...]",
+                        help="instead of the flagship workload: prefill and "
+                             "decode throughput of a Mededra-design model "
+                             "beside the Laperax model of equal width and "
+                             "depth (sizes: " + ", ".join(MEDEDRA_SIZES) + ")")
     parser.add_argument("--compare-only", type=str, default=None,
                         choices=["desalix", "llama", "voborax", "laperax",
-                                 "merulorn"],
+                                 "merulorn", "mededra"],
                         help="with --desalix-compare / --voborax-compare / "
-                             "--laperax-compare: run one side only (e.g. "
-                             "under a profiler)")
+                             "--laperax-compare / --mededra-compare: run one "
+                             "side only (e.g. under a profiler)")
     parser.add_argument("--profile-cpu", action="store_true",
                         help="cProfile the timed loop and print hot functions")
     args = parser.parse_args()
@@ -554,6 +659,8 @@ def main():
         return voborax_compare(args)
     if args.laperax_compare:
         return laperax_compare(args)
+    if args.mededra_compare:
+        return mededra_compare(args)
 
     import torch
 

@@ -57,8 +57,10 @@ class LayerCache(NamedTuple):
     #                                         per cached key row
 
 
-def _param(*shape, dtype):
-    return nn.Parameter(torch.empty(*shape, dtype=dtype), requires_grad=False)
+def _param(*shape, dtype, device=None):
+    return nn.Parameter(
+        torch.empty(*shape, dtype=dtype, device=device), requires_grad=False
+    )
 
 
 class SSDMixer(nn.Module):
@@ -1102,7 +1104,9 @@ class TalkingHeadsAttention(nn.Module):
         dt = self.dtype
         rel = get(prefix + "rel").float()
         if rel.shape != self.rel.shape:
-            self.rel = _param(*rel.shape, dtype=torch.float32).to(self.qkg.device)
+            self.rel = _param(
+                *rel.shape, dtype=torch.float32, device=self.rel.device
+            )
         self.rel.copy_(rel)
         self.qkg.copy_(
             torch.cat([get(prefix + n).to(dt) for n in ("q", "k", "g")], dim=0)
@@ -1180,13 +1184,13 @@ class ChannelDeltaMixer(nn.Module):
         # rows padded to whole 16-byte units so that every token's row of the
         # projection starts aligned
         self.proj_width = -(-(self.b_at + s.heads) // 8) * 8
-        self.proj = _param(self.proj_width, self.width, dtype=self.dtype)
-        self.low2 = _param(
-            self.decay_w + self.v_w, a_rank + g_rank, dtype=self.dtype
+        self.proj = _param(
+            self.proj_width, self.width, dtype=self.dtype, device=device
         )
-        if device is not None:
-            self.proj.data = self.proj.data.to(device)
-            self.low2.data = self.low2.data.to(device)
+        self.low2 = _param(
+            self.decay_w + self.v_w, a_rank + g_rank, dtype=self.dtype,
+            device=device,
+        )
 
     def state_shapes(self):
         s = self.spec

@@ -24,6 +24,7 @@
 //    running softmax and multiplies with the keys as values, whose weights
 //    never leave the registers. A wave works on NH heads at once; SHARE: they
 //    belong to one key group, so every key fragment is loaded once for all.
+//    Loads run ahead of the products that use them.
 //    More heads than 8 NH: further blocks (grid z) take the next ones and
 //    recompute the scores of all heads.
 //  * talk_attention decode (one token per sequence): a block takes one split
@@ -86,6 +87,41 @@ __global__ void __launch_bounds__(256) talk_prep_cache_kernel(
   }
 }
 
+// loads of the first (contraction) and second (values) product; FULL: heads of
+// exactly the padded width in aligned rows, no guards around the loads
+template <bool FULL, typename T>
+__device__ __forceinline__ void load_chunk(Chunk8<T>& c, const T* p, bool vec,
+                                           int valid) {
+  if constexpr (FULL) {
+    c.load(p, true, 8);
+  } else {
+    if (valid > 0) c.load(p, vec, valid);
+    else c.zero();
+  }
+}
+// four values kept in the cache dtype until they are used
+template <typename T>
+struct Quad;
+template <>
+struct Quad<short> {
+  short4_t x;
+  __device__ __forceinline__ float get(int i) const { return bf16_bits_to_float(x[i]); }
+};
+template <>
+struct Quad<float> {
+  f32x4 x;
+  __device__ __forceinline__ float get(int i) const { return x[i]; }
+};
+template <bool FULL, typename T>
+__device__ __forceinline__ void load_quad(Quad<T>& q, const T* p, bool vec, int valid) {
+  if (FULL || (vec && valid >= 4)) {
+    q.x = *reinterpret_cast<const decltype(q.x)*>(p);
+  } else {
+#pragma unroll
+    for (int i = 0; i < 4; ++i) q.x[i] = i < valid ? p[i] : (T)0;
+  }
+}
+
 // cache row (of kv head 0) and score factor of `count` keys from k0 on; keys
 // past `last` repeat the last one (masked later)
 __device__ __forceinline__ void key_rows(int* rows, float* ksc, int k0, int last,
@@ -100,9 +136,15 @@ __device__ __forceinline__ void key_rows(int* rows, float* ksc, int k0, int last
   }
 }
 
+// 16-key tiles per step of the prefill kernel: two where the registers (heads
+// of a wave times the head size) and the LDS (heads) allow
+constexpr int key_tiles(int DP, int NH, int HT) {
+  return HT <= 2 && DP * NH < 512 ? 2 : 1;
+}
+
 // LDS floats of the prefill kernel: scores [H4][16 NKT][QS] | talk^T [H4][16 HT]
 // | rows [2][16 NKT] | factors [2][16 NKT]
-template <typename T, int DP, int NH, int HT, bool SHARE>
+template <typename T, int DP, int NH, int HT, bool SHARE, bool FULL>
 __global__ void __launch_bounds__(NT) talk_prefill_kernel(
     T* __restrict__ out, const float* __restrict__ q,
     const T* __restrict__ k_cache, const float* __restrict__ k_scale,
@@ -111,7 +153,7 @@ __global__ void __launch_bounds__(NT) talk_prefill_kernel(
     const float* __restrict__ talk, const float* __restrict__ bias, int bias_n,
     const T* __restrict__ gate, long gate_stride, float scale, int heads,
     int kv_heads, int D, int block_size, int window) {
-  constexpr int NKT = HT <= 2 ? 2 : 1;
+  constexpr int NKT = key_tiles(DP, NH, HT);
   constexpr int BK = 16 * NKT;
   extern __shared__ float lds[];
   const int H4 = (heads + 3) & ~3;
@@ -179,34 +221,45 @@ __global__ void __launch_bounds__(NT) talk_prefill_kernel(
       long krow[NKT];
 #pragma unroll
       for (int t = 0; t < NKT; ++t) krow[t] = rows[16 * t + li];
-#pragma unroll
-      for (int k8 = 0; k8 < DP / 32; ++k8) {
-        // contraction step c of lane group lg stands for d = 32 k8 + 8 lg + c
+      // Steps (k8, head) in order, the query fragment two steps ahead and the
+      // key fragments one k8 ahead of their products. Contraction step c of
+      // lane group lg stands for d = 32 k8 + 8 lg + c.
+      constexpr int K8 = DP / 32, STEPS = K8 * NH, KB = SHARE ? 1 : NH;
+      constexpr int KR = SHARE ? 2 : 1;  // key fragments in flight
+      Chunk8<T> kf[KR][KB][NKT];
+      Chunk8<float> qf[3];
+      auto load_k = [&](int k8) {
         const int d0 = 32 * k8 + 8 * lg;
-        Chunk8<T> kf[NKT];
 #pragma unroll
-        for (int a = 0; a < NH; ++a) {
-          if (a == 0 || !SHARE) {
-            const int g = hh[a] / rep;
+        for (int a = 0; a < KB; ++a) {
+          const int g = hh[a] / rep;
 #pragma unroll
-            for (int t = 0; t < NKT; ++t) {
-              if (d0 < D)
-                kf[t].load(k_cache + (krow[t] + (long)g * block_size) * D + d0, vec,
-                           D - d0);
-              else
-                kf[t].zero();
-            }
-          }
-          Chunk8<float> qf;
-          if (d0 < D) qf.load(qrow + hh[a] * D + d0, vec, D - d0);
-          else qf.zero();
-#pragma unroll
-          for (int c = 0; c < 8; ++c)
-#pragma unroll
-            for (int t = 0; t < NKT; ++t)
-              acc[a][t] = __builtin_amdgcn_mfma_f32_16x16x4f32(
-                  kf[t].get(c), qf.get(c), acc[a][t], 0, 0, 0);
+          for (int t = 0; t < NKT; ++t)
+            load_chunk<FULL>(kf[k8 % KR][a][t],
+                             k_cache + (krow[t] + (long)g * block_size) * D + d0, vec,
+                             D - d0);
         }
+      };
+      auto load_q = [&](int step) {
+        const int d0 = 32 * (step / NH) + 8 * lg;
+        load_chunk<FULL>(qf[step % 3], qrow + hh[step % NH] * D + d0, vec, D - d0);
+      };
+      load_k(0);
+      load_q(0);
+      if (STEPS > 1) load_q(1);
+#pragma unroll
+      for (int st = 0; st < STEPS; ++st) {
+        const int a = st % NH, k8 = st / NH;
+        if (a == 0 && KR == 2 && k8 + 1 < K8) load_k(k8 + 1);
+        if (a == 0 && KR == 1 && k8 > 0) load_k(k8);
+        if (st + 2 < STEPS) load_q(st + 2);
+#pragma unroll
+        for (int c = 0; c < 8; ++c)
+#pragma unroll
+          for (int t = 0; t < NKT; ++t)
+            acc[a][t] = __builtin_amdgcn_mfma_f32_16x16x4f32(
+                kf[k8 % KR][SHARE ? 0 : a][t].get(c), qf[st % 3].get(c), acc[a][t], 0,
+                0, 0);
       }
 #pragma unroll
       for (int a = 0; a < NH; ++a) {
@@ -250,6 +303,20 @@ __global__ void __launch_bounds__(NT) talk_prefill_kernel(
     __syncthreads();
     // (3) softmax and values of this wave's heads
     if (item3 < items) {
+      // values of 16 keys at a time, the next ones in flight
+      constexpr int VJ = DP / 64;
+      auto load_v = [&](Quad<T>(&dst)[VJ], int t, int v, int a) {
+        const int g = min(item3 * NH + a, heads - 1) / rep;
+        const T* row = k_cache + (rows[16 * t + 4 * lg + v] + (long)g * block_size) * D;
+#pragma unroll
+        for (int j = 0; j < VJ; ++j)
+          load_quad<FULL>(dst[j], row + 64 * j + 4 * li, vec, D - (64 * j + 4 * li));
+      };
+      Quad<T> vs[4][VJ];
+      if (SHARE) {
+#pragma unroll
+        for (int v = 0; v < 4; ++v) load_v(vs[v], 0, v, 0);
+      }
       float p[NH][NKT][4];
 #pragma unroll
       for (int a = 0; a < NH; ++a) {
@@ -289,30 +356,25 @@ __global__ void __launch_bounds__(NT) talk_prefill_kernel(
         for (int i = 0; i < DP / 16; ++i) o[a][i] *= corr;
       }
 #pragma unroll
-      for (int t = 0; t < NKT; ++t)
+      for (int t = 0; t < NKT; ++t) {
+        if (SHARE && t > 0) {
 #pragma unroll
-        for (int v = 0; v < 4; ++v) {
-          const long vrow = rows[16 * t + 4 * lg + v];
+          for (int v = 0; v < 4; ++v) load_v(vs[v], t, v, 0);
+        }
+        // row li of output tile 4 j + c is value column 64 j + 4 li + c
 #pragma unroll
-          for (int j = 0; j < DP / 64; ++j) {
-            // row li of output tile 4 j + c is value column 64 j + 4 li + c
-            const int d0 = 64 * j + 4 * li;
-            f32x4 vv = f32x4{0.f, 0.f, 0.f, 0.f};
+        for (int v = 0; v < 4; ++v)
 #pragma unroll
-            for (int a = 0; a < NH; ++a) {
-              if (a == 0 || !SHARE) {
-                const int g = min(item3 * NH + a, heads - 1) / rep;
-                if (d0 < D)
-                  vv = load4_f32(k_cache + (vrow + (long)g * block_size) * D + d0,
-                                 vec, D - d0);
-              }
+          for (int a = 0; a < NH; ++a) {
+            if (!SHARE) load_v(vs[0], t, v, a);
+#pragma unroll
+            for (int j = 0; j < VJ; ++j)
 #pragma unroll
               for (int c = 0; c < 4; ++c)
                 o[a][4 * j + c] = __builtin_amdgcn_mfma_f32_16x16x4f32(
-                    vv[c], p[a][t][v], o[a][4 * j + c], 0, 0, 0);
-            }
+                    vs[SHARE ? v : 0][j].get(c), p[a][t][v], o[a][4 * j + c], 0, 0, 0);
           }
-        }
+      }
     }
     // step (1) of the next tile writes other heads' scores than this wave's
     if (gridDim.z > 1) __syncthreads();
@@ -356,7 +418,7 @@ constexpr int DS = DBK + 4;   // floats per head row of a decode score tile
 // LDS floats of the decode kernel: q [H][DP + 4] | scores [H4][DS] | mixed
 // [H][DS] | talk^T [H4][HP] | max, sum, correction [H] each | factors [2][DBK]
 // | rows [2][DBK]. Value work items: (kv head, 16 query heads, 64 columns).
-template <typename T, int DP, int IPW>
+template <typename T, int DP, int IPW, bool FULL>
 __global__ void __launch_bounds__(NT) talk_decode_kernel(
     float* __restrict__ ws, const float* __restrict__ q,
     const T* __restrict__ k_cache, const float* __restrict__ k_scale,
@@ -436,8 +498,7 @@ __global__ void __launch_bounds__(NT) talk_decode_kernel(
 #pragma unroll
       for (int k8 = 0; k8 < DP / 32; ++k8) {
         const int d0 = 32 * k8 + 8 * lg;
-        if (d0 < D) kf[k8].load(k_cache + krow * D + d0, vec, D - d0);
-        else kf[k8].zero();
+        load_chunk<FULL>(kf[k8], k_cache + krow * D + d0, vec, D - d0);
       }
 #pragma unroll
       for (int k8 = 0; k8 < DP / 32; ++k8) {
@@ -508,18 +569,17 @@ __global__ void __launch_bounds__(NT) talk_decode_kernel(
 #pragma unroll
         for (int kt = 0; kt < 4; ++kt) {
           const f32x4 p = *reinterpret_cast<const f32x4*>(P + h * DS + 16 * kt + 4 * lg);
-          f32x4 vv[4];
+          Quad<T> vv[4];
 #pragma unroll
           for (int v = 0; v < 4; ++v) {
             const long vrow = rows[16 * kt + 4 * lg + v] + (long)g * block_size;
-            vv[v] = f32x4{0.f, 0.f, 0.f, 0.f};
-            if (d0 < D) vv[v] = load4_f32(k_cache + vrow * D + d0, vec, D - d0);
+            load_quad<FULL>(vv[v], k_cache + vrow * D + d0, vec, D - d0);
           }
 #pragma unroll
           for (int v = 0; v < 4; ++v)
 #pragma unroll
             for (int c = 0; c < 4; ++c)
-              o[i][c] = __builtin_amdgcn_mfma_f32_16x16x4f32(vv[v][c], p[v], o[i][c], 0, 0, 0);
+              o[i][c] = __builtin_amdgcn_mfma_f32_16x16x4f32(vv[v].get(c), p[v], o[i][c], 0, 0, 0);
         }
       }
     }
@@ -611,13 +671,16 @@ hipError_t allow_lds(F fn, size_t smem) {
                              hipFuncAttributeMaxDynamicSharedMemorySize, (int)smem);
 }
 
-template <typename T, int DP, int NH, int HT, bool SHARE>
+template <typename T, int DP, int NH, int HT, bool SHARE, bool FULL = false>
 hipError_t launch_prefill(const TalkArgs& a) {
-  constexpr int BK = HT <= 2 ? 32 : 16;
+  if constexpr (SHARE && !FULL && DP <= 128 && sizeof(T) == 2) {
+    if (a.D == DP) return launch_prefill<T, DP, NH, HT, SHARE, true>(a);
+  }
+  constexpr int BK = 16 * key_tiles(DP, NH, HT);
   const int H4 = (a.heads + 3) & ~3;
   const size_t smem =
       sizeof(float) * ((size_t)H4 * BK * QS + (size_t)H4 * 16 * HT + 4 * BK);
-  auto fn = talk_prefill_kernel<T, DP, NH, HT, SHARE>;
+  auto fn = talk_prefill_kernel<T, DP, NH, HT, SHARE, FULL>;
   hipError_t e = allow_lds(fn, smem);
   if (e != hipSuccess) return e;
   dim3 grid(cdiv(a.max_q_len, 16), a.num_seqs, cdiv(cdiv(a.heads, NH), NWV));
@@ -654,14 +717,17 @@ hipError_t dispatch_prefill(const TalkArgs& a) {
   }
 }
 
-template <typename T, int DP, int IPW>
+template <typename T, int DP, int IPW, bool FULL = false>
 hipError_t launch_decode(const TalkArgs& a, int items) {
+  if constexpr (!FULL && DP <= 128 && sizeof(T) == 2) {
+    if (a.D == DP) return launch_decode<T, DP, IPW, true>(a, items);
+  }
   const int H4 = (a.heads + 3) & ~3, HP = (a.heads + 15) & ~15;
   const size_t smem =
       sizeof(float) * ((size_t)a.heads * (DP + 4) + (size_t)H4 * DS +
                        (size_t)a.heads * DS + (size_t)H4 * HP + 3 * (size_t)H4 +
                        4 * DBK);
-  auto fn = talk_decode_kernel<T, DP, IPW>;
+  auto fn = talk_decode_kernel<T, DP, IPW, FULL>;
   hipError_t e = allow_lds(fn, smem);
   if (e != hipSuccess) return e;
   dim3 grid(a.nsplit, a.num_seqs, cdiv(items, NWV * IPW));
