@@ -190,9 +190,7 @@ def context_attention_varlen(
 
 def greedy_sample(logits: torch.Tensor) -> torch.Tensor:
     if logits.is_cuda:
-        if logits.dtype != torch.bfloat16:
-            # fp32 engines: the argmax must see every bit of the logits
-            return torch.argmax(logits, dim=-1)
+        # bf16 or fp32: an fp32 argmax sees every bit of the logits
         out = torch.empty(
             logits.shape[0], dtype=torch.int64, device=logits.device
         )

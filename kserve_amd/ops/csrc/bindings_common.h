@@ -9,7 +9,7 @@
 #include <hip/hip_runtime.h>
 
 extern "C" {
-hipError_t ks_greedy_sample(void*, const void*, int, int, hipStream_t);
+hipError_t ks_greedy_sample(void*, const void*, int, int, int, hipStream_t);
 hipError_t ks_gumbel_sample(void*, const void*, const void*, const void*,
                             const void*, int, int, hipStream_t);
 hipError_t ks_topk_topp_sample(void*, const void*, const void*, const void*,
@@ -34,10 +34,16 @@ void check_hip(hipError_t err, const char* op) {
   TORCH_CHECK((t).is_cuda(), #t " must be on GPU")
 
 void greedy_sample(at::Tensor& out, at::Tensor& logits) {
-  CHECK_BF16_CONTIG(logits);
-  TORCH_CHECK(out.scalar_type() == at::kLong, "out int64");
+  const bool f32 = logits.scalar_type() == at::kFloat;
+  if (f32)
+    TORCH_CHECK(logits.is_cuda() && logits.is_contiguous(), "logits [S, V] on GPU");
+  else
+    CHECK_BF16_CONTIG(logits);
+  TORCH_CHECK(out.scalar_type() == at::kLong && logits.dim() == 2 &&
+                  out.numel() == logits.size(0),
+              "out int64 [S]");
   check_hip(ks_greedy_sample(out.data_ptr(), logits.data_ptr(),
-                             logits.size(0), logits.size(1),
+                             logits.size(0), logits.size(1), f32 ? 1 : 0,
                              current_stream()),
             "greedy_sample");
 }

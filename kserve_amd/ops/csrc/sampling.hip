@@ -101,6 +101,47 @@ __global__ __launch_bounds__(256) void argmax_kernel(
   }
 }
 
+// fp32 logits [S, V]: argmax of every bit, ties to the lower index; one block
+// (256 threads) per row
+__global__ __launch_bounds__(256) void argmax_f32_kernel(
+    long* __restrict__ out, const float* __restrict__ logits, const int V) {
+  const float* row = logits + (long)blockIdx.x * V;
+  float best = -INFINITY;
+  int best_idx = 0;
+  for (int i = threadIdx.x; i < V; i += 256) {
+    const float val = row[i];
+    if (val > best) {
+      best = val;
+      best_idx = i;
+    }
+  }
+  __shared__ float s_val[4];
+  __shared__ int s_idx[4];
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+#pragma unroll
+  for (int off = 32; off > 0; off >>= 1) {
+    const float ov = __shfl_xor(best, off, 64);
+    const int oi = __shfl_xor(best_idx, off, 64);
+    if (ov > best || (ov == best && oi < best_idx)) {
+      best = ov;
+      best_idx = oi;
+    }
+  }
+  if (lane == 0) {
+    s_val[wave] = best;
+    s_idx[wave] = best_idx;
+  }
+  __syncthreads();
+  if (threadIdx.x == 0) {
+    for (int w = 1; w < 4; ++w)
+      if (s_val[w] > best || (s_val[w] == best && s_idx[w] < best_idx)) {
+        best = s_val[w];
+        best_idx = s_idx[w];
+      }
+    out[blockIdx.x] = best_idx;
+  }
+}
+
 // ---------------------------------------------------------------------------
 // Fused top-k/top-p + Gumbel-max sampler.
 //
@@ -275,8 +316,14 @@ __global__ __launch_bounds__(256) void topk_topp_sample_kernel(
 extern "C" {
 
 hipError_t ks_greedy_sample(void* out, const void* logits, int num_seqs,
-                            int vocab, hipStream_t stream) {
+                            int vocab, int is_f32, hipStream_t stream) {
   if (num_seqs == 0) return hipSuccess;
+  if (is_f32) {
+    hipLaunchKernelGGL(argmax_f32_kernel, dim3(num_seqs), dim3(256), 0, stream,
+                       (long*)out, (const float*)logits, vocab);
+    HIP_CHECK_KERNEL();
+    return hipSuccess;
+  }
   hipLaunchKernelGGL((argmax_kernel<false>), dim3(num_seqs), dim3(256), 0,
                      stream, (long*)out, (const short*)logits, nullptr,
                      nullptr, nullptr, vocab);

@@ -122,19 +122,34 @@ __device__ __forceinline__ void load_quad(Quad<T>& q, const T* p, bool vec, int 
   }
 }
 
-// cache row (of kv head 0) and score factor of `count` keys from k0 on; keys
-// past `last` repeat the last one (masked later)
-__device__ __forceinline__ void key_rows(int* rows, float* ksc, int k0, int last,
-                                         int count, const int* bt,
-                                         int block_size, int kv_heads,
-                                         const float* k_scale, float mult) {
-  if ((int)threadIdx.x < count) {
-    const int kp = min(k0 + (int)threadIdx.x, last);
-    const int blk = bt[kp / block_size], po = kp % block_size;
-    rows[threadIdx.x] = blk * kv_heads * block_size + po;
-    ksc[threadIdx.x] = k_scale[(long)blk * block_size + po] * mult;
+// Cache row (of kv head 0) and score factor of a tile's keys, one key per
+// thread, in steps so that the dependent loads of the next tile hide behind
+// this tile's work: find(), then load(), then store() to LDS. Keys past
+// `last` repeat the last one (masked later).
+struct KeyRows {
+  int blk, po;
+  float f;
+  __device__ __forceinline__ void find(int k0, int last, int count, const int* bt,
+                                       int block_size) {
+    if ((int)threadIdx.x < count) {
+      const int kp = min(k0 + (int)threadIdx.x, last);
+      blk = bt[kp / block_size];
+      po = kp % block_size;
+    }
   }
-}
+  __device__ __forceinline__ void load(int count, int block_size,
+                                       const float* k_scale) {
+    if ((int)threadIdx.x < count) f = k_scale[(long)blk * block_size + po];
+  }
+  __device__ __forceinline__ void store(int* rows, float* ksc, int count,
+                                        int block_size, int kv_heads,
+                                        float mult) const {
+    if ((int)threadIdx.x < count) {
+      rows[threadIdx.x] = blk * kv_heads * block_size + po;
+      ksc[threadIdx.x] = f * mult;
+    }
+  }
+};
 
 // 16-key tiles per step of the prefill kernel: two where the registers (heads
 // of a wave times the head size) and the LDS (heads) allow
@@ -188,7 +203,10 @@ __global__ void __launch_bounds__(NT) talk_prefill_kernel(
     Tt[e] = (g < heads && h < heads) ? talk[h * heads + g] : 0.f;
   }
   for (int e = heads * BK * QS + threadIdx.x; e < H4 * BK * QS; e += NT) S[e] = 0.f;
-  key_rows(Rows, Ksc, kbeg, last_pos, BK, bt, block_size, kv_heads, k_scale, mult);
+  KeyRows kr;
+  kr.find(kbeg, last_pos, BK, bt, block_size);
+  kr.load(BK, block_size, k_scale);
+  kr.store(Rows, Ksc, BK, block_size, kv_heads, mult);
 
   // this wave's heads in steps (1) and (3) when one block covers all heads;
   // otherwise step (1) walks all of them and step (3) takes this block's
@@ -208,6 +226,7 @@ __global__ void __launch_bounds__(NT) talk_prefill_kernel(
   for (int k0 = kbeg; k0 <= last_pos; k0 += BK, buf ^= 1) {
     const int* rows = Rows + buf * BK;
     const float* ksc = Ksc + buf * BK;
+    kr.find(k0 + BK, last_pos, BK, bt, block_size);
     // (1) scores of all heads
     for (int item = wave; item < items; item += NWV) {
       int hh[NH];
@@ -247,12 +266,18 @@ __global__ void __launch_bounds__(NT) talk_prefill_kernel(
       load_k(0);
       load_q(0);
       if (STEPS > 1) load_q(1);
+      f32x4 kfac[NKT];
+#pragma unroll
+      for (int t = 0; t < NKT; ++t)
+        kfac[t] = *reinterpret_cast<const f32x4*>(ksc + 16 * t + 4 * lg);
 #pragma unroll
       for (int st = 0; st < STEPS; ++st) {
         const int a = st % NH, k8 = st / NH;
         if (a == 0 && KR == 2 && k8 + 1 < K8) load_k(k8 + 1);
         if (a == 0 && KR == 1 && k8 > 0) load_k(k8);
         if (st + 2 < STEPS) load_q(st + 2);
+        // keep the loads ahead of this step's products
+        __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
         for (int c = 0; c < 8; ++c)
 #pragma unroll
@@ -269,37 +294,49 @@ __global__ void __launch_bounds__(NT) talk_prefill_kernel(
 #pragma unroll
             for (int v = 0; v < 4; ++v) {
               const int key = 16 * t + 4 * lg + v;
-              S[(hh[a] * BK + key) * QS + li] = acc[a][t][v] * ksc[key];
+              S[(hh[a] * BK + key) * QS + li] = acc[a][t][v] * kfac[t][v];
             }
         }
       }
     }
+    kr.load(BK, block_size, k_scale);
     __syncthreads();
-    // the next tile's rows: every wave is past the previous tile's last use
-    // of the other buffer
-    key_rows(Rows + (buf ^ 1) * BK, Ksc + (buf ^ 1) * BK, k0 + BK, last_pos, BK, bt,
-             block_size, kv_heads, k_scale, mult);
-    // (2) mix over the heads, one key at a time; the wave reads a key's scores
-    // of all heads before it writes any
-    for (int key = wave; key < BK; key += NWV) {
-      f32x4 mx[HT];
+    // (2) mix over the heads, in place: the wave reads its keys' scores of all
+    // heads before it writes any
+    {
+      constexpr int KPW = BK / NWV;  // keys of a wave: wave * KPW ...
+      f32x4 mx[KPW][HT];
 #pragma unroll
-      for (int t = 0; t < HT; ++t) mx[t] = f32x4{0.f, 0.f, 0.f, 0.f};
+      for (int k = 0; k < KPW; ++k)
+#pragma unroll
+        for (int t = 0; t < HT; ++t) mx[k][t] = f32x4{0.f, 0.f, 0.f, 0.f};
       for (int g4 = 0; g4 < H4; g4 += 4) {
-        const float b = S[((g4 + lg) * BK + key) * QS + li];
+        float ta[HT], sb[KPW];
 #pragma unroll
-        for (int t = 0; t < HT; ++t)
-          mx[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(
-              Tt[(g4 + lg) * 16 * HT + 16 * t + li], b, mx[t], 0, 0, 0);
+        for (int t = 0; t < HT; ++t) ta[t] = Tt[(g4 + lg) * 16 * HT + 16 * t + li];
+#pragma unroll
+        for (int k = 0; k < KPW; ++k)
+          sb[k] = S[((g4 + lg) * BK + wave * KPW + k) * QS + li];
+#pragma unroll
+        for (int k = 0; k < KPW; ++k)
+#pragma unroll
+          for (int t = 0; t < HT; ++t)
+            mx[k][t] = __builtin_amdgcn_mfma_f32_16x16x4f32(ta[t], sb[k], mx[k][t], 0, 0, 0);
       }
 #pragma unroll
       for (int t = 0; t < HT; ++t)
 #pragma unroll
         for (int v = 0; v < 4; ++v) {
           const int h = 16 * t + 4 * lg + v;
-          if (h < heads) S[(h * BK + key) * QS + li] = mx[t][v];
+          if (h < heads) {
+#pragma unroll
+            for (int k = 0; k < KPW; ++k)
+              S[(h * BK + wave * KPW + k) * QS + li] = mx[k][t][v];
+          }
         }
     }
+    // every wave is past the previous tile's last use of the other buffer
+    kr.store(Rows + (buf ^ 1) * BK, Ksc + (buf ^ 1) * BK, BK, block_size, kv_heads, mult);
     __syncthreads();
     // (3) softmax and values of this wave's heads
     if (item3 < items) {
@@ -312,25 +349,37 @@ __global__ void __launch_bounds__(NT) talk_prefill_kernel(
         for (int j = 0; j < VJ; ++j)
           load_quad<FULL>(dst[j], row + 64 * j + 4 * li, vec, D - (64 * j + 4 * li));
       };
-      Quad<T> vs[4][VJ];
+      Quad<T> vs[SHARE ? NKT : 1][4][VJ];
       if (SHARE) {
 #pragma unroll
-        for (int v = 0; v < 4; ++v) load_v(vs[v], 0, v, 0);
+        for (int v = 0; v < 4; ++v) load_v(vs[0][v], 0, v, 0);
       }
-      float p[NH][NKT][4];
+      // bias of every (head, key) of this lane, all loads in flight at once
+      float p[NH][NKT][4], bs[NH][NKT][4];
 #pragma unroll
       for (int a = 0; a < NH; ++a) {
         const int h = min(item3 * NH + a, heads - 1);
         const float* bh = bias + (long)h * bias_n;
-        float mt = -INFINITY;
 #pragma unroll
         for (int t = 0; t < NKT; ++t)
 #pragma unroll
           for (int v = 0; v < 4; ++v) {
             const int key = 16 * t + 4 * lg + v;
-            const int kp = k0 + key;
-            const int n = min(max(qpos - kp, 0), bias_n - 1);
-            const float sc = S[(h * BK + key) * QS + li] + bh[n] * LOG2E;
+            bs[a][t][v] = bh[min(max(qpos - (k0 + key), 0), bias_n - 1)];
+            p[a][t][v] = S[(h * BK + key) * QS + li];
+          }
+      }
+      __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+      for (int a = 0; a < NH; ++a) {
+        float mt = -INFINITY;
+#pragma unroll
+        for (int t = 0; t < NKT; ++t)
+#pragma unroll
+          for (int v = 0; v < 4; ++v) {
+            const int kp = k0 + 16 * t + 4 * lg + v;
+            float sc = p[a][t][v] + bs[a][t][v] * LOG2E;
+            asm volatile("" : "+v"(sc));  // a select below, no branch around the loads
             p[a][t][v] = (kp <= qpos && kp >= qstart) ? sc : -INFINITY;
             mt = fmaxf(mt, p[a][t][v]);
           }
@@ -357,22 +406,23 @@ __global__ void __launch_bounds__(NT) talk_prefill_kernel(
       }
 #pragma unroll
       for (int t = 0; t < NKT; ++t) {
-        if (SHARE && t > 0) {
+        if (SHARE && t + 1 < NKT) {
 #pragma unroll
-          for (int v = 0; v < 4; ++v) load_v(vs[v], t, v, 0);
+          for (int v = 0; v < 4; ++v) load_v(vs[t + 1][v], t + 1, v, 0);
+          __builtin_amdgcn_sched_barrier(0);
         }
         // row li of output tile 4 j + c is value column 64 j + 4 li + c
 #pragma unroll
         for (int v = 0; v < 4; ++v)
 #pragma unroll
           for (int a = 0; a < NH; ++a) {
-            if (!SHARE) load_v(vs[0], t, v, a);
+            if (!SHARE) load_v(vs[0][0], t, v, a);
 #pragma unroll
             for (int j = 0; j < VJ; ++j)
 #pragma unroll
               for (int c = 0; c < 4; ++c)
                 o[a][4 * j + c] = __builtin_amdgcn_mfma_f32_16x16x4f32(
-                    vs[SHARE ? v : 0][j].get(c), p[a][t][v], o[a][4 * j + c], 0, 0, 0);
+                    vs[SHARE ? t : 0][SHARE ? v : 0][j].get(c), p[a][t][v], o[a][4 * j + c], 0, 0, 0);
           }
       }
     }
@@ -471,7 +521,10 @@ __global__ void __launch_bounds__(NT) talk_decode_kernel(
   }
   const int kfirst = kbeg + split * DBK;
   const int kstep = nsplit * DBK;
-  key_rows(Rows, Ksc, kfirst, pos, DBK, bt, block_size, kv_heads, k_scale, mult);
+  KeyRows kr;
+  kr.find(kfirst, pos, DBK, bt, block_size);
+  kr.load(DBK, block_size, k_scale);
+  kr.store(Rows, Ksc, DBK, block_size, kv_heads, mult);
 
   // value items of this wave: kv head, first query head, number of them, columns
   const int items = kv_heads * ct * nj;
@@ -487,6 +540,7 @@ __global__ void __launch_bounds__(NT) talk_decode_kernel(
   for (int k0 = kfirst; k0 <= pos; k0 += kstep, buf ^= 1) {
     const int* rows = Rows + buf * DBK;
     const float* ksc = Ksc + buf * DBK;
+    kr.find(k0 + kstep, pos, DBK, bt, block_size);
     // (1) scores: 16 keys x the heads of one key group
     for (int u = wave; u < kv_heads * ct * 4; u += NWV) {
       const int kt = u & 3, gc = u >> 2;
@@ -516,9 +570,8 @@ __global__ void __launch_bounds__(NT) talk_decode_kernel(
         *reinterpret_cast<f32x4*>(S + h * DS + 16 * kt + 4 * lg) = (acc + acc2) * f;
       }
     }
+    kr.load(DBK, block_size, k_scale);
     __syncthreads();
-    key_rows(Rows + (buf ^ 1) * DBK, Ksc + (buf ^ 1) * DBK, k0 + kstep, pos, DBK, bt,
-             block_size, kv_heads, k_scale, mult);
     // (2) mix over the heads: 16 heads x 16 keys a unit
     for (int u = wave; u < (HP / 16) * 4; u += NWV) {
       const int kt = u & 3, ht = u >> 2;
@@ -533,6 +586,7 @@ __global__ void __launch_bounds__(NT) talk_decode_kernel(
         if (h < heads) P[h * DS + 16 * kt + li] = mx[v];
       }
     }
+    kr.store(Rows + (buf ^ 1) * DBK, Ksc + (buf ^ 1) * DBK, DBK, block_size, kv_heads, mult);
     __syncthreads();
     // (3) softmax, one key per lane
     for (int h = wave; h < heads; h += NWV) {

@@ -552,3 +552,15 @@ class TestTalkingHeads:
                 w = k * math.exp(-2.0) / (1 + k * math.exp(-2.0))
                 assert abs(float(out[i, 0]) - w) < 1e-6
                 assert abs(float(out[i, 5]) - w / 2) < 1e-6
+
+
+class TestGreedyFp32:
+    @pytest.mark.parametrize("V", [1, 61, 255, 4097])
+    def test_every_bit_and_ties(self, dev, V):
+        """fp32 logits that differ below the bf16 step; ties go to the lower
+        index; masked (-inf) entries."""
+        x = 1.0 + 1e-4 * rnd(9, V, seed=20).to(dev)
+        assert (ops.greedy_sample(x).cpu() == x.cpu().argmax(-1)).all()
+        x = torch.full((3, V), -math.inf)
+        x[:, V // 2 :] = 2.5
+        assert (ops.greedy_sample(x.to(dev)).cpu() == V // 2).all()
