@@ -35,10 +35,11 @@ void check_hip(hipError_t err, const char* op) {
 
 void greedy_sample(at::Tensor& out, at::Tensor& logits) {
   const bool f32 = logits.scalar_type() == at::kFloat;
-  if (f32)
+  if (f32) {
     TORCH_CHECK(logits.is_cuda() && logits.is_contiguous(), "logits [S, V] on GPU");
-  else
+  } else {
     CHECK_BF16_CONTIG(logits);
+  }
   TORCH_CHECK(out.scalar_type() == at::kLong && logits.dim() == 2 &&
                   out.numel() == logits.size(0),
               "out int64 [S]");
