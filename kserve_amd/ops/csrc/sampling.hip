@@ -102,42 +102,64 @@ __global__ __launch_bounds__(256) void argmax_kernel(
 }
 
 // fp32 logits [S, V]: argmax of every bit, ties to the lower index; one block
-// (256 threads) per row
-__global__ __launch_bounds__(256) void argmax_f32_kernel(
-    long* __restrict__ out, const float* __restrict__ logits, const int V) {
+// of 1024 threads per row. vec: rows start on 16-byte boundaries.
+constexpr int AM_NT = 1024;
+
+__global__ __launch_bounds__(AM_NT) void argmax_f32_kernel(
+    long* __restrict__ out, const float* __restrict__ logits, const int V,
+    const int vec) {
   const float* row = logits + (long)blockIdx.x * V;
-  float best = -INFINITY;
+  // finite: one of the modules this file is built into assumes finite math
+  float best = -3.4e38f;
   int best_idx = 0;
-  for (int i = threadIdx.x; i < V; i += 256) {
-    const float val = row[i];
+  auto take = [&](float val, int idx) {
+    // a thread's indexes only grow, so ">" keeps its lowest
     if (val > best) {
       best = val;
-      best_idx = i;
+      best_idx = idx;
     }
-  }
-  __shared__ float s_val[4];
-  __shared__ int s_idx[4];
-  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  };
+  int done = 0;
+  if (vec) {
+    const float4_t* rv = reinterpret_cast<const float4_t*>(row);
+    const int nvec = V >> 2;
+    int i = threadIdx.x;
+    for (; i + 3 * AM_NT < nvec; i += 4 * AM_NT) {
+      float4_t v[4];
 #pragma unroll
-  for (int off = 32; off > 0; off >>= 1) {
-    const float ov = __shfl_xor(best, off, 64);
-    const int oi = __shfl_xor(best_idx, off, 64);
+      for (int u = 0; u < 4; ++u) v[u] = rv[i + u * AM_NT];
+#pragma unroll
+      for (int u = 0; u < 4; ++u)
+#pragma unroll
+        for (int c = 0; c < 4; ++c) take(v[u][c], (i + u * AM_NT) * 4 + c);
+    }
+    for (; i < nvec; i += AM_NT) {
+      const float4_t v = rv[i];
+#pragma unroll
+      for (int c = 0; c < 4; ++c) take(v[c], i * 4 + c);
+    }
+    done = nvec * 4;
+  }
+  for (int i = done + threadIdx.x; i < V; i += AM_NT) take(row[i], i);
+  __shared__ float s_val[AM_NT / 64];
+  __shared__ int s_idx[AM_NT / 64];
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  auto merge = [&](float ov, int oi) {
     if (ov > best || (ov == best && oi < best_idx)) {
       best = ov;
       best_idx = oi;
     }
-  }
+  };
+#pragma unroll
+  for (int off = 32; off > 0; off >>= 1)
+    merge(__shfl_xor(best, off, 64), __shfl_xor(best_idx, off, 64));
   if (lane == 0) {
     s_val[wave] = best;
     s_idx[wave] = best_idx;
   }
   __syncthreads();
   if (threadIdx.x == 0) {
-    for (int w = 1; w < 4; ++w)
-      if (s_val[w] > best || (s_val[w] == best && s_idx[w] < best_idx)) {
-        best = s_val[w];
-        best_idx = s_idx[w];
-      }
+    for (int w = 1; w < AM_NT / 64; ++w) merge(s_val[w], s_idx[w]);
     out[blockIdx.x] = best_idx;
   }
 }
@@ -319,8 +341,9 @@ hipError_t ks_greedy_sample(void* out, const void* logits, int num_seqs,
                             int vocab, int is_f32, hipStream_t stream) {
   if (num_seqs == 0) return hipSuccess;
   if (is_f32) {
-    hipLaunchKernelGGL(argmax_f32_kernel, dim3(num_seqs), dim3(256), 0, stream,
-                       (long*)out, (const float*)logits, vocab);
+    const int vec = vocab % 4 == 0 && ((uintptr_t)logits % 16) == 0;
+    hipLaunchKernelGGL(argmax_f32_kernel, dim3(num_seqs), dim3(AM_NT), 0, stream,
+                       (long*)out, (const float*)logits, vocab, vec);
     HIP_CHECK_KERNEL();
     return hipSuccess;
   }

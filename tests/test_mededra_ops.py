@@ -555,7 +555,7 @@ class TestTalkingHeads:
 
 
 class TestGreedyFp32:
-    @pytest.mark.parametrize("V", [1, 61, 255, 4097])
+    @pytest.mark.parametrize("V", [1, 61, 256, 4097, 40000])
     def test_every_bit_and_ties(self, dev, V):
         """fp32 logits that differ below the bf16 step; ties go to the lower
         index; masked (-inf) entries."""
