@@ -167,6 +167,13 @@ class ModelConfig:
         )
 
 
+def rot_scaling_spec(rot: dict) -> Optional[dict]:
+    """``rot.scaling`` of a mixer entry as numbers: the keys of linear scaling
+    (``factor``) or of YaRN (``factor, original, fast, slow``)."""
+    sc = rot.get("scaling")
+    return {k: float(v) for k, v in sc.items()} if sc else None
+
+
 @dataclass
 class AttentionMixerSpec:
     """Softmax attention sublayer with grouped KV heads. Independent query/key
@@ -190,6 +197,10 @@ class AttentionMixerSpec:
     # sliding window: a query sees itself and the window-1 positions before
     # it; 0 = no window
     window: int = 0
+    # with a window: the first ``keep_first`` positions stay visible
+    keep_first: int = 0
+    # None, {"factor"} (linear) or {"factor", "original", "fast", "slow"} (YaRN)
+    rot_scaling: Optional[dict] = None
 
     @classmethod
     def from_dict(cls, d: dict, mask: str = "chunk") -> "AttentionMixerSpec":
@@ -197,7 +208,8 @@ class AttentionMixerSpec:
         that is being read: "chunk" or "window"."""
         qt = d.get("q_temp") or {}
         rot = d.get("rot") or {}
-        size = int((d.get("mask") or {}).get("size", 0))
+        m = d.get("mask") or {}
+        size = int(m.get("size", 0))
         chunk = size if mask == "chunk" else 0
         window = size if mask == "window" else 0
         return cls(
@@ -212,6 +224,8 @@ class AttentionMixerSpec:
             rot_base=float(rot.get("base", 10000.0)),
             chunk=chunk,
             window=window,
+            keep_first=int(m.get("keep_first", 0)) if window else 0,
+            rot_scaling=rot_scaling_spec(rot),
         )
 
 
@@ -280,6 +294,30 @@ class DeltaMixerSpec:
             vdim=int(d.get("vdim", d["dim"])),
             conv=int(d.get("conv", 4)),
             channel_decay=channel_decay,
+        )
+
+
+@dataclass
+class GatedLinearMixerSpec:
+    """Linear attention with a data-dependent decay per head and key channel
+    and no softmax: a = sigmoid(z)^(1/tau) with z from a projection through
+    ``a_rank`` columns, S <- diag(a) S + k v^T, o = S^T q dim^-1/2, head
+    outputs RMS-normed and gated. ``a_rank`` 0: one head's size until a
+    checkpoint's tensor shapes say otherwise."""
+
+    heads: int
+    dim: int
+    vdim: int
+    tau: float
+    a_rank: int = 0
+
+    @classmethod
+    def from_dict(cls, d: dict) -> "GatedLinearMixerSpec":
+        return cls(
+            heads=int(d["heads"]),
+            dim=int(d["dim"]),
+            vdim=int(d.get("vdim", d["dim"])),
+            tau=float(d["tau"]),
         )
 
 
@@ -493,8 +531,11 @@ class LatentAttentionSpec:
     """Attention whose keys and values are expanded per head from one cached
     latent vector per token: the cache holds ``kv_rank`` normed latent
     coordinates and (with ``rot_dim`` > 0) one rotated key part shared by all
-    heads. Queries go through a normed latent of ``q_rank`` coordinates and
+    heads. Queries go through a normed latent of ``q_rank`` coordinates (0:
+    they are projected from the input) and
     have ``dim`` unrotated + ``rot_dim`` rotated coordinates per head.
+    ``rot_pairs``: coordinates 2i and 2i+1 turn together, otherwise i and
+    i + rot_dims/2.
     ``window`` > 0: a query sees itself and the window-1 positions before it;
     ``sink``: one more term exp(sink_h) in the softmax denominator; ``gate``:
     head outputs times sigmoid of a projection of the sublayer input;
@@ -514,13 +555,17 @@ class LatentAttentionSpec:
     sink: bool = False
     gate: bool = False
     kv_from: Optional[int] = None
+    rot_pairs: bool = True
+    rot_scaling: Optional[dict] = None
 
     @property
     def cache_dim(self) -> int:
         return self.kv_rank + self.rot_dim
 
     @classmethod
-    def from_dict(cls, d: dict, sink: bool, gate: bool) -> "LatentAttentionSpec":
+    def from_dict(
+        cls, d: dict, sink: bool, gate: bool, rot_pairs: bool = True
+    ) -> "LatentAttentionSpec":
         rot = d.get("rot") or {}
         mask = d.get("mask") or {}
         rot_dim = int(d.get("rot_dim", 0))
@@ -530,7 +575,7 @@ class LatentAttentionSpec:
             dim=int(d["dim"]),
             vdim=int(d.get("vdim", d["dim"])),
             kv_rank=int(d["kv_rank"]),
-            q_rank=int(d["q_rank"]),
+            q_rank=int(d.get("q_rank", 0)),
             scale=float(d["scale"]),
             rot_dim=rot_dim,
             rot_dims=int(rot.get("dims", rot_dim)) if rot_dim else 0,
@@ -539,6 +584,8 @@ class LatentAttentionSpec:
             sink=sink,
             gate=gate,
             kv_from=None if kv_from is None else int(kv_from),
+            rot_pairs=rot_pairs,
+            rot_scaling=rot_scaling_spec(rot),
         )
 
 
@@ -561,20 +608,27 @@ class SoftmaxMoESpec:
     (uncorrected) scores renormalised to sum 1, and the weight multiplies the
     expert's OUTPUT. The last ``identity`` router outputs stand for experts
     that return their input; ``experts`` counts the real ones. An optional
-    shared expert of the same form runs for every token."""
+    shared expert of the same form runs for every token. ``over_chosen``: the
+    choice goes by the logits themselves and the weights are the softmax over
+    the chosen logits only (no correction). ``router_bias``: a bias on the
+    router logits."""
 
     experts: int
     top: int
     ff: int
     identity: int = 0
     shared_ff: int = 0
+    over_chosen: bool = False
+    router_bias: bool = False
 
     @property
     def router_outputs(self) -> int:
         return self.experts + self.identity
 
     @classmethod
-    def from_dict(cls, d: dict) -> "SoftmaxMoESpec":
+    def from_dict(
+        cls, d: dict, over_chosen: bool = False, router_bias: bool = False
+    ) -> "SoftmaxMoESpec":
         r = d["router"]
         sh = d.get("shared")
         return cls(
@@ -583,6 +637,8 @@ class SoftmaxMoESpec:
             ff=int(d["expert"]["ff"]),
             identity=int(r.get("identity", 0)),
             shared_ff=int(sh["ff"]) if sh else 0,
+            over_chosen=over_chosen,
+            router_bias=router_bias,
         )
 
 
@@ -640,6 +696,36 @@ def mededra_layer_spec(kind: str, mixer: dict, mlp: Optional[dict]):
     raise ValueError(f"unknown layer type {kind!r}")
 
 
+def kebesun_layer_spec(kind: str, mixer: dict, mlp: Optional[dict]):
+    """One Kebesun layer: windowed attention with kept first positions,
+    latent attention or gated linear attention, and beside it an optional
+    dense or routed feed-forward reading the same norm."""
+    ff = None
+    if mlp:
+        if mlp.get("kind", "moe" if "router" in mlp else "dense") == "moe":
+            ff = SoftmaxMoESpec.from_dict(mlp, over_chosen=True, router_bias=True)
+        else:
+            ff = SiluGLUSpec.from_dict(mlp)
+    if kind == "attention":
+        return HybridLayerSpec(
+            kind, attention=AttentionMixerSpec.from_dict(mixer, mask="window"),
+            mlp=ff,
+        )
+    if kind == "latent_attention":
+        return HybridLayerSpec(
+            kind,
+            latent=LatentAttentionSpec.from_dict(
+                mixer, sink=False, gate=False, rot_pairs=False
+            ),
+            mlp=ff,
+        )
+    if kind == "gla":
+        return HybridLayerSpec(
+            kind, gated_linear=GatedLinearMixerSpec.from_dict(mixer), mlp=ff
+        )
+    raise ValueError(f"unknown layer type {kind!r}")
+
+
 @dataclass
 class LoopSpec:
     """Layers ``start .. stop-1`` run ``times`` times in a row with the same
@@ -664,6 +750,7 @@ class HybridLayerSpec:
     delta: Optional[DeltaMixerSpec] = None
     differential: Optional[DifferentialMixerSpec] = None
     talking: Optional[TalkingMixerSpec] = None
+    gated_linear: Optional[GatedLinearMixerSpec] = None
     attention_scale: float = 1.0
     ssm_scale: float = 1.0
     # GLUSpec, SiluGLUSpec, MoESpec, MLPSpec, SoftmaxMoESpec or
@@ -717,6 +804,7 @@ class HybridModelConfig:
     def has_recurrent_state(self) -> bool:
         return any(
             l.ssm is not None or l.retention is not None or l.delta is not None
+            or l.gated_linear is not None
             or (l.differential is not None and l.differential.conv > 1)
             for l in self.layers
         )
@@ -748,6 +836,9 @@ class HybridModelConfig:
         for entry in cfg["layers"]:
             kind = entry["type"]
             mixer = entry["mixer"]
+            if arch == "Kebesun":
+                layers.append(kebesun_layer_spec(kind, mixer, entry.get("mlp")))
+                continue
             if arch == "Mededra":
                 layers.append(mededra_layer_spec(kind, mixer, entry.get("mlp")))
                 continue

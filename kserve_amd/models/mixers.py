@@ -15,7 +15,7 @@ they need ``cu_seqlens`` / ``seq_of_token`` (flat-batch layout) and
 from __future__ import annotations
 
 import math
-from typing import NamedTuple, Optional
+from typing import NamedTuple, Optional, Tuple
 
 import torch
 import torch.nn as nn
@@ -26,6 +26,7 @@ from kserve_amd.engine.config import (
     AttentionMixerSpec,
     DeltaMixerSpec,
     DifferentialMixerSpec,
+    GatedLinearMixerSpec,
     GLUSpec,
     LatentAttentionSpec,
     MLPSpec,
@@ -39,6 +40,8 @@ from kserve_amd.engine.config import (
 from kserve_amd.ops.torch_ref import (
     distance_buckets,
     rotary_inv_freq,
+    rotate_by_layout,
+    scaled_inv_freq,
     yarn_inv_freq,
 )
 
@@ -190,7 +193,9 @@ class RotaryChunkSinkAttention(nn.Module):
     that are rotated by their own position over all of ``vdim`` before they
     are cached, with every head output turned back by the query's position
     (``value_unit_norm`` / ``rotate_values``). ``spec.window`` adds a sliding
-    window. With ``norm_weights`` off the q/k norm has no weights (it then
+    window, ``spec.keep_first`` positions that stay visible outside it,
+    ``spec.rot_scaling`` changes the rotation's frequencies. ``qk_norm`` off
+    leaves q and k un-normed. With ``norm_weights`` off the q/k norm has no weights (it then
     commutes with the rotation, so "rotate, then norm" is the same sublayer).
     No biases, no gate. The q|k|v projections are one fused GEMM."""
 
@@ -198,11 +203,14 @@ class RotaryChunkSinkAttention(nn.Module):
         self, width: int, spec: AttentionMixerSpec, eps: float, dtype,
         sink: bool = True, value_unit_norm: bool = True,
         rotate_values: bool = True, norm_weights: bool = True,
+        qk_norm: bool = True,
     ):
         super().__init__()
         self.spec = spec
         self.eps = eps
         self.dtype = dtype
+        self.qk_norm = qk_norm
+        norm_weights = norm_weights and qk_norm
         self.q_w = spec.heads * spec.dim
         self.k_w = spec.kv_heads * spec.dim
         self.v_w = spec.kv_heads * spec.vdim
@@ -216,11 +224,12 @@ class RotaryChunkSinkAttention(nn.Module):
         self.sink = _param(spec.heads, dtype=torch.float32) if sink else None
         self.o_proj = _param(width, spec.heads * spec.vdim, dtype=dtype)
         self.value_unit_norm = value_unit_norm
-        self.register_buffer(
-            "qk_inv_freq",
-            rotary_inv_freq(spec.rot_dims, spec.rot_base) if spec.rot_dims else None,
-            persistent=False,
-        )
+        inv_freq, self.rot_mult = None, 1.0
+        if spec.rot_dims:
+            inv_freq, self.rot_mult = scaled_inv_freq(
+                spec.rot_dims, spec.rot_base, spec.rot_scaling
+            )
+        self.register_buffer("qk_inv_freq", inv_freq, persistent=False)
         self.register_buffer(
             "v_inv_freq",
             rotary_inv_freq(spec.vdim, spec.rot_base) if rotate_values else None,
@@ -247,12 +256,14 @@ class RotaryChunkSinkAttention(nn.Module):
             proj[:, :a], proj[:, a:b], proj[:, b:], self.q_norm, self.k_norm,
             positions, meta.slot_mapping, cache.k, cache.v, self.eps, s.heads,
             self.qk_inv_freq, self.value_unit_norm, self.v_inv_freq,
+            rot_mult=self.rot_mult, qk_norm=self.qk_norm,
         )
         o = ops.ctx_attention_f32(
             qn, cache.k, cache.v, meta.block_tables, meta.cu_seqlens,
             meta.context_lens, s.scale, meta.max_seqlen, s.heads,
             out_dtype=self.dtype, sink=self.sink, chunk=s.chunk,
             out_inv_freq=self.v_inv_freq, window=s.window,
+            keep_first=s.keep_first,
         )
         return F.linear(o, self.o_proj)
 
@@ -419,7 +430,9 @@ class LatentAttention(nn.Module):
     Options: ``window`` (sliding), ``sink`` (softmax denominator term),
     ``gate``, ``rot_dim`` = 0 (no positions at all), ``kv_from`` (no kv
     projection: the layer attends to the pages of an earlier layer with its
-    own U_k / U_v).
+    own U_k / U_v), ``q_rank`` = 0 (queries projected from the input, in the
+    same GEMM), ``rot_pairs`` off (coordinate i turns with i + half),
+    ``rot_scaling``.
 
     Rows wider than the attention kernel takes (``MAX_CACHE_DIM``) switch the
     layer to the expanded form: every step reads the sequences' cached rows,
@@ -448,37 +461,42 @@ class LatentAttention(nn.Module):
             )
         self.own_kv = s.kv_from is None
         self.kv_cols = s.cache_dim if self.own_kv else 0
+        q_cols = s.heads * (s.dim + s.rot_dim)
+        # columns ahead of the kv part: the query latent, or the queries
+        self.q_in = s.q_rank or q_cols
         self.in_proj = _param(
-            s.q_rank + self.kv_cols + (s.heads if s.gate else 0), width, dtype=dtype
+            self.q_in + self.kv_cols + (s.heads if s.gate else 0), width, dtype=dtype
         )
-        self.q_norm = _param(s.q_rank, dtype=torch.float32)
+        self.q_norm = _param(s.q_rank, dtype=torch.float32) if s.q_rank else None
         self.kv_norm = (
             _param(s.kv_rank, dtype=torch.float32) if self.own_kv else None
         )
-        self.uq = _param(s.heads * (s.dim + s.rot_dim), s.q_rank, dtype=dtype)
+        self.uq = _param(q_cols, s.q_rank, dtype=dtype) if s.q_rank else None
         # U_k transposed per head, [heads, kv_rank, dim]: it maps a query
         # head into latent coordinates; U_v as stored, [heads, vdim, kv_rank]
         self.uk_t = _param(s.heads, s.kv_rank, s.dim, dtype=dtype)
         self.uv = _param(s.heads, s.vdim, s.kv_rank, dtype=dtype)
         self.sink = _param(s.heads, dtype=torch.float32) if s.sink else None
         self.o_proj = _param(width, s.heads * s.vdim, dtype=dtype)
-        self.register_buffer(
-            "inv_freq",
-            rotary_inv_freq(s.rot_dims, s.rot_base) if s.rot_dims else None,
-            persistent=False,
-        )
+        inv_freq, self.rot_mult = None, 1.0
+        if s.rot_dims:
+            inv_freq, self.rot_mult = scaled_inv_freq(
+                s.rot_dims, s.rot_base, s.rot_scaling
+            )
+        self.register_buffer("inv_freq", inv_freq, persistent=False)
 
     def load(self, get, prefix: str):
         dt, s = self.dtype, self.spec
-        parts = [get(prefix + "dq").to(dt)]
+        parts = [get(prefix + ("dq" if s.q_rank else "q")).to(dt)]
         if self.own_kv:
             parts.append(get(prefix + "dkv").to(dt))
             self.kv_norm.copy_(get(prefix + "dkv.norm").float())
         if s.gate:
             parts.append(get(prefix + "g").to(dt))
         self.in_proj.copy_(torch.cat(parts, dim=0))
-        self.q_norm.copy_(get(prefix + "dq.norm").float())
-        self.uq.copy_(get(prefix + "uq").to(dt))
+        if s.q_rank:
+            self.q_norm.copy_(get(prefix + "dq.norm").float())
+            self.uq.copy_(get(prefix + "uq").to(dt))
         self.uk_t.copy_(
             get(prefix + "uk").to(dt).view(s.heads, s.dim, s.kv_rank).transpose(1, 2)
         )
@@ -491,14 +509,17 @@ class LatentAttention(nn.Module):
         """``cache.k``: this layer's pages, or those of layer ``kv_from``."""
         s = self.spec
         proj = F.linear(h, self.in_proj)
-        cq = ops.latent_norm_rope_cache(
-            proj, s.q_rank, s.kv_rank if self.own_kv else 0,
-            s.rot_dim if self.own_kv else 0, self.q_norm, self.kv_norm,
-            positions, meta.slot_mapping, cache.k if self.own_kv else None,
-            self.eps, self.inv_freq,
-        )
-        q = F.linear(cq, self.uq)
-        gate = proj[:, s.q_rank + self.kv_cols :] if s.gate else None
+        turn = {"pairs": s.rot_pairs, "rot_mult": self.rot_mult}
+        if s.q_rank or self.own_kv:
+            cq = ops.latent_norm_rope_cache(
+                proj if s.q_rank else proj[:, self.q_in :], s.q_rank,
+                s.kv_rank if self.own_kv else 0,
+                s.rot_dim if self.own_kv else 0, self.q_norm, self.kv_norm,
+                positions, meta.slot_mapping, cache.k if self.own_kv else None,
+                self.eps, self.inv_freq, **turn,
+            )
+        q = F.linear(cq, self.uq) if s.q_rank else proj[:, : self.q_in]
+        gate = proj[:, self.q_in + self.kv_cols :] if s.gate else None
         if self.expanded:
             return F.linear(
                 self._expanded_attention(q, gate, positions, cache, meta),
@@ -506,7 +527,7 @@ class LatentAttention(nn.Module):
             )
         qf = ops.head_matmul_rope(
             q, self.uk_t, s.heads, s.rot_dim, positions, self.inv_freq,
-            torch.float32,
+            torch.float32, **turn,
         )
         o_lat = ops.ctx_attention_f32(
             qf, cache.k, cache.k[..., : s.kv_rank], meta.block_tables,
@@ -521,17 +542,16 @@ class LatentAttention(nn.Module):
         """Per-head keys and values of every sequence's whole context, built
         from its cached rows into scratch pages (numbered 0.. in sequence
         order), then plain multi-head attention. -> [T, heads * vdim]."""
-        from kserve_amd.ops.torch_ref import rotate_pairs
-
         s = self.spec
         H, R, rd = s.heads, s.kv_rank, s.rot_dim
         T = q.shape[0]
-        q3 = q.view(T, H, s.dim + rd).float()
+        q3 = q.reshape(T, H, s.dim + rd).float()
         if rd:
-            q3 = torch.cat(
-                [q3[..., : s.dim], rotate_pairs(q3[..., s.dim :], positions, self.inv_freq)],
-                dim=-1,
+            turned = rotate_by_layout(
+                q3[..., s.dim :], positions, self.inv_freq, s.rot_pairs,
+                self.rot_mult,
             )
+            q3 = torch.cat([q3[..., : s.dim], turned], dim=-1)
         qf = q3.reshape(T, H * (s.dim + rd)).contiguous()
         n_seq = meta.cu_seqlens.numel() - 1
         ctx = meta.context_lens[:n_seq].tolist()  # host read
@@ -543,13 +563,16 @@ class LatentAttention(nn.Module):
         rows = cache.k[ids, 0]                       # [pages, bs, R + rd]
         n_pages = rows.shape[0]
         lat = rows[..., :R].reshape(-1, R)
-        keys = torch.matmul(lat, self.uk_t)                                  # [H, n, dim]
+        # one plain GEMM each: rows [n, R] against all heads' matrices
+        uk = self.uk_t.transpose(1, 2).reshape(H * s.dim, R)
+        keys = F.linear(lat, uk).view(n_pages, bs, H, s.dim)
         if rd:
-            shared = rows[..., R:].reshape(1, -1, rd).expand(H, -1, -1)
+            shared = rows[..., R:].unsqueeze(2).expand(-1, -1, H, -1)
             keys = torch.cat([keys, shared], dim=-1)
-        vals = torch.matmul(lat, self.uv.transpose(1, 2))                    # [H, n, vdim]
-        k_tmp = keys.view(H, n_pages, bs, -1).transpose(0, 1).contiguous()
-        v_tmp = vals.view(H, n_pages, bs, -1).transpose(0, 1).contiguous()
+        vals = F.linear(lat, self.uv.view(H * s.vdim, R))
+        vals = vals.view(n_pages, bs, H, s.vdim)
+        k_tmp = keys.transpose(1, 2).contiguous()
+        v_tmp = vals.transpose(1, 2).contiguous()
         tables = torch.zeros(
             (n_seq, max(nbs)), dtype=torch.int32, device=q.device
         )
@@ -606,12 +629,26 @@ class SiluGLU(nn.Module):
         return F.linear(ops.glu_silu_scale(F.linear(h, self.gate_up)), self.down)
 
 
+class ExpertRows(NamedTuple):
+    """A mixture's output before its last sum: token t's output is the sum
+    over k of weights[t*top + k] * y[index[t*top + k]], or y[t] itself when
+    ``index`` is None."""
+
+    y: torch.Tensor
+    index: Optional[torch.Tensor] = None
+    weights: Optional[torch.Tensor] = None
+    top: int = 1
+
+
 class SoftmaxRoutedMoE(nn.Module):
     """Mixture of gated silu experts. fp32 router logits over
     ``experts + identity`` outputs, softmax scores; the ``top`` outputs by
     score + correction are chosen and weighted by their scores renormalised
     to sum 1; the weight multiplies the expert's OUTPUT. An identity expert
     returns the token's input. A shared expert is added for every token.
+    ``spec.over_chosen``: the ``top`` largest logits (of the router product
+    plus a bias, with ``spec.router_bias``), weighted by the softmax over those
+    logits.
 
     Weights: gate|up stacked as [E, 2 ff, width] (also one [E * 2 ff, width]
     matrix), down as [width, E, ff] (also one [width, E * ff] matrix).
@@ -636,7 +673,10 @@ class SoftmaxRoutedMoE(nn.Module):
             raise ValueError("top must be between 1 and the router's outputs")
         self.dense_max_tokens = max(16, self.DENSE_ROW_BUDGET * spec.top // max(E, 1))
         self.router = _param(R, width, dtype=torch.float32)
-        self.correction = _param(R, dtype=torch.float32)
+        self.correction = (
+            None if spec.over_chosen else _param(R, dtype=torch.float32)
+        )
+        self.router_b = _param(R, dtype=torch.float32) if spec.router_bias else None
         self.gate_up = _param(E, 2 * spec.ff, width, dtype=dtype)
         self.down = _param(width, E, spec.ff, dtype=dtype)
         self.shared = SiluGLU(width, spec.shared_ff, dtype) if spec.shared_ff else None
@@ -644,7 +684,10 @@ class SoftmaxRoutedMoE(nn.Module):
     def load(self, get, prefix: str):
         dt = self.dtype
         self.router.copy_(get(prefix + "router").float())
-        self.correction.copy_(get(prefix + "correction").float())
+        if self.correction is not None:
+            self.correction.copy_(get(prefix + "correction").float())
+        if self.router_b is not None:
+            self.router_b.copy_(get(prefix + "router.b").float())
         for e in range(self.spec.experts):
             p = f"{prefix}e{e}."
             self.gate_up[e].copy_(
@@ -654,24 +697,19 @@ class SoftmaxRoutedMoE(nn.Module):
         if self.shared is not None:
             self.shared.load(get, prefix + "shared.")
 
-    def _dense(self, h, dense_w, extra):
+    def _dense_rows(self, h, dense_w):
+        """The real experts' weighted sum, in the activation dtype."""
         E, ff = self.spec.experts, self.spec.ff
         T, W = h.shape
-        scaled = scaled_w = None
-        if self.spec.identity:
-            scaled, scaled_w = h, dense_w[:, E:].sum(dim=1)
-        ar = torch.arange(T, dtype=torch.int32, device=h.device)
         if E == 0:
-            y = torch.zeros((T, W), dtype=h.dtype, device=h.device)
-        else:
-            gu = F.linear(h, self.gate_up.view(E * 2 * ff, W))
-            act = ops.glu_silu_scale(
-                gu.view(T * E, 2 * ff), dense_w[:, :E].reshape(-1)
-            )
-            y = F.linear(act.view(T, E * ff), self.down.view(W, E * ff))
-        return ops.combine_rows(y, ar, 1, extra, None, scaled, scaled_w)
+            return torch.zeros((T, W), dtype=h.dtype, device=h.device)
+        gu = F.linear(h, self.gate_up.view(E * 2 * ff, W))
+        act = ops.glu_silu_scale(
+            gu.view(T * E, 2 * ff), dense_w[:, :E].reshape(-1)
+        )
+        return F.linear(act.view(T, E * ff), self.down.view(W, E * ff))
 
-    def _sorted(self, h, idx, w, extra):
+    def _sorted_rows(self, h, idx, w) -> ExpertRows:
         E, top = self.spec.experts, self.spec.top
         R = self.spec.router_outputs
         flat = idx.view(-1).long()
@@ -699,23 +737,45 @@ class SoftmaxRoutedMoE(nn.Module):
         # pair p = t*top + k sits at sorted row inv[p]
         inv = torch.empty_like(order)
         inv[order] = torch.arange(n, device=h.device)
-        return ops.combine_rows(ys, inv.to(torch.int32), top, extra, w.view(-1))
+        return ExpertRows(ys, inv.to(torch.int32), w.view(-1), top)
+
+    def _route(self, h) -> Tuple[torch.Tensor, torch.Tensor, Optional[torch.Tensor]]:
+        dense = h.shape[0] <= self.dense_max_tokens or (
+            h.is_cuda and torch.cuda.is_current_stream_capturing()
+        )
+        over = self.spec.over_chosen
+        idx, w, dense_w, _ = ops.route_tokens(
+            h, self.router, self.spec.top, softmax=not over, renorm=not over,
+            dense=dense, correction=self.correction,
+            renorm_eps=self.RENORM_EPS, over_chosen=over, bias=self.router_b,
+        )
+        return idx, w, dense_w
+
+    def rows(self, h) -> ExpertRows:
+        """The output left for the caller's next kernel to sum up (mixtures
+        without identity or shared experts)."""
+        if self.spec.identity or self.shared is not None:
+            raise ValueError("identity and shared experts need the full sum")
+        idx, w, dense_w = self._route(h)
+        if dense_w is not None:
+            return ExpertRows(self._dense_rows(h, dense_w))
+        return self._sorted_rows(h, idx, w)
 
     def forward(self, h):
         """[T, width] in the activation dtype -> fp32 [T, width]."""
-        T = h.shape[0]
+        T, E = h.shape[0], self.spec.experts
         extra = self.shared(h) if self.shared is not None else None
-        dense = T <= self.dense_max_tokens or (
-            h.is_cuda and torch.cuda.is_current_stream_capturing()
+        idx, w, dense_w = self._route(h)
+        if dense_w is None:
+            r = self._sorted_rows(h, idx, w)
+            return ops.combine_rows(r.y, r.index, r.top, extra, r.weights)
+        scaled = scaled_w = None
+        if self.spec.identity:
+            scaled, scaled_w = h, dense_w[:, E:].sum(dim=1)
+        ar = torch.arange(T, dtype=torch.int32, device=h.device)
+        return ops.combine_rows(
+            self._dense_rows(h, dense_w), ar, 1, extra, None, scaled, scaled_w
         )
-        idx, w, dense_w, _ = ops.route_tokens(
-            h, self.router, self.spec.top, softmax=True, renorm=True,
-            dense=dense, correction=self.correction,
-            renorm_eps=self.RENORM_EPS,
-        )
-        if dense:
-            return self._dense(h, dense_w, extra)
-        return self._sorted(h, idx, w, extra)
 
 
 class RetentionMixer(nn.Module):
@@ -854,6 +914,78 @@ class GatedDeltaMixer(nn.Module):
         )
         on = ops.gated_group_rms_norm(
             o, gate, self.norm_w, self.eps, s.heads, self.dtype, gate_after=True
+        )
+        return F.linear(on, self.o_proj)
+
+
+class GatedLinearMixer(nn.Module):
+    """Linear attention with a decay per head and key channel that depends on
+    the token (no softmax, no denominator): a = sigmoid(z)^(1/tau),
+    z = W_a2 (W_a1 h) + b; the fp32 state S <- diag(a) S + k v^T is read as
+    S^T q dim^-1/2; head outputs are RMS-normed with one weight vector shared
+    by the heads, gated by silu of a projection of the input, out-projected.
+    q|k|v|gate|a1 are one fused GEMM, whose columns the recurrence reads as
+    they are; W_a2 and everything after it are fp32."""
+
+    def __init__(self, width: int, spec: GatedLinearMixerSpec, eps: float, dtype):
+        super().__init__()
+        s = spec
+        self.spec = s
+        self.eps = eps
+        self.dtype = dtype
+        self.width = width
+        self.qk_w = s.heads * s.dim
+        self.v_w = s.heads * s.vdim
+        self.low_at = 2 * self.qk_w + 2 * self.v_w
+        self.a2_b = _param(self.qk_w, dtype=torch.float32)
+        self.norm_w = _param(s.vdim, dtype=torch.float32)
+        self.o_proj = _param(width, self.v_w, dtype=dtype)
+        self._make_projections(s.a_rank or s.dim, None)
+
+    def _make_projections(self, a_rank: int, device):
+        self.a_rank = a_rank
+        # rows padded to whole 16-byte units so that every token's row of the
+        # projection starts aligned
+        self.proj = _param(
+            -(-(self.low_at + a_rank) // 8) * 8, self.width, dtype=self.dtype,
+            device=device,
+        )
+        self.a2 = _param(self.qk_w, a_rank, dtype=torch.float32, device=device)
+
+    def state_shapes(self):
+        s = self.spec
+        return {"ssm": ((s.heads, s.vdim, s.dim), torch.float32)}
+
+    def load(self, get, prefix: str):
+        dt = self.dtype
+        a1 = get(prefix + "a1")
+        if a1.shape[0] != self.a_rank:
+            self._make_projections(a1.shape[0], self.o_proj.device)
+        self.proj.zero_()
+        self.proj[: self.low_at + self.a_rank].copy_(
+            torch.cat([get(prefix + n).to(dt) for n in ("q", "k", "v", "g", "a1")], dim=0)
+        )
+        self.a2.copy_(get(prefix + "a2").float())
+        self.a2_b.copy_(get(prefix + "a2.b").float())
+        self.norm_w.copy_(get(prefix + "norm").float())
+        self.o_proj.copy_(get(prefix + "o").to(dt))
+
+    def forward(self, h, positions, cache: LayerCache, meta):
+        s = self.spec
+        proj = F.linear(h, self.proj)
+        a, b, c = self.qk_w, 2 * self.qk_w, 2 * self.qk_w + self.v_w
+        decay = ops.lowrank_channel_decay(
+            proj[:, self.low_at : self.low_at + self.a_rank], self.a2, self.a2_b,
+            s.tau,
+        )
+        o = ops.linear_scan(
+            proj[:, :a], proj[:, a:b], proj[:, b:c], cache.ssm, positions,
+            meta.cu_seqlens, meta.state_slots, s.heads, channel_decay=decay,
+            q_scale=s.dim ** -0.5,
+        )
+        on = ops.gated_group_rms_norm(
+            o, proj[:, c : self.low_at], self.norm_w, self.eps, s.heads,
+            self.dtype, gate_after=True,
         )
         return F.linear(on, self.o_proj)
 

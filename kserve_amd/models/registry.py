@@ -68,6 +68,12 @@ register(
     "kserve_amd.models.mededra.MededraForCausalLM",
     ("kserve_amd_seq_C",),
 )
+register(
+    "Kebesun",
+    "kserve_amd.engine.config.HybridModelConfig",
+    "kserve_amd.models.kebesun.KebesunForCausalLM",
+    ("kserve_amd_seq_C",),
+)
 
 
 def architecture_of(config_json: dict) -> str:

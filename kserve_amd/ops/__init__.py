@@ -346,19 +346,28 @@ def embed_scale_sinpos(table, tokens, positions, inv_freq, scale: float):
 
 def add_rms_norm_f32res(
     residual, weight, eps: float, w_offset: float, out_dtype,
-    d0=None, s0: float = 1.0, d1=None, s1: float = 1.0,
+    d0=None, s0: float = 1.0, d1=None, s1: float = 1.0, c0=None, c1=None,
+    d1_index=None, d1_weights=None, d1_top: int = 1, want_out: bool = True,
 ):
-    """residual (fp32, in place) += s0*d0 + s1*d1, then RMS norm with weight
-    (w_offset + w); returns the normed rows in ``out_dtype``."""
+    """residual (fp32, in place) += s0*c0*d0 + s1*c1*d1 (``c0``, ``c1``: fp32
+    factors per channel, None for 1), then RMS norm with weight (w_offset + w);
+    returns the normed rows in ``out_dtype`` (``weight`` None: the new residual
+    itself; ``want_out`` off: nothing). With ``d1_index`` [T*d1_top] int32 the
+    second delta of token t is the sum over k of d1_weights[t*d1_top + k] *
+    d1[d1_index[t*d1_top + k]] (fp32 weights or None for 1)."""
     if residual.is_cuda:
-        out = torch.empty(residual.shape, dtype=out_dtype, device=residual.device)
+        out = (
+            torch.empty(residual.shape, dtype=out_dtype, device=residual.device)
+            if want_out else None
+        )
         _native_seq("add_rms_norm_f32res").add_rms_norm_f32res(
             residual, d0, float(s0), d1, float(s1), weight, float(w_offset),
-            float(eps), out,
+            float(eps), out, c0, c1, d1_index, d1_weights, int(d1_top),
         )
         return out
     return torch_ref.add_rms_norm_f32res(
-        residual, weight, eps, w_offset, out_dtype, d0, s0, d1, s1
+        residual, weight, eps, w_offset, out_dtype, d0, s0, d1, s1, c0, c1,
+        d1_index, d1_weights, d1_top, want_out,
     )
 
 
@@ -441,13 +450,14 @@ def ctx_attention_f32(
     q, k_cache, v_cache, block_tables, cu_q, ctx_lens, scale: float,
     max_q_len: int, heads: int, gate=None, out_dtype=torch.float32,
     sink=None, chunk: int = 0, out_inv_freq=None, window: int = 0,
-    maps: int = 1, softcap: float = 0.0,
+    maps: int = 1, softcap: float = 0.0, keep_first: int = 0,
 ):
     """Paged causal attention with fp32 scores and weights. Optional parts:
     ``gate`` [T, heads] (output times sigmoid), ``sink`` [heads] fp32 (one
     more term exp(sink) in the softmax denominator), ``chunk`` (a query sees
     only keys of its own block of that many positions), ``window`` (a query
-    sees itself and the window-1 positions before it), ``out_inv_freq``
+    sees itself and the window-1 positions before it, and with ``keep_first``
+    the sequence's first positions), ``out_inv_freq``
     [vdim/2] fp32 (each head output turned back by its query position).
     ``v_cache`` may be a view of the leading columns of ``k_cache`` (values
     that are a prefix of the keys are stored once). ``maps``: every cached key
@@ -464,11 +474,13 @@ def ctx_attention_f32(
             out, q, k_cache, v_cache, block_tables, cu_q, ctx_lens, gate,
             float(scale), int(max_q_len), int(heads), sink, int(chunk),
             out_inv_freq, int(window), int(maps), float(softcap),
+            int(keep_first),
         )
         return out
     return torch_ref.ctx_attention_f32(
         q, k_cache, v_cache, block_tables, cu_q, ctx_lens, scale, heads,
         gate, out_dtype, sink, chunk, out_inv_freq, window, maps, softcap,
+        keep_first,
     )
 
 
@@ -476,8 +488,9 @@ def qk_headnorm_rope_cache(
     q, k, v, qw, kw, positions, slot_mapping, k_cache, v_cache, eps: float,
     heads: int, qk_inv_freq=None, v_unit_norm: bool = False, v_inv_freq=None,
     pairs: bool = False, rot_mult: float = 1.0, maps: int = 1,
+    qk_norm: bool = True,
 ):
-    """Per-head q/k RMS norm (weights [dim]) + rotary positions (``pairs``:
+    """Per-head q/k RMS norm (weights [dim]; off with ``qk_norm``) + rotary positions (``pairs``:
     coordinate 2i turns with 2i+1 instead of i with i + half; turned
     coordinates times ``rot_mult``), optional unit-norm and rotation of the
     values, KV page scatter (``maps`` k heads share a cached row and a value
@@ -487,12 +500,13 @@ def qk_headnorm_rope_cache(
         _native_seq("qk_headnorm_rope_cache").qk_headnorm_rope_cache(
             q_out, q, k, v, qw, kw, positions, slot_mapping, k_cache, v_cache,
             float(eps), int(heads), qk_inv_freq, bool(v_unit_norm), v_inv_freq,
-            bool(pairs), float(rot_mult), int(maps),
+            bool(pairs), float(rot_mult), int(maps), bool(qk_norm),
         )
         return q_out
     return torch_ref.qk_headnorm_rope_cache(
         q, k, v, qw, kw, positions, slot_mapping, k_cache, v_cache, eps,
         heads, qk_inv_freq, v_unit_norm, v_inv_freq, pairs, rot_mult, maps,
+        qk_norm,
     )
 
 
@@ -524,11 +538,13 @@ def post_norm_add_rms_norm(
 def router_topk(
     logits, top: int, softmax: bool = False, renorm: bool = False,
     dense: bool = False, correction=None, renorm_eps: float = 0.0,
-    weight_scale: float = 1.0,
+    weight_scale: float = 1.0, over_chosen: bool = False,
 ):
     """fp32 router logits [T, E] -> (expert ids int32 [T, top], weights fp32
     [T, top], dense [T, E] weights or None) by sigmoid (or softmax) score;
-    with ``correction`` [E] fp32 the choice goes by score + correction."""
+    with ``correction`` [E] fp32 the choice goes by score + correction.
+    ``over_chosen``: the largest logits, weighted by the softmax over those
+    logits only."""
     if logits.is_cuda:
         T, E = logits.shape
         idx = torch.empty((T, top), dtype=torch.int32, device=logits.device)
@@ -539,12 +555,12 @@ def router_topk(
         )
         _native_seq("router_topk").router_topk(
             idx, w, dw, logits, bool(softmax), bool(renorm), correction,
-            float(renorm_eps), float(weight_scale),
+            float(renorm_eps), float(weight_scale), bool(over_chosen),
         )
         return idx, w, dw
     return torch_ref.router_topk(
         logits, top, softmax, renorm, dense, correction, renorm_eps,
-        weight_scale,
+        weight_scale, over_chosen,
     )
 
 
@@ -552,9 +568,11 @@ def route_tokens(
     h, router, top: int, softmax: bool = False, renorm: bool = False,
     dense: bool = False, want_logits: bool = False, correction=None,
     renorm_eps: float = 0.0, weight_scale: float = 1.0,
+    over_chosen: bool = False, bias=None,
 ):
     """The router in one kernel: fp32 logits of h [T, W] (activation dtype)
-    against fp32 router rows [E, W], scores, the ``top`` experts. Returns
+    against fp32 router rows [E, W] (+ fp32 ``bias`` [E]), scores, the ``top``
+    experts (as in ``router_topk``). Returns
     (expert ids int32 [T, top], weights fp32 [T, top], dense [T, E] weights or
     None, logits fp32 [T, E] or None)."""
     if h.is_cuda:
@@ -566,12 +584,12 @@ def route_tokens(
         lg = torch.empty((T, E), dtype=torch.float32, device=dev) if want_logits else None
         _native_seq("route_tokens").route_tokens(
             idx, w, dw, lg, h, router, bool(softmax), bool(renorm), correction,
-            float(renorm_eps), float(weight_scale),
+            float(renorm_eps), float(weight_scale), bool(over_chosen), bias,
         )
         return idx, w, dw, lg
     return torch_ref.route_tokens(
         h, router, top, softmax, renorm, dense, want_logits, correction,
-        renorm_eps, weight_scale,
+        renorm_eps, weight_scale, over_chosen, bias,
     )
 
 
@@ -636,32 +654,40 @@ def post_layer_norm_add(
 
 def latent_norm_rope_cache(
     proj, q_rank: int, kv_rank: int, rot_dim: int, qw, kw, positions,
-    slot_mapping, cache, eps: float, inv_freq,
+    slot_mapping, cache, eps: float, inv_freq, pairs: bool = True,
+    rot_mult: float = 1.0,
 ):
     """Rows [query latent | kv latent | key part | ...] -> the RMS-normed
-    query latent (returned, activation dtype) and, when ``cache`` is given,
-    [normed kv latent | key part rotated in pairs (2i, 2i+1)] scattered into
-    the paged cache [blocks, 1, block, kv_rank + rot_dim]."""
+    query latent (returned, activation dtype; None when ``q_rank`` is 0) and,
+    when ``cache`` is given, [normed kv latent | key part rotated in pairs
+    (2i, 2i+1)] scattered into the paged cache [blocks, 1, block,
+    kv_rank + rot_dim]. ``pairs`` off: coordinate i turns with i + half;
+    turned coordinates times ``rot_mult``."""
     if proj.is_cuda:
-        cq = torch.empty((proj.shape[0], q_rank), dtype=proj.dtype, device=proj.device)
+        cq = (
+            torch.empty((proj.shape[0], q_rank), dtype=proj.dtype, device=proj.device)
+            if q_rank else None
+        )
         _native_seq("latent_norm_rope_cache").latent_norm_rope_cache(
             cq, proj, int(q_rank), int(kv_rank), int(rot_dim), qw, kw,
-            positions, slot_mapping, cache, float(eps), inv_freq,
+            positions, slot_mapping, cache, float(eps), inv_freq, bool(pairs),
+            float(rot_mult),
         )
         return cq
     return torch_ref.latent_norm_rope_cache(
         proj, q_rank, kv_rank, rot_dim, qw, kw, positions, slot_mapping,
-        cache, eps, inv_freq,
+        cache, eps, inv_freq, pairs, rot_mult,
     )
 
 
 def head_matmul_rope(
     x, w, heads: int, tail: int = 0, positions=None, inv_freq=None,
-    out_dtype=None,
+    out_dtype=None, pairs: bool = True, rot_mult: float = 1.0,
 ):
     """Per-head matrix product with an optional rotated tail:
     x [T, heads*(k + tail)], w [heads, n, k] -> [T, heads*(n + tail)], the
-    tail coordinates turned in pairs by the token's position."""
+    tail coordinates turned in pairs (``pairs`` off: i with i + half) by the
+    token's position and multiplied by ``rot_mult``."""
     out_dtype = out_dtype or x.dtype
     if x.is_cuda:
         n = w.shape[1]
@@ -669,11 +695,12 @@ def head_matmul_rope(
             (x.shape[0], heads * (n + tail)), dtype=out_dtype, device=x.device
         )
         _native_seq("head_matmul_rope").head_matmul_rope(
-            out, x, w, int(heads), int(tail), positions, inv_freq
+            out, x, w, int(heads), int(tail), positions, inv_freq, bool(pairs),
+            float(rot_mult),
         )
         return out
     return torch_ref.head_matmul_rope(
-        x, w, heads, tail, positions, inv_freq, out_dtype
+        x, w, heads, tail, positions, inv_freq, out_dtype, pairs, rot_mult
     )
 
 
@@ -738,7 +765,7 @@ def unit_norm_heads(
 def linear_scan(
     q, k, v, state, positions, cu_seqlens, slots, qk_heads: int,
     decay=None, a_raw=None, b_raw=None, a_log=None, dt_bias=None,
-    channel_decay=None,
+    channel_decay=None, q_scale: float = 1.0,
 ):
     """Linear-attention recurrence over a flat varlen batch; carries
     ``state[slot]`` ([heads, V, K] fp32). q, k [T, qk_heads*K] and
@@ -747,19 +774,43 @@ def linear_scan(
     g = exp(-exp(a_log) softplus(a_raw + dt_bias)), b = sigmoid(b_raw):
     S <- g S; S <- S + k (b (v - S^T k))^T; ``channel_decay`` [T, heads*K] fp32
     gives g per head and key channel (then a_raw, a_log, dt_bias are not
-    used). Output o = S^T q, fp32."""
+    used); ``channel_decay`` without ``b_raw``: S <- diag(g) S + k v^T, and
+    q, k, v may be bf16. Output o = S^T q * q_scale, fp32."""
     if q.is_cuda:
         heads, V = state.shape[1], state.shape[2]
         o = _f32_like(q.shape[0], heads * V, q)
         _native_seq("linear_scan").linear_scan(
             o, q, k, v, decay, a_raw, b_raw, a_log, dt_bias, channel_decay,
-            state, positions, cu_seqlens, slots, int(qk_heads),
+            state, positions, cu_seqlens, slots, int(qk_heads), float(q_scale),
         )
         return o
     return torch_ref.linear_scan(
         q, k, v, state, positions, cu_seqlens, slots, qk_heads, decay, a_raw,
-        b_raw, a_log, dt_bias, channel_decay,
+        b_raw, a_log, dt_bias, channel_decay, q_scale,
     )
+
+
+def lowrank_channel_decay(low, w2, bias, tau: float):
+    """Decays of a gated linear recurrence: sigmoid(z)^(1/tau) with
+    z = low @ w2^T + bias in fp32; low [T, r] in the activation dtype (rows may
+    be strided), w2 [n, r] and bias [n] fp32 -> fp32 [T, n]."""
+    if low.is_cuda:
+        out = _f32_like(low.shape[0], w2.shape[0], low)
+        _native_seq("lowrank_channel_decay").lowrank_channel_decay(
+            out, low, w2, bias, float(tau)
+        )
+        return out
+    return torch_ref.lowrank_channel_decay(low, w2, bias, tau)
+
+
+def linear_f32out(x, w):
+    """x @ w^T with an fp32 result that is never rounded to the activation
+    dtype (a product that replaces an fp32 stream, or logits)."""
+    if x.dtype == torch.float32:
+        return torch.nn.functional.linear(x, w)
+    if x.is_cuda:
+        return torch.mm(x, w.t(), out_dtype=torch.float32)
+    return torch_ref.linear_f32out(x, w)
 
 
 def relu2_scale(x, scales=None):

@@ -7,7 +7,8 @@
 //        1 + coef * ln(floor((pos + 1) / every) + 1),
 //    write q (fp32) out and scatter k / v into the paged cache.
 //  * qk_headnorm_rope_cache: per token and per HEAD, RMS-normalise q and k
-//    with a weight of the head size shared by the heads, rotate the first
+//    with a weight of the head size shared by the heads (or leave them
+//    un-normed), rotate the first
 //    2*half coordinates (coordinate i pairs with i + half, angle
 //    pos * inv_freq[i] in fp32), optionally divide each value head by its
 //    RMS and rotate it by the token's position over its whole width, write
@@ -38,7 +39,10 @@
 //    partial (max, sum, O) through LDS at the end, so the group's K/V is read
 //    once. Head sizes are padded up to 64/128/256 with zeros. An optional
 //    per-(token, head) gate multiplies the result by sigmoid(gate).
-//    Optional: scores soft-capped with cap * tanh(score / cap); and `maps` keys
+//    Optional: a window's kept first positions (the tiles of [0, keep_first)
+//    come ahead of the window's own when the two ranges are apart, otherwise
+//    one run of tiles covers both);
+//    scores soft-capped with cap * tanh(score / cap); and `maps` keys
 //    side by side in one cached row, query head h reading number h % maps.
 //    Prefill reads the map's columns of the row as a head of its own; decode
 //    keeps all maps of a group in one block, reads the whole row once and
@@ -158,7 +162,7 @@ __global__ void qk_headnorm_rope_cache_kernel(
     T* __restrict__ v_cache, float eps, int heads, int kv_heads, int D, int DV,
     int block_size, const float* __restrict__ qk_inv_freq, int qk_half,
     int v_unit_norm, const float* __restrict__ v_inv_freq, int v_half,
-    int pairs, float rot_mult, int maps) {
+    int pairs, float rot_mult, int maps, int qk_norm) {
   extern __shared__ float lds[];
   if (!qk_inv_freq) qk_half = 0;
   if (!v_inv_freq) v_half = 0;
@@ -187,7 +191,7 @@ __global__ void qk_headnorm_rope_cache_kernel(
     const float* w = nullptr;
     const float* cs;
     int width, half;
-    bool norm = true;
+    bool norm = qk_norm != 0;
     float* dst_f = nullptr;
     T* dst_c = nullptr;
     if (job < heads) {
@@ -357,7 +361,7 @@ __global__ void __launch_bounds__(NT) ctx_attention_f32_kernel(
     int kv_heads, int D, int DV, int block_size, int hpb,
     const float* __restrict__ sink, int chunk,
     const float* __restrict__ out_inv_freq, int window, long v_row_stride,
-    float* __restrict__ ws, int maps, float softcap, int out_f32) {
+    float* __restrict__ ws, int maps, float softcap, int out_f32, int keep) {
   // D: columns of a key row this launch reads per query (decode: all maps of
   // a row; prefill: one map, at columns (head % maps) D of rows of maps * D)
   extern __shared__ float lds[];
@@ -383,7 +387,6 @@ __global__ void __launch_bounds__(NT) ctx_attention_f32_kernel(
   // x takes the tiles x, x + nsplit, ... of the visible keys
   const int nsplit = SPLITK ? gridDim.x : 1;
   const int split = SPLITK ? blockIdx.x : 0;
-  const int kstep = nsplit * BK;
   const int tok0 = SPLITK ? 0 : blockIdx.x * tpb;
   if (tok0 >= q_len) return;
   const int head0 = blockIdx.z * hpb;
@@ -411,9 +414,15 @@ __global__ void __launch_bounds__(NT) ctx_attention_f32_kernel(
                      : chunk > 0  ? qpos / chunk * chunk
                      : window > 0 ? max(qpos - window + 1, 0)
                                   : 0;
-  const int kbeg = chunk > 0    ? base_pos / chunk * chunk
-                   : window > 0 ? max(base_pos - window + 1, 0)
-                                : 0;
+  int kbeg = chunk > 0    ? base_pos / chunk * chunk
+             : window > 0 ? max(base_pos - window + 1, 0)
+                          : 0;
+  // kept first positions [0, keep) (0 without a window): tiles of their own
+  // ahead of the window's, or part of one run of tiles when the ranges touch
+  if (kbeg <= keep) kbeg = 0;
+  const int kept = kbeg > 0 ? keep : 0;
+  const int kept_tiles = (kept + BK - 1) / BK;
+  const int ntiles = kept_tiles + (last_pos - kbeg + BK) / BK;
   // keys this wave needs: from its first row's chunk up to its own last
   // row's position
   const int wave_last =
@@ -488,22 +497,26 @@ __global__ void __launch_bounds__(NT) ctx_attention_f32_kernel(
   // the next tile's global loads are in flight while this one is computed
   TileStage<T, DP> kst;
   TileStage<T, DVP> vst;
-  const int kfirst = kbeg + split * BK;
-  kst.fetch(kc, bt, kfirst, min(BK, last_pos + 1 - kfirst), g, kv_heads, D, k_row_stride, block_size, bs_shift, kvec);
-  if (!VK)
-    vst.fetch(v_cache, bt, kfirst, min(BK, last_pos + 1 - kfirst), g, kv_heads, DV, v_row_stride, block_size, bs_shift, vvec);
-  for (int k0 = kfirst; k0 <= last_pos; k0 += kstep) {
+  // tile -> its first key and the end of its range
+  auto tile_at = [&](int t) {
+    return t < kept_tiles ? t * BK : kbeg + (t - kept_tiles) * BK;
+  };
+  auto tile_end = [&](int t) { return t < kept_tiles ? kept : last_pos + 1; };
+  auto fetch_tile = [&](int t) {
+    const int ks = tile_at(t), nn = min(BK, tile_end(t) - ks);
+    kst.fetch(kc, bt, ks, nn, g, kv_heads, D, k_row_stride, block_size, bs_shift, kvec);
+    if (!VK)
+      vst.fetch(v_cache, bt, ks, nn, g, kv_heads, DV, v_row_stride, block_size, bs_shift, vvec);
+  };
+  if (split < ntiles) fetch_tile(split);
+  for (int tl = split; tl < ntiles; tl += nsplit) {
+    const int k0 = tile_at(tl), kend = tile_end(tl);
     __syncthreads();  // previous tile fully consumed
     kst.store(Ks);
     if (!VK) vst.store(Vs);
     __syncthreads();
-    if (k0 + kstep <= last_pos) {
-      const int nn = min(BK, last_pos + 1 - (k0 + kstep));
-      kst.fetch(kc, bt, k0 + kstep, nn, g, kv_heads, D, k_row_stride, block_size, bs_shift, kvec);
-      if (!VK)
-        vst.fetch(v_cache, bt, k0 + kstep, nn, g, kv_heads, DV, v_row_stride, block_size, bs_shift, vvec);
-    }
-    if (k0 > wave_last || k0 + BK <= wave_first) continue;
+    if (tl + nsplit < ntiles) fetch_tile(tl + nsplit);
+    if (k0 > wave_last || (k0 + BK <= wave_first && k0 >= keep)) continue;
 
     // S^T sub-tiles: acc[kt][v] = score(key k0 + 16 kt' + 4 lg + v, query li)
     // k-steps outermost, two accumulators per sub-tile: 2 KT independent
@@ -541,7 +554,8 @@ __global__ void __launch_bounds__(NT) ctx_attention_f32_kernel(
 #pragma unroll
       for (int v = 0; v < 4; ++v) {
         const int kp = k0 + 16 * kt + 4 * lg + v;
-        sc[t][v] = (kp <= qpos && kp >= qstart) ? sc[t][v] : -INFINITY;
+        const bool vis = kp <= qpos && kp < kend && (kp >= qstart || kp < keep);
+        sc[t][v] = vis ? sc[t][v] : -INFINITY;
         mt = fmaxf(mt, sc[t][v]);
       }
     }
@@ -807,7 +821,7 @@ extern "C" hipError_t ks_qk_headnorm_rope_cache(
     int tokens, int heads, int kv_heads, int D, int DV, int block_size,
     const void* qk_inv_freq, int qk_half, int v_unit_norm,
     const void* v_inv_freq, int v_half, int pairs, float rot_mult, int maps,
-    int in_f32, int is_f32, hipStream_t stream) {
+    int qk_norm, int in_f32, int is_f32, hipStream_t stream) {
   if (tokens == 0) return hipSuccess;
   if (2 * qk_half > D || 2 * v_half > DV || maps < 1 ||
       (pairs && v_inv_freq) || (is_f32 && !in_f32))
@@ -817,7 +831,8 @@ extern "C" hipError_t ks_qk_headnorm_rope_cache(
       (const float*)qw, (const float*)kw, (const long*)positions,            \
       (const int*)slot_mapping, (TT*)k_cache, (TT*)v_cache, eps, heads,      \
       kv_heads, D, DV, block_size, (const float*)qk_inv_freq, qk_half,       \
-      v_unit_norm, (const float*)v_inv_freq, v_half, pairs, rot_mult, maps
+      v_unit_norm, (const float*)v_inv_freq, v_half, pairs, rot_mult, maps,  \
+      qk_norm
 #define HN_LAUNCH(TI, TT)                                                    \
   do {                                                                       \
     if (vec)                                                                 \
@@ -860,12 +875,16 @@ static int decode_heads_per_block(int heads, int kv_heads) {
 // without keys writes an empty partial.
 extern "C" int ks_ctx_attention_decode_splits(int num_seqs, int heads,
                                               int kv_heads, int window,
+                                              int keep_first,
                                               int has_out_rotation) {
   if (has_out_rotation) return 1;
   const int blocks = num_seqs * (heads / decode_heads_per_block(heads, kv_heads));
   int n = cdiv(1024, blocks > 0 ? blocks : 1);
   if (n > 8) n = 8;
-  if (window > 0 && n > cdiv(window, BK)) n = cdiv(window, BK);
+  if (window > 0) {
+    const int tiles = cdiv(window, BK) + cdiv(keep_first, BK);
+    if (n > tiles) n = tiles;
+  }
   return n < 1 ? 1 : n;
 }
 
@@ -888,6 +907,7 @@ struct CtxArgs {
   int maps;
   float softcap;
   int out_f32;
+  int keep;
   bool decode;  // one token per sequence, in the split-key form
 };
 
@@ -930,7 +950,7 @@ hipError_t launch_ctx_attention(const CtxArgs& a) {
                      a.kv_heads, a.D, a.DV, a.block_size, hpb,
                      (const float*)a.sink, a.chunk,
                      (const float*)a.out_inv_freq, a.window, a.v_row_stride,
-                     (float*)a.ws, a.maps, a.softcap, a.out_f32);
+                     (float*)a.ws, a.maps, a.softcap, a.out_f32, a.keep);
   hipError_t e = hipGetLastError();
   if (e != hipSuccess || nsplit <= 1) return e;
   hipLaunchKernelGGL(ctx_attention_merge_kernel<T>,
@@ -974,7 +994,8 @@ extern "C" hipError_t ks_ctx_attention_f32(
     int num_seqs, int max_q_len, int heads, int kv_heads, int D, int DV,
     int block_size, int is_f32, const void* sink, int chunk,
     const void* out_inv_freq, int window, long v_row_stride, void* ws,
-    int nsplit, int maps, float softcap, int out_f32, hipStream_t stream) {
+    int nsplit, int maps, float softcap, int out_f32, int keep_first,
+    hipStream_t stream) {
   if (num_seqs == 0 || max_q_len == 0) return hipSuccess;
   // D: columns of one key (a cached row holds maps of them)
   if (maps < 1 || heads % (kv_heads > 0 ? kv_heads * maps : 1) != 0)
@@ -987,12 +1008,13 @@ extern "C" hipError_t ks_ctx_attention_f32(
       heads % kv_heads != 0 || chunk < 0 || window < 0 ||
       (chunk > 0 && window > 0) || v_row_stride < DV ||
       (out_inv_freq && DV % 2 != 0) || nsplit < 1 || (nsplit > 1 && !ws) ||
-      (nsplit > 1 && out_inv_freq))
+      (nsplit > 1 && out_inv_freq) || keep_first < 0 ||
+      (keep_first > 0 && window == 0))
     return hipErrorInvalidValue;
   const CtxArgs a{out, q, k_cache, v_cache, block_tables, bt_stride, cu_q,
                   ctx_lens, gate, gate_stride, scale, num_seqs, max_q_len,
                   heads, kv_heads, D, DV, block_size, sink, chunk,
                   out_inv_freq, window, v_row_stride, ws, nsplit, stream,
-                  maps, softcap, out_f32, decode};
+                  maps, softcap, out_f32, keep_first, decode};
   return is_f32 ? dispatch_d<float>(a) : dispatch_d<short>(a);
 }

@@ -9,8 +9,10 @@ hipError_t ks_embed_scale_sinpos(void*, const void*, const void*, const void*,
                                  const void*, float, int, int, int,
                                  hipStream_t);
 hipError_t ks_add_rms_norm_f32res(void*, const void*, long, float, const void*,
-                                  long, float, const void*, float, float,
-                                  void*, int, int, int, int, hipStream_t);
+                                  long, float, const void*, const void*,
+                                  const void*, const void*, int, const void*,
+                                  float, float, void*, int, int, int, int,
+                                  hipStream_t);
 hipError_t ks_gated_group_rms_norm(void*, const void*, const void*, long,
                                    const void*, int, float, int, int, int, int,
                                    int, int, hipStream_t);
@@ -32,24 +34,25 @@ hipError_t ks_ctx_attention_f32(void*, const void*, const void*, const void*,
                                 const void*, long, float, int, int, int, int,
                                 int, int, int, int, const void*, int,
                                 const void*, int, long, void*, int, int, float,
-                                int, hipStream_t);
-int ks_ctx_attention_decode_splits(int, int, int, int, int);
+                                int, int, hipStream_t);
+int ks_ctx_attention_decode_splits(int, int, int, int, int, int);
 hipError_t ks_qk_headnorm_rope_cache(void*, const void*, const void*,
                                      const void*, long, const void*,
                                      const void*, const void*, const void*,
                                      void*, void*, float, int, int, int, int,
                                      int, int, const void*, int, int,
                                      const void*, int, int, float, int, int,
-                                     int, hipStream_t);
+                                     int, int, hipStream_t);
 hipError_t ks_post_norm_add_rms_norm(void*, const void*, long, int, float,
                                      const void*, const void*, const void*,
                                      float, float, void*, int, int, int,
                                      hipStream_t);
 hipError_t ks_router_topk(void*, void*, void*, const void*, int, int, int, int,
-                          int, const void*, float, float, hipStream_t);
+                          int, const void*, float, float, int, hipStream_t);
 hipError_t ks_route_tokens(void*, void*, void*, void*, const void*, long,
                            const void*, int, int, int, int, int, int,
-                           const void*, float, float, int, hipStream_t);
+                           const void*, float, float, int, const void*, int,
+                           hipStream_t);
 hipError_t ks_gather_scale_rows(void*, const void*, long, const void*,
                                 const void*, int, int, int, hipStream_t);
 hipError_t ks_combine_rows(void*, const void*, const void*, int, const void*,
@@ -61,10 +64,11 @@ hipError_t ks_post_layer_norm_add(void*, const void*, long, int, const void*,
 hipError_t ks_latent_norm_rope_cache(void*, const void*, long, int, int, int,
                                      int, const void*, const void*,
                                      const void*, const void*, void*, float,
-                                     const void*, int, int, hipStream_t);
+                                     const void*, int, int, float, int,
+                                     hipStream_t);
 hipError_t ks_head_matmul_rope(void*, const void*, long, const void*, int, int,
                                int, int, int, const void*, const void*, int,
-                               int, int, hipStream_t);
+                               int, float, int, int, hipStream_t);
 hipError_t ks_glu_silu_scale(void*, const void*, const void*, int, int, int,
                              hipStream_t);
 hipError_t ks_bias_gelu_tanh(void*, const void*, const void*, int, int, int,
@@ -81,10 +85,14 @@ hipError_t ks_rope_scale_heads(void*, const void*, long, const void*,
 hipError_t ks_unit_norm_heads(void*, long, int, int, float, int, float, int,
                               float, hipStream_t);
 hipError_t ks_linear_scan(void*, const void*, long, const void*, long,
-                          const void*, long, const void*, const void*,
-                          const void*, long, int, const void*, const void*,
-                          const void*, void*, const void*, const void*,
-                          const void*, int, int, int, int, int, hipStream_t);
+                          const void*, long, int, float, const void*,
+                          const void*, const void*, long, int, const void*,
+                          const void*, const void*, void*, const void*,
+                          const void*, const void*, int, int, int, int, int,
+                          hipStream_t);
+hipError_t ks_lowrank_channel_decay(void*, const void*, long, const void*,
+                                    const void*, float, int, int, int, int,
+                                    hipStream_t);
 hipError_t ks_delta_unit_decay(void*, long, void*, const void*, long,
                                const void*, const void*, int, int, int, float,
                                float, int, int, hipStream_t);
@@ -162,15 +170,32 @@ void embed_scale_sinpos(at::Tensor& out, at::Tensor& table, at::Tensor& tokens,
 void add_rms_norm_f32res(at::Tensor& residual,
                          const c10::optional<at::Tensor>& d0, double s0,
                          const c10::optional<at::Tensor>& d1, double s1,
-                         at::Tensor& weight, double w_offset, double eps,
-                         at::Tensor& out) {
+                         const c10::optional<at::Tensor>& weight,
+                         double w_offset, double eps,
+                         const c10::optional<at::Tensor>& out,
+                         const c10::optional<at::Tensor>& c0,
+                         const c10::optional<at::Tensor>& c1,
+                         const c10::optional<at::Tensor>& index,
+                         const c10::optional<at::Tensor>& row_w, int64_t top) {
   CHECK_F32(residual);
-  CHECK_F32(weight);
-  TORCH_CHECK(residual.dim() == 2 && out.is_contiguous(), "residual [T, W]");
+  TORCH_CHECK(residual.dim() == 2, "residual [T, W]");
   const int rows = residual.size(0), width = residual.size(1);
-  TORCH_CHECK(weight.numel() == width && out.numel() == residual.numel(),
-              "add_rms_norm_f32res: shape mismatch");
-  const int f32 = act_is_f32(out, "out");
+  // fp32 vectors of one entry per channel
+  auto channels = [&](const c10::optional<at::Tensor>& v) -> const void* {
+    if (!v.has_value()) return nullptr;
+    CHECK_F32(*v);
+    TORCH_CHECK(v->numel() == width, "add_rms_norm_f32res: vector [W]");
+    return v->data_ptr();
+  };
+  // no output: only the deltas are added (their dtype then stands for it)
+  int f32 = 1;
+  if (out.has_value()) {
+    TORCH_CHECK(out->is_contiguous() && out->numel() == residual.numel(),
+                "add_rms_norm_f32res: shape mismatch");
+    f32 = act_is_f32(*out, "out");
+  } else if (d0.has_value() || d1.has_value()) {
+    f32 = act_is_f32(d0.has_value() ? *d0 : *d1, "delta");
+  }
   // the deltas share a dtype: the output's, or fp32 beside a bf16 output
   int df32 = f32;
   if (d0.has_value()) df32 = act_is_f32(*d0, "d0");
@@ -188,16 +213,31 @@ void add_rms_norm_f32res(at::Tensor& residual,
   }
   if (d1.has_value()) {
     CHECK_ROWS(*d1);
-    TORCH_CHECK(act_is_f32(*d1, "d1") == df32 && d1->size(0) == rows &&
+    TORCH_CHECK(act_is_f32(*d1, "d1") == df32 &&
+                    (index.has_value() || d1->size(0) == rows) &&
                     d1->size(1) == width,
                 "d1: dtype/shape mismatch");
     p1 = d1->data_ptr();
     st1 = d1->stride(0);
   }
-  check_hip(ks_add_rms_norm_f32res(residual.data_ptr(), p0, st0, (float)s0, p1,
-                                   st1, (float)s1, weight.data_ptr(),
-                                   (float)w_offset, (float)eps, out.data_ptr(),
-                                   rows, width, f32, df32, current_stream()),
+  const void *ip = nullptr, *wp = nullptr;
+  if (index.has_value()) {
+    CHECK_I32(*index);
+    TORCH_CHECK(p1 && top >= 1 && index->numel() == (int64_t)rows * top,
+                "index [T * top] int32 of rows of d1");
+    ip = index->data_ptr();
+    if (row_w.has_value()) {
+      CHECK_F32(*row_w);
+      TORCH_CHECK(row_w->numel() == index->numel(), "row weights [T * top]");
+      wp = row_w->data_ptr();
+    }
+  }
+  check_hip(ks_add_rms_norm_f32res(
+                residual.data_ptr(), p0, st0, (float)s0, p1, st1, (float)s1,
+                channels(c0), channels(c1), ip, wp, (int)top, channels(weight),
+                (float)w_offset, (float)eps,
+                out.has_value() ? out->data_ptr() : nullptr, rows, width, f32,
+                df32, current_stream()),
             "add_rms_norm_f32res");
 }
 
@@ -355,7 +395,8 @@ void ctx_attention_f32(at::Tensor& out, at::Tensor& q, at::Tensor& k_cache,
                        int64_t max_q_len, int64_t heads,
                        const c10::optional<at::Tensor>& sink, int64_t chunk,
                        const c10::optional<at::Tensor>& out_inv_freq,
-                       int64_t window, int64_t maps, double softcap) {
+                       int64_t window, int64_t maps, double softcap,
+                       int64_t keep_first) {
   CHECK_F32(q);
   CHECK_I32(cu_q);
   CHECK_I32(ctx_lens);
@@ -413,13 +454,16 @@ void ctx_attention_f32(at::Tensor& out, at::Tensor& q, at::Tensor& k_cache,
   }
   TORCH_CHECK(chunk >= 0 && window >= 0 && !(chunk > 0 && window > 0),
               "chunk / window: not negative, at most one of them");
+  TORCH_CHECK(keep_first >= 0, "kept first positions: not negative");
+  if (window == 0) keep_first = 0;  // everything before the query is visible
   // a decode batch splits every sequence's keys over several blocks, which
   // leave partial results in a scratch tensor for a merge pass
   int nsplit = 1;
   at::Tensor ws;
   if (max_q_len == 1 && maps * D <= 256) {
     nsplit = ks_ctx_attention_decode_splits(num_seqs, (int)heads, G,
-                                            (int)window, fp != nullptr);
+                                            (int)window, (int)keep_first,
+                                            fp != nullptr);
     if (nsplit > 1)
       ws = at::empty({(int64_t)num_seqs * heads * nsplit * (DV + 2)},
                      q.options().dtype(at::kFloat));
@@ -432,7 +476,7 @@ void ctx_attention_f32(at::Tensor& out, at::Tensor& q, at::Tensor& k_cache,
                 (int)max_q_len, (int)heads, G, D, DV, bs, f32, sp, (int)chunk,
                 fp, (int)window, (long)vrs,
                 nsplit > 1 ? ws.data_ptr() : nullptr, nsplit, (int)maps,
-                (float)softcap, out_f32, current_stream()),
+                (float)softcap, out_f32, (int)keep_first, current_stream()),
             "ctx_attention_f32");
 }
 
@@ -446,7 +490,8 @@ void qk_headnorm_rope_cache(at::Tensor& q_out, at::Tensor& q, at::Tensor& k,
                             const c10::optional<at::Tensor>& qk_inv_freq,
                             bool v_unit_norm,
                             const c10::optional<at::Tensor>& v_inv_freq,
-                            bool pairs, double rot_mult, int64_t maps) {
+                            bool pairs, double rot_mult, int64_t maps,
+                            bool qk_norm) {
   CHECK_F32(q_out);
   TORCH_CHECK(maps >= 1 && k_cache.size(3) % maps == 0 &&
                   !(pairs && v_inv_freq.has_value()),
@@ -509,7 +554,8 @@ void qk_headnorm_rope_cache(at::Tensor& q_out, at::Tensor& q, at::Tensor& k,
                 positions.data_ptr(), slot_mapping.data_ptr(),
                 k_cache.data_ptr(), v_cache.data_ptr(), (float)eps, tokens,
                 (int)heads, G, D, DV, bs, qf, qh, v_unit_norm ? 1 : 0, vf, vh,
-                pairs ? 1 : 0, (float)rot_mult, (int)maps, in_f32, f32,
+                pairs ? 1 : 0, (float)rot_mult, (int)maps, qk_norm ? 1 : 0,
+                in_f32, f32,
                 current_stream()),
             "qk_headnorm_rope_cache");
 }
@@ -568,7 +614,7 @@ void router_topk(at::Tensor& idx, at::Tensor& w,
                  const c10::optional<at::Tensor>& dense, at::Tensor& logits,
                  bool softmax, bool renorm,
                  const c10::optional<at::Tensor>& correction,
-                 double renorm_eps, double weight_scale) {
+                 double renorm_eps, double weight_scale, bool over_chosen) {
   CHECK_F32(logits);
   CHECK_F32(w);
   CHECK_I32(idx);
@@ -591,7 +637,7 @@ void router_topk(at::Tensor& idx, at::Tensor& w,
   check_hip(ks_router_topk(idx.data_ptr(), w.data_ptr(), dp, logits.data_ptr(),
                            T, E, top, softmax ? 1 : 0, renorm ? 1 : 0, cp,
                            (float)renorm_eps, (float)weight_scale,
-                           current_stream()),
+                           over_chosen ? 1 : 0, current_stream()),
             "router_topk");
 }
 
@@ -600,7 +646,8 @@ void route_tokens(at::Tensor& idx, at::Tensor& w,
                   const c10::optional<at::Tensor>& logits_out, at::Tensor& h,
                   at::Tensor& router, bool softmax, bool renorm,
                   const c10::optional<at::Tensor>& correction,
-                  double renorm_eps, double weight_scale) {
+                  double renorm_eps, double weight_scale, bool over_chosen,
+                  const c10::optional<at::Tensor>& bias) {
   CHECK_ROWS(h);
   CHECK_F32(router);
   CHECK_F32(w);
@@ -628,11 +675,17 @@ void route_tokens(at::Tensor& idx, at::Tensor& w,
     TORCH_CHECK(correction->numel() == E, "correction [E]");
     cp = correction->data_ptr();
   }
+  const void* bp = nullptr;
+  if (bias.has_value()) {
+    CHECK_F32(*bias);
+    TORCH_CHECK(bias->numel() == E, "router bias [E]");
+    bp = bias->data_ptr();
+  }
   check_hip(ks_route_tokens(idx.data_ptr(), w.data_ptr(), dp, lp, h.data_ptr(),
                             h.stride(0), router.data_ptr(), T, W, E, top,
                             softmax ? 1 : 0, renorm ? 1 : 0, cp,
                             (float)renorm_eps, (float)weight_scale,
-                            act_is_f32(h, "h"),
+                            over_chosen ? 1 : 0, bp, act_is_f32(h, "h"),
                             current_stream()),
             "route_tokens");
 }
@@ -762,26 +815,37 @@ void post_layer_norm_add(at::Tensor& residual,
             "post_layer_norm_add");
 }
 
-void latent_norm_rope_cache(at::Tensor& cq_out, at::Tensor& proj,
-                            int64_t q_rank, int64_t kv_rank, int64_t rot_dim,
-                            at::Tensor& qw,
+void latent_norm_rope_cache(const c10::optional<at::Tensor>& cq_out,
+                            at::Tensor& proj, int64_t q_rank, int64_t kv_rank,
+                            int64_t rot_dim,
+                            const c10::optional<at::Tensor>& qw,
                             const c10::optional<at::Tensor>& kw,
                             at::Tensor& positions, at::Tensor& slot_mapping,
                             const c10::optional<at::Tensor>& cache, double eps,
-                            const c10::optional<at::Tensor>& inv_freq) {
+                            const c10::optional<at::Tensor>& inv_freq,
+                            bool pairs, double rot_mult) {
   CHECK_ROWS(proj);
-  CHECK_F32(qw);
   CHECK_I64(positions);
   CHECK_I32(slot_mapping);
   const int f32 = act_is_f32(proj, "proj");
   const int tokens = proj.size(0);
-  TORCH_CHECK(q_rank >= 1 && kv_rank >= 0 && rot_dim >= 0 &&
+  TORCH_CHECK(q_rank >= 0 && kv_rank >= 0 && rot_dim >= 0 &&
                   proj.size(1) >= q_rank + kv_rank + rot_dim &&
-                  qw.numel() == q_rank && cq_out.is_contiguous() &&
-                  act_is_f32(cq_out, "cq_out") == f32 &&
-                  cq_out.numel() == (int64_t)tokens * q_rank &&
                   positions.numel() >= tokens,
               "latent_norm_rope_cache: dtype/shape mismatch");
+  // a query latent comes with its norm weight and its output
+  void* cqp = nullptr;
+  const void* qwp = nullptr;
+  if (q_rank > 0) {
+    TORCH_CHECK(qw.has_value() && cq_out.has_value(), "query latent: qw, cq_out");
+    CHECK_F32(*qw);
+    TORCH_CHECK(qw->numel() == q_rank && cq_out->is_contiguous() &&
+                    act_is_f32(*cq_out, "cq_out") == f32 &&
+                    cq_out->numel() == (int64_t)tokens * q_rank,
+                "query latent: dtype/shape mismatch");
+    cqp = cq_out->data_ptr();
+    qwp = qw->data_ptr();
+  }
   const void *kp = nullptr, *fp = nullptr;
   void* cp = nullptr;
   int half = 0;
@@ -804,17 +868,18 @@ void latent_norm_rope_cache(at::Tensor& cq_out, at::Tensor& proj,
     }
   }
   check_hip(ks_latent_norm_rope_cache(
-                cq_out.data_ptr(), proj.data_ptr(), proj.stride(0), tokens,
-                (int)q_rank, (int)kv_rank, (int)rot_dim, qw.data_ptr(), kp,
-                positions.data_ptr(), slot_mapping.data_ptr(), cp, (float)eps,
-                fp, half, f32, current_stream()),
+                cqp, proj.data_ptr(), proj.stride(0), tokens, (int)q_rank,
+                (int)kv_rank, (int)rot_dim, qwp, kp, positions.data_ptr(),
+                slot_mapping.data_ptr(), cp, (float)eps, fp, half,
+                pairs ? 0 : 1, (float)rot_mult, f32, current_stream()),
             "latent_norm_rope_cache");
 }
 
 void head_matmul_rope(at::Tensor& out, at::Tensor& x, at::Tensor& w,
                       int64_t heads, int64_t tail,
                       const c10::optional<at::Tensor>& positions,
-                      const c10::optional<at::Tensor>& inv_freq) {
+                      const c10::optional<at::Tensor>& inv_freq, bool pairs,
+                      double rot_mult) {
   CHECK_ROWS(x);
   TORCH_CHECK(w.dim() == 3 && w.is_contiguous() && w.size(0) == heads,
               "w [heads, n, k] contiguous");
@@ -839,7 +904,8 @@ void head_matmul_rope(at::Tensor& out, at::Tensor& x, at::Tensor& w,
   }
   check_hip(ks_head_matmul_rope(out.data_ptr(), x.data_ptr(), x.stride(0),
                                 w.data_ptr(), tokens, (int)heads, K, N,
-                                (int)tail, pp, fp, half, in_f32, out_f32,
+                                (int)tail, pp, fp, half, pairs ? 0 : 1,
+                                (float)rot_mult, in_f32, out_f32,
                                 current_stream()),
             "head_matmul_rope");
 }
@@ -945,7 +1011,7 @@ void linear_scan(at::Tensor& o, at::Tensor& q, at::Tensor& k, at::Tensor& v,
                  const c10::optional<at::Tensor>& dt_bias,
                  const c10::optional<at::Tensor>& channel_decay,
                  at::Tensor& state, at::Tensor& positions, at::Tensor& cu_seqlens,
-                 at::Tensor& slots, int64_t qk_heads) {
+                 at::Tensor& slots, int64_t qk_heads, double q_scale) {
   CHECK_F32(o);
   CHECK_F32(state);
   CHECK_ROWS(q);
@@ -954,9 +1020,10 @@ void linear_scan(at::Tensor& o, at::Tensor& q, at::Tensor& k, at::Tensor& v,
   CHECK_I64(positions);
   CHECK_I32(cu_seqlens);
   CHECK_I32(slots);
-  TORCH_CHECK(q.scalar_type() == at::kFloat && k.scalar_type() == at::kFloat &&
-                  v.scalar_type() == at::kFloat && q.is_cuda() && k.is_cuda() &&
-                  v.is_cuda(),
+  // bf16 rows: the channel-decay form without a write strength only
+  const int qkv_f32 = act_is_f32(q, "q");
+  TORCH_CHECK(act_is_f32(k, "k") == qkv_f32 && act_is_f32(v, "v") == qkv_f32 &&
+                  (qkv_f32 || (channel_decay.has_value() && !b_raw.has_value())),
               "q, k, v must be fp32 GPU tensors");
   TORCH_CHECK(state.dim() == 4, "state [slots, heads, V, K]");
   const int heads = state.size(1), V = state.size(2), K = state.size(3);
@@ -979,15 +1046,16 @@ void linear_scan(at::Tensor& o, at::Tensor& q, at::Tensor& k, at::Tensor& v,
     dp = decay->data_ptr();
   } else if (channel_decay.has_value()) {
     CHECK_F32(*channel_decay);
-    TORCH_CHECK(b_raw.has_value() &&
-                    channel_decay->numel() == (int64_t)tokens * heads * K,
-                "the channel-decay form needs decays [T, heads*K] and b_raw");
-    CHECK_ROWS(*b_raw);
-    ab_f32 = act_is_f32(*b_raw, "b_raw");
-    TORCH_CHECK(b_raw->size(0) == tokens && b_raw->size(1) == heads,
-                "b_raw [T, heads]");
-    bp = b_raw->data_ptr();
-    ab_stride = b_raw->stride(0);
+    TORCH_CHECK(channel_decay->numel() == (int64_t)tokens * heads * K,
+                "channel decays [T, heads*K]");
+    if (b_raw.has_value()) {
+      CHECK_ROWS(*b_raw);
+      ab_f32 = act_is_f32(*b_raw, "b_raw");
+      TORCH_CHECK(b_raw->size(0) == tokens && b_raw->size(1) == heads,
+                  "b_raw [T, heads]");
+      bp = b_raw->data_ptr();
+      ab_stride = b_raw->stride(0);
+    }
     cdp = channel_decay->data_ptr();
   } else {
     TORCH_CHECK(a_raw.has_value() && b_raw.has_value() && a_log.has_value() &&
@@ -1012,11 +1080,31 @@ void linear_scan(at::Tensor& o, at::Tensor& q, at::Tensor& k, at::Tensor& v,
   }
   check_hip(ks_linear_scan(o.data_ptr(), q.data_ptr(), q.stride(0),
                            k.data_ptr(), k.stride(0), v.data_ptr(),
-                           v.stride(0), dp, ap, bp, ab_stride, ab_f32, alp, dtp, cdp,
+                           v.stride(0), qkv_f32, (float)q_scale, dp, ap, bp,
+                           ab_stride, ab_f32, alp, dtp, cdp,
                            state.data_ptr(), positions.data_ptr(),
                            cu_seqlens.data_ptr(), slots.data_ptr(), num_seqs,
                            heads, (int)qk_heads, V, K, current_stream()),
             "linear_scan");
+}
+
+void lowrank_channel_decay(at::Tensor& out, at::Tensor& low, at::Tensor& w2,
+                           at::Tensor& bias, double tau) {
+  CHECK_F32(out);
+  CHECK_F32(w2);
+  CHECK_F32(bias);
+  CHECK_ROWS(low);
+  const int f32 = act_is_f32(low, "low");
+  TORCH_CHECK(w2.dim() == 2, "w2 [n, r]");
+  const int tokens = low.size(0), r = low.size(1), n = w2.size(0);
+  TORCH_CHECK(w2.size(1) == r && bias.numel() == n &&
+                  out.numel() == (int64_t)tokens * n,
+              "lowrank_channel_decay: shape mismatch");
+  check_hip(ks_lowrank_channel_decay(out.data_ptr(), low.data_ptr(),
+                                     low.stride(0), w2.data_ptr(),
+                                     bias.data_ptr(), (float)tau, tokens, r, n,
+                                     f32, current_stream()),
+            "lowrank_channel_decay");
 }
 
 void delta_unit_decay(at::Tensor& x, at::Tensor& g, at::Tensor& a_raw,
@@ -1268,6 +1356,8 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
         "whole-row query norm, key pages and their 1/rms");
   m.def("talk_attention", &talk_attention,
         "paged fp32 attention with scores mixed over the heads");
+  m.def("lowrank_channel_decay", &lowrank_channel_decay,
+        "per-channel decays of a gated linear recurrence from a low-rank projection");
   m.def("linear_scan", &linear_scan,
         "decay / gated-delta linear-attention recurrence, per-slot fp32 state");
   def_sampling(m);

@@ -5,8 +5,9 @@
 //    RMS-normed (x / sqrt(mean(x^2) + eps) * w) and written out in the
 //    activation dtype. With a cache, the kv latent is RMS-normed the same way
 //    and the key part is rotated in pairs (2i, 2i+1) by pos * inv_freq[i]
-//    (fp32 angle, exact sin/cos; pairs past the frequency table and an odd
-//    last coordinate are copied); [normed latent | rotated key part] is the
+//    (fp32 angle, exact sin/cos; coordinates past the frequency table are
+//    copied), or with `halves` in pairs (i, i + half), turned coordinates
+//    times rot_mult; q_rank 0: no query latent; [normed latent | rotated key part] is the
 //    token's row of the paged cache [blocks, 1, block, kv_rank + rot_dim].
 //  * head_matmul_rope: per head h, out[t, h, :n] = W[h] x[t, h, :k] with
 //    W [heads, n, k] (fp32 sums), and the `tail` coordinates after the first
@@ -23,25 +24,51 @@ namespace {
 constexpr int NT = 256;
 constexpr int NW = NT / WAVE_SIZE;
 
+// A tail of n coordinates of a token at position `pos`, item p of n: with
+// `halves` coordinates i and i + half turn together, otherwise 2i and 2i + 1
+// (i < half; cos and sin times rot_mult); the rest is copied. Items 0..half-1
+// are the pairs, items half.. the copied coordinates.
+template <typename T, typename TO>
+__device__ __forceinline__ void turn_item(TO* __restrict__ dst,
+                                          const T* __restrict__ src, int p,
+                                          float pos,
+                                          const float* __restrict__ inv_freq,
+                                          int half, int halves, float rot_mult) {
+  if (p >= half) {
+    st_f32(dst, half + p, ld_f32(src, half + p));
+    return;
+  }
+  const int a = halves ? p : 2 * p, b = halves ? p + half : 2 * p + 1;
+  const float u = ld_f32(src, a), v = ld_f32(src, b);
+  float sn, cs;
+  sincosf(pos * inv_freq[p], &sn, &cs);
+  sn *= rot_mult;
+  cs *= rot_mult;
+  st_f32(dst, a, u * cs - v * sn);
+  st_f32(dst, b, v * cs + u * sn);
+}
+
 template <typename T>
 __global__ void __launch_bounds__(NT) latent_norm_rope_cache_kernel(
     T* __restrict__ cq_out, const T* __restrict__ proj, long row_stride,
     int q_rank, int kv_rank, int rot_dim, const float* __restrict__ qw,
     const float* __restrict__ kw, const long* __restrict__ positions,
     const int* __restrict__ slot_mapping, T* __restrict__ cache, float eps,
-    const float* __restrict__ inv_freq, int half) {
+    const float* __restrict__ inv_freq, int half, int halves, float rot_mult) {
   __shared__ float scratch[NW];
   const long t = blockIdx.x;
   const T* row = proj + t * row_stride;
   float ss = 0.f;
-  for (int i = threadIdx.x; i < q_rank; i += NT) {
-    const float x = ld_f32(row, i);
-    ss += x * x;
+  if (q_rank > 0) {
+    for (int i = threadIdx.x; i < q_rank; i += NT) {
+      const float x = ld_f32(row, i);
+      ss += x * x;
+    }
+    ss = block_sum_sync<NW>(ss, scratch);
+    const float qinv = 1.0f / sqrtf(ss / (float)q_rank + eps);
+    for (int i = threadIdx.x; i < q_rank; i += NT)
+      st_f32(cq_out, t * q_rank + i, ld_f32(row, i) * qinv * qw[i]);
   }
-  ss = block_sum_sync<NW>(ss, scratch);
-  const float qinv = 1.0f / sqrtf(ss / (float)q_rank + eps);
-  for (int i = threadIdx.x; i < q_rank; i += NT)
-    st_f32(cq_out, t * q_rank + i, ld_f32(row, i) * qinv * qw[i]);
   if (!cache) return;
   const long slot = slot_mapping[t];
   if (slot < 0) return;  // the whole block leaves together
@@ -58,48 +85,30 @@ __global__ void __launch_bounds__(NT) latent_norm_rope_cache_kernel(
     st_f32(dst, i, ld_f32(c, i) * cinv * kw[i]);
   const T* kr = c + kv_rank;
   const float pos = (float)positions[t];
-  for (int p = threadIdx.x; 2 * p < rot_dim; p += NT) {
-    const float u = ld_f32(kr, 2 * p);
-    if (2 * p + 1 >= rot_dim) {
-      st_f32(dst, kv_rank + 2 * p, u);
-    } else {
-      const float v = ld_f32(kr, 2 * p + 1);
-      float sn = 0.f, cs = 1.f;
-      if (p < half) sincosf(pos * inv_freq[p], &sn, &cs);
-      st_f32(dst, kv_rank + 2 * p, u * cs - v * sn);
-      st_f32(dst, kv_rank + 2 * p + 1, v * cs + u * sn);
-    }
-  }
+  for (int p = threadIdx.x; p < rot_dim - half; p += NT)
+    turn_item(dst + kv_rank, kr, p, pos, inv_freq, half, halves, rot_mult);
 }
 
 constexpr int TT = 32;         // tokens per block
 constexpr int TPW = TT / NW;   // tokens per wave
 constexpr int CPL = 4;         // columns per lane (64 apart)
 
-// Pair rotation of the tail coordinates behind the product, for the tokens
+// Rotation of the tail coordinates behind the product, for the tokens
 // [t0, t0 + nt) of head h (all threads of the block take part).
 template <typename T, typename TO>
 __device__ __forceinline__ void rotate_tail(
     TO* __restrict__ out, const T* __restrict__ x, long x_stride, int t0,
     int nt, int h, int heads, int K, int N, int tail,
     const long* __restrict__ positions, const float* __restrict__ inv_freq,
-    int half) {
+    int half, int halves, float rot_mult) {
   const int in_w = K + tail, out_w = N + tail;
-  const int pairs = (tail + 1) / 2;
-  for (int e = threadIdx.x; e < nt * pairs; e += NT) {
-    const int tt = e / pairs, p = e % pairs;
+  const int items = tail - half;
+  for (int e = threadIdx.x; e < nt * items; e += NT) {
+    const int tt = e / items, p = e % items;
     const long src = (long)(t0 + tt) * x_stride + (long)h * in_w + K;
     const long o = ((long)(t0 + tt) * heads + h) * out_w + N;
-    const float u = ld_f32(x, src + 2 * p);
-    if (2 * p + 1 >= tail) {
-      st_f32(out, o + 2 * p, u);
-    } else {
-      const float v = ld_f32(x, src + 2 * p + 1);
-      float sn = 0.f, cs = 1.f;
-      if (p < half) sincosf((float)positions[t0 + tt] * inv_freq[p], &sn, &cs);
-      st_f32(out, o + 2 * p, u * cs - v * sn);
-      st_f32(out, o + 2 * p + 1, v * cs + u * sn);
-    }
+    const float pos = half > 0 ? (float)positions[t0 + tt] : 0.f;
+    turn_item(out + o, x + src, p, pos, inv_freq, half, halves, rot_mult);
   }
 }
 
@@ -110,7 +119,7 @@ __global__ void __launch_bounds__(NT) head_matmul_rope_kernel(
     TO* __restrict__ out, const T* __restrict__ x, long x_stride,
     const T* __restrict__ w, int tokens, int heads, int K, int N, int tail,
     const long* __restrict__ positions, const float* __restrict__ inv_freq,
-    int half) {
+    int half, int halves, float rot_mult) {
   extern __shared__ float xs[];  // [TT][K]
   const int t0 = blockIdx.x * TT;
   const int h = blockIdx.y;
@@ -159,7 +168,7 @@ __global__ void __launch_bounds__(NT) head_matmul_rope_kernel(
   }
   if (tail == 0 || blockIdx.z != 0) return;
   rotate_tail(out, x, x_stride, t0, nt, h, heads, K, N, tail, positions,
-              inv_freq, half);
+              inv_freq, half, halves, rot_mult);
 }
 
 // Matrix-core form for 16-byte aligned operands (K, the head widths and the
@@ -214,7 +223,7 @@ __global__ void __launch_bounds__(NT) head_matmul_rope_mfma_kernel(
     TO* __restrict__ out, const T* __restrict__ x, long x_stride,
     const T* __restrict__ w, int tokens, int heads, int K, int N, int tail,
     const long* __restrict__ positions, const float* __restrict__ inv_freq,
-    int half) {
+    int half, int halves, float rot_mult) {
   constexpr int KB = Frag<T>::KB;
   constexpr int CH = KB / 4;  // elements per lane and step
   constexpr int NTILE = 4;    // 16-column tiles per wave
@@ -282,7 +291,7 @@ __global__ void __launch_bounds__(NT) head_matmul_rope_mfma_kernel(
   }
   if (tail == 0 || blockIdx.z != 0) return;
   rotate_tail(out, x, x_stride, t0, min(64 * MT, tokens - t0), h, heads, K, N,
-              tail, positions, inv_freq, half);
+              tail, positions, inv_freq, half, halves, rot_mult);
 }
 
 }  // namespace
@@ -291,9 +300,10 @@ extern "C" hipError_t ks_latent_norm_rope_cache(
     void* cq_out, const void* proj, long row_stride, int tokens, int q_rank,
     int kv_rank, int rot_dim, const void* qw, const void* kw,
     const void* positions, const void* slot_mapping, void* cache, float eps,
-    const void* inv_freq, int half, int is_f32, hipStream_t stream) {
+    const void* inv_freq, int half, int halves, float rot_mult, int is_f32,
+    hipStream_t stream) {
   if (tokens == 0) return hipSuccess;
-  if (q_rank < 1 || (cache && (kv_rank < 1 || !kw)) || 2 * half > rot_dim ||
+  if (q_rank < 0 || (q_rank > 0 && (!cq_out || !qw)) || (cache && (kv_rank < 1 || !kw)) || 2 * half > rot_dim ||
       (half > 0 && !inv_freq))
     return hipErrorInvalidValue;
   if (is_f32)
@@ -302,14 +312,14 @@ extern "C" hipError_t ks_latent_norm_rope_cache(
                        row_stride, q_rank, kv_rank, rot_dim, (const float*)qw,
                        (const float*)kw, (const long*)positions,
                        (const int*)slot_mapping, (float*)cache, eps,
-                       (const float*)inv_freq, half);
+                       (const float*)inv_freq, half, halves, rot_mult);
   else
     hipLaunchKernelGGL(latent_norm_rope_cache_kernel<short>, dim3(tokens),
                        dim3(NT), 0, stream, (short*)cq_out, (const short*)proj,
                        row_stride, q_rank, kv_rank, rot_dim, (const float*)qw,
                        (const float*)kw, (const long*)positions,
                        (const int*)slot_mapping, (short*)cache, eps,
-                       (const float*)inv_freq, half);
+                       (const float*)inv_freq, half, halves, rot_mult);
   HIP_CHECK_KERNEL();
   return hipSuccess;
 }
@@ -320,6 +330,7 @@ static hipError_t launch_head_matmul(void* out, const void* x, long x_stride,
                                      int K, int N, int tail,
                                      const void* positions,
                                      const void* inv_freq, int half,
+                                     int halves, float rot_mult,
                                      hipStream_t stream) {
   constexpr int CH = 16 / sizeof(T);
   const bool aligned = K % CH == 0 && (K + tail) % CH == 0 &&
@@ -336,7 +347,7 @@ static hipError_t launch_head_matmul(void* out, const void* x, long x_stride,
                   : head_matmul_rope_mfma_kernel<T, TO, 1>;
     hipLaunchKernelGGL(fn, grid, dim3(NT), 0, stream, (TO*)out, (const T*)x,
                        x_stride, (const T*)w, tokens, heads, K, N, tail,
-                       (const long*)positions, (const float*)inv_freq, half);
+                       (const long*)positions, (const float*)inv_freq, half, halves, rot_mult);
     return hipGetLastError();
   }
   const size_t smem = sizeof(float) * (size_t)TT * K;
@@ -349,7 +360,7 @@ static hipError_t launch_head_matmul(void* out, const void* x, long x_stride,
   dim3 grid(cdiv(tokens, TT), heads, cdiv(N, 64 * CPL));
   hipLaunchKernelGGL(fn, grid, dim3(NT), smem, stream, (TO*)out, (const T*)x,
                      x_stride, (const T*)w, tokens, heads, K, N, tail,
-                     (const long*)positions, (const float*)inv_freq, half);
+                     (const long*)positions, (const float*)inv_freq, half, halves, rot_mult);
   return hipGetLastError();
 }
 
@@ -360,6 +371,7 @@ extern "C" hipError_t ks_head_matmul_rope(void* out, const void* x,
                                           int tokens, int heads, int K, int N,
                                           int tail, const void* positions,
                                           const void* inv_freq, int half,
+                                          int halves, float rot_mult,
                                           int in_f32, int out_f32,
                                           hipStream_t stream) {
   if (tokens == 0) return hipSuccess;
@@ -369,7 +381,7 @@ extern "C" hipError_t ks_head_matmul_rope(void* out, const void* x,
     return hipErrorInvalidValue;
 #define HM_ARGS                                                              \
   out, x, x_stride, w, tokens, heads, K, N, tail, positions, inv_freq, half, \
-      stream
+      halves, rot_mult, stream
   if (in_f32) return launch_head_matmul<float, float>(HM_ARGS);
   if (out_f32) return launch_head_matmul<short, float>(HM_ARGS);
   return launch_head_matmul<short, short>(HM_ARGS);

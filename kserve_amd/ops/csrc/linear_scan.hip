@@ -15,6 +15,11 @@
 // fp32 rows: S <- diag(g) S first (one multiplication per state element), then
 // the delta form with g = 1.
 //
+// A fourth form is the decay form with such per-channel decays,
+//   channel decay (gated linear attention): S <- diag(g) S + k v^T,
+// and reads q, k, v in the activation dtype straight from the columns of a
+// projection (q times q_scale).
+//
 // d is a constant per head; g = exp(-exp(A_log) softplus(a + dt_bias)) and
 // b = sigmoid(beta_raw) are computed here in fp32 from raw per-token, per-head
 // projection columns. Both forms are evaluated from the OLD state with two
@@ -37,6 +42,8 @@
 //    after them are only widened to fp32 (values).
 //  * unit_norm_heads: x / sqrt(sum(x^2) + eps) * scale per head, in place on
 //    fp32 rows; two runs of heads with a scale each (queries, keys).
+//  * lowrank_channel_decay: sigmoid(z)^(1/tau), z = W2 low + b, the decays of
+//    the fourth form from a low-rank projection; fp32 after the first factor.
 //  * delta_unit_decay: the unit norms, and for the third form the decays
 //    g = exp(-exp(A_log) softplus(a + dt_bias)) per head and key channel.
 #include "dtype_io.h"
@@ -139,19 +146,71 @@ __global__ void delta_unit_decay_kernel(
   }
 }
 
+// A block takes DT tokens (their low rows in LDS as fp32) x 256 columns; a lane
+// keeps one column's sums of all DT tokens and reads that column's row of w2.
+constexpr int DT = 16;
+
+template <typename T>
+__global__ void __launch_bounds__(NT) lowrank_channel_decay_kernel(
+    float* __restrict__ out, const T* __restrict__ low, long low_stride,
+    const float* __restrict__ w2, const float* __restrict__ bias, float inv_tau,
+    int tokens, int r, int n) {
+  extern __shared__ float ls[];  // [DT][r]
+  const long t0 = (long)blockIdx.x * DT;
+  const int cnt = min((long)DT, tokens - t0);
+  for (int e = threadIdx.x; e < DT * r; e += NT) {
+    const int tt = e / r;
+    ls[e] = tt < cnt ? ld_f32(low, (t0 + tt) * low_stride + e % r) : 0.f;
+  }
+  __syncthreads();
+  const int c = blockIdx.y * NT + threadIdx.x;
+  if (c >= n) return;
+  const float* w = w2 + (long)c * r;
+  const bool vec = r % 4 == 0 && ((uintptr_t)w2 % 16) == 0;
+  float acc[DT];
+  const float b = bias[c];
+#pragma unroll
+  for (int a = 0; a < DT; ++a) acc[a] = b;
+  if (vec) {
+    for (int k = 0; k < r; k += 4) {
+      const float4_t w4 = *reinterpret_cast<const float4_t*>(w + k);
+#pragma unroll
+      for (int a = 0; a < DT; ++a) {
+        const float4_t x = *reinterpret_cast<const float4_t*>(ls + a * r + k);
+        acc[a] += w4[0] * x[0] + w4[1] * x[1] + w4[2] * x[2] + w4[3] * x[3];
+      }
+    }
+  } else {
+    for (int k = 0; k < r; ++k) {
+      const float wk = w[k];
+#pragma unroll
+      for (int a = 0; a < DT; ++a) acc[a] += wk * ls[a * r + k];
+    }
+  }
+#pragma unroll
+  for (int a = 0; a < DT; ++a) {
+    if (a < cnt) {
+      // log sigmoid(z) = min(z, 0) - log(1 + exp(-|z|))
+      const float z = acc[a];
+      const float lg = fminf(z, 0.f) - log1pf(expf(-fabsf(z)));
+      out[(t0 + a) * n + c] = expf(lg * inv_tau);
+    }
+  }
+}
+
 constexpr int SCAN_TC = 16;  // tokens per chunk
 
 // recurrence forms
-constexpr int DECAY = 0, HEAD_DELTA = 1, CHANNEL_DELTA = 2;
+constexpr int DECAY = 0, HEAD_DELTA = 1, CHANNEL_DELTA = 2, CHANNEL_DECAY = 3;
 
 // R = state rows per lane (K <= 16 R), PC = columns per lane (a block covers
-// 16 PC value columns of one head).
-template <int R, int PC, int FORM>
+// 16 PC value columns of one head). TQ: dtype of q, k, v.
+template <int R, int PC, int FORM, typename TQ>
 __global__ void __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(4)))
 linear_scan_kernel(
-    float* __restrict__ o, const float* __restrict__ q, long q_stride,
-    const float* __restrict__ k, long k_stride, const float* __restrict__ v,
-    long v_stride, const float* __restrict__ decay,
+    float* __restrict__ o, const TQ* __restrict__ q, long q_stride,
+    const TQ* __restrict__ k, long k_stride, const TQ* __restrict__ v,
+    long v_stride, float q_scale, const float* __restrict__ decay,
     const float* __restrict__ a_f32, const short* __restrict__ a_bf16,
     const float* __restrict__ b_f32, const short* __restrict__ b_bf16,
     long ab_stride, const float* __restrict__ a_log,
@@ -160,8 +219,8 @@ linear_scan_kernel(
     const long* __restrict__ positions, const int* __restrict__ cu_seqlens,
     const int* __restrict__ slots, int heads, int qk_heads, int V, int K) {
   extern __shared__ float lds[];
-  constexpr bool DELTA = FORM != DECAY;
-  constexpr bool CHAN = FORM == CHANNEL_DELTA;
+  constexpr bool DELTA = FORM == HEAD_DELTA || FORM == CHANNEL_DELTA;
+  constexpr bool CHAN = FORM == CHANNEL_DELTA || FORM == CHANNEL_DECAY;
   constexpr int tc = SCAN_TC;
   constexpr int XS = 16 * PC;
   const int s = blockIdx.z;
@@ -177,7 +236,7 @@ linear_scan_kernel(
   const int inner = heads * V;
   const long slot = slots[s];
   const bool fresh = positions[first] == 0;
-  const float fixed = DELTA ? 1.f : decay[h];
+  const float fixed = FORM == DECAY ? decay[h] : 1.f;
   const float A = FORM == HEAD_DELTA ? -expf(a_log[h]) : 0.f;
   const float bias = FORM == HEAD_DELTA ? dt_bias[h] : 0.f;
 
@@ -211,21 +270,21 @@ linear_scan_kernel(
   auto prefetch = [&](int t0, int cnt) {
     const bool on = stk < cnt;
     const long t = first + t0 + (on ? stk : 0);
-    const float* krow = k + t * k_stride + (long)hq * K;
-    const float* qrow = q + t * q_stride + (long)hq * K;
-    const float* vrow = v + t * v_stride + (long)h * V + p0;
+    const TQ* krow = k + t * k_stride + (long)hq * K;
+    const TQ* qrow = q + t * q_stride + (long)hq * K;
+    const TQ* vrow = v + t * v_stride + (long)h * V + p0;
 #pragma unroll
     for (int r = 0; r < R; ++r) {
       const int n = sl + 16 * r;
       const bool ok = on && n < K;
-      sK[r] = ok ? krow[n] : 0.f;
-      sQ[r] = ok ? qrow[n] : 0.f;
+      sK[r] = ok ? ld_f32(krow, n) : 0.f;
+      sQ[r] = ok ? ld_f32(qrow, n) * q_scale : 0.f;
       if (CHAN) sC[r] = ok ? channel_decay[(t * heads + h) * K + n] : 0.f;
     }
 #pragma unroll
     for (int c = 0; c < PC; ++c) {
       const int col = sl + 16 * c;
-      sV[c] = (on && col < pt) ? vrow[col] : 0.f;
+      sV[c] = (on && col < pt) ? ld_f32(vrow, col) : 0.f;
     }
     if (DELTA && on && sl == 0) {
       const long i = t * ab_stride + h;
@@ -385,10 +444,32 @@ extern "C" hipError_t ks_delta_unit_decay(
   return hipSuccess;
 }
 
+extern "C" hipError_t ks_lowrank_channel_decay(
+    void* out, const void* low, long low_stride, const void* w2,
+    const void* bias, float tau, int tokens, int r, int n, int is_f32,
+    hipStream_t stream) {
+  if (tokens == 0) return hipSuccess;
+  if (r < 1 || n < 1 || r > 768 || !(tau > 0.f)) return hipErrorInvalidValue;
+  const dim3 grid(cdiv(tokens, DT), cdiv(n, NT));
+  const size_t smem = sizeof(float) * (size_t)DT * r;
+  if (is_f32)
+    hipLaunchKernelGGL(lowrank_channel_decay_kernel<float>, grid, dim3(NT), smem,
+                       stream, (float*)out, (const float*)low, low_stride,
+                       (const float*)w2, (const float*)bias, 1.0f / tau, tokens,
+                       r, n);
+  else
+    hipLaunchKernelGGL(lowrank_channel_decay_kernel<short>, grid, dim3(NT), smem,
+                       stream, (float*)out, (const short*)low, low_stride,
+                       (const float*)w2, (const float*)bias, 1.0f / tau, tokens,
+                       r, n);
+  HIP_CHECK_KERNEL();
+  return hipSuccess;
+}
+
 #define LSCAN_LAUNCH(RR, PCC, DD)                                             \
-  hipLaunchKernelGGL((linear_scan_kernel<RR, PCC, DD>), grid, dim3(256), smem, \
-                     stream, (float*)o, (const float*)q, q_stride,            \
-                     (const float*)k, k_stride, (const float*)v, v_stride,    \
+  hipLaunchKernelGGL((linear_scan_kernel<RR, PCC, DD, TQ>), grid, dim3(256),  \
+                     smem, stream, (float*)o, (const TQ*)q, q_stride,         \
+                     (const TQ*)k, k_stride, (const TQ*)v, v_stride, q_scale, \
                      (const float*)decay,                                     \
                      ab_is_f32 ? (const float*)a_raw : nullptr,               \
                      ab_is_f32 ? nullptr : (const short*)a_raw,               \
@@ -416,12 +497,14 @@ extern "C" hipError_t ks_delta_unit_decay(
     else LSCAN_LAUNCH(16, 2, DD);                                             \
   } while (0)
 
-// decay != null: decay form; otherwise a delta form, which reads b_raw
-// [T, heads] and either channel_decay [T, heads*K] or a_raw [T, heads] (a and
+// decay != null: decay form; channel_decay without b_raw: channel-decay form
+// (the only one that takes bf16 q, k, v); otherwise a delta form, which reads
+// b_raw [T, heads] and either channel_decay [T, heads*K] or a_raw [T, heads] (a and
 // b: two column ranges of rows with one stride), a_log and dt_bias.
 extern "C" hipError_t ks_linear_scan(
     void* o, const void* q, long q_stride, const void* k, long k_stride,
-    const void* v, long v_stride, const void* decay, const void* a_raw,
+    const void* v, long v_stride, int qkv_is_f32, float q_scale,
+    const void* decay, const void* a_raw,
     const void* b_raw, long ab_stride, int ab_is_f32, const void* a_log,
     const void* dt_bias, const void* channel_decay, void* state,
     const void* positions, const void* cu_seqlens, const void* slots,
@@ -429,8 +512,11 @@ extern "C" hipError_t ks_linear_scan(
   if (num_seqs == 0) return hipSuccess;
   if (qk_heads <= 0 || heads % qk_heads != 0 || K < 1 || K > 256 || V < 1)
     return hipErrorInvalidValue;
-  if (!decay && (!b_raw || (!channel_decay && (!a_raw || !a_log || !dt_bias))))
+  const bool chan = !decay && channel_decay && !b_raw;
+  if (!decay && !chan &&
+      (!b_raw || (!channel_decay && (!a_raw || !a_log || !dt_bias))))
     return hipErrorInvalidValue;
+  if (!qkv_is_f32 && !chan) return hipErrorInvalidValue;
   const int R = cdiv(K, 16);
   int pc = V > 32 ? 4 : (V > 16 ? 2 : 1);
   if (R > 8 && pc > 2) pc = 2;
@@ -440,9 +526,16 @@ extern "C" hipError_t ks_linear_scan(
   const int xs = 16 * pc;
   const size_t smem = sizeof(float) * ((size_t)SCAN_TC * ((channel_decay ? 3 : 2) * K + 2 * xs + 3));
   dim3 grid(cdiv(V, xs), heads, num_seqs);
-  if (decay) LSCAN_LAUNCH_R(DECAY);
-  else if (channel_decay) LSCAN_LAUNCH_R(CHANNEL_DELTA);
-  else LSCAN_LAUNCH_R(HEAD_DELTA);
+  if (!qkv_is_f32) {
+    using TQ = short;
+    LSCAN_LAUNCH_R(CHANNEL_DECAY);
+  } else {
+    using TQ = float;
+    if (decay) LSCAN_LAUNCH_R(DECAY);
+    else if (chan) LSCAN_LAUNCH_R(CHANNEL_DECAY);
+    else if (channel_decay) LSCAN_LAUNCH_R(CHANNEL_DELTA);
+    else LSCAN_LAUNCH_R(HEAD_DELTA);
+  }
   HIP_CHECK_KERNEL();
   return hipSuccess;
 }

@@ -5,11 +5,14 @@
 //    (ties go to the lower expert), optionally renormalised to sum 1
 //    (divided by their sum + renorm_eps) and multiplied by weight_scale. With a correction vector the
 //    choice goes by score + correction[e] while the weights stay the scores.
+//    over_chosen: the largest logits are chosen and the weights are the softmax
+//    over those logits only.
 //    Outputs expert ids and weights [T, top] and, if asked, the same weights
 //    as a dense [T, E] matrix that is zero for experts not chosen.
 //  * route_tokens: the router's matrix product fused in front of the same
 //    choice: a block per token, the input row in LDS as fp32, fp32 router
-//    rows, fp32 sums; the logits never travel through memory.
+//    rows, fp32 sums, an optional bias per expert; the logits never travel
+//    through memory.
 //  * gather_scale_rows: out[r] = x[rows[r]] * scales[r], product in fp32,
 //    rounded to the activation dtype (an expert's input is the token's input
 //    times its routing weight); without scales a plain row gather.
@@ -34,7 +37,8 @@ __device__ __forceinline__ void wave_topk(int* __restrict__ idx_out,
                                           const float* z, long t, int E,
                                           int top, int softmax, int renorm,
                                           const float* __restrict__ correction,
-                                          float renorm_eps, float weight_scale) {
+                                          float renorm_eps, float weight_scale,
+                                          int over_chosen) {
   const int lane = threadIdx.x & 63;
   float sc[MAX_PER_LANE];  // scores of experts lane + 64 j
   float mx = -INFINITY;
@@ -44,7 +48,10 @@ __device__ __forceinline__ void wave_topk(int* __restrict__ idx_out,
     sc[j] = e < E ? z[e] : -INFINITY;
     mx = fmaxf(mx, sc[j]);
   }
-  if (softmax) {
+  if (over_chosen) {
+    // the logits are the scores; exp and sum follow the choice
+    mx = wave_reduce_max(mx);
+  } else if (softmax) {
     mx = wave_reduce_max(mx);
     float sum = 0.f;
 #pragma unroll
@@ -94,14 +101,16 @@ __device__ __forceinline__ void wave_topk(int* __restrict__ idx_out,
     }
     if (be == 0x7fffffff) be = 0;  // nothing comparable left (NaN scores)
     if ((be & 63) == lane) chosen |= 1u << (be >> 6);
-    total += bs;
+    // the chosen logits' maximum is the maximum of all
+    total += over_chosen ? expf(bs - mx) : bs;
     if (lane == k) {
-      my_w = bs;
+      my_w = over_chosen ? expf(bs - mx) : bs;
       my_e = be;
     }
   }
   const float norm =
-      (renorm ? 1.0f / (total + renorm_eps) : 1.0f) * weight_scale;
+      (over_chosen ? 1.0f / total : renorm ? 1.0f / (total + renorm_eps) : 1.0f) *
+      weight_scale;
   if (lane < top) {
     idx_out[t * top + lane] = my_e;
     w_out[t * top + lane] = my_w * norm;
@@ -110,7 +119,10 @@ __device__ __forceinline__ void wave_topk(int* __restrict__ idx_out,
 #pragma unroll
     for (int j = 0; j < MAX_PER_LANE; ++j) {
       const int e = lane + 64 * j;
-      if (e < E) dense_out[t * E + e] = (chosen >> j & 1u) ? sc[j] * norm : 0.f;
+      if (e < E)
+        dense_out[t * E + e] =
+            (chosen >> j & 1u) ? (over_chosen ? expf(sc[j] - mx) : sc[j]) * norm
+                               : 0.f;
     }
   }
 }
@@ -121,11 +133,12 @@ __global__ void router_topk_kernel(int* __restrict__ idx_out,
                                    const float* __restrict__ logits, int tokens,
                                    int E, int top, int softmax, int renorm,
                                    const float* __restrict__ correction,
-                                   float renorm_eps, float weight_scale) {
+                                   float renorm_eps, float weight_scale,
+                                   int over_chosen) {
   const long t = (long)blockIdx.x * NW + (threadIdx.x >> 6);
   if (t >= tokens) return;  // whole waves leave together
   wave_topk(idx_out, w_out, dense_out, logits + t * E, t, E, top, softmax,
-            renorm, correction, renorm_eps, weight_scale);
+            renorm, correction, renorm_eps, weight_scale, over_chosen);
 }
 
 // Router logits and the choice in one kernel: a block per token keeps the
@@ -137,7 +150,8 @@ __global__ void __launch_bounds__(NT) route_tokens_kernel(
     float* __restrict__ dense_out, float* __restrict__ logits_out,
     const T* __restrict__ h, long h_stride, const float* __restrict__ router,
     int W, int E, int top, int softmax, int renorm,
-    const float* __restrict__ correction, float renorm_eps, float weight_scale) {
+    const float* __restrict__ correction, float renorm_eps, float weight_scale,
+    int over_chosen, const float* __restrict__ bias) {
   extern __shared__ float lds[];
   float* row = lds;      // [W]
   float* z = lds + ((W + 3) & ~3);  // [E]
@@ -182,6 +196,7 @@ __global__ void __launch_bounds__(NT) route_tokens_kernel(
     }
     acc = wave_reduce_sum(acc);
     if (lane == 0) {
+      if (bias) acc += bias[e];
       z[e] = acc;
       if (logits_out) logits_out[t * E + e] = acc;
     }
@@ -189,7 +204,7 @@ __global__ void __launch_bounds__(NT) route_tokens_kernel(
   __syncthreads();
   if (wave == 0)
     wave_topk(idx_out, w_out, dense_out, z, t, E, top, softmax, renorm,
-              correction, renorm_eps, weight_scale);
+              correction, renorm_eps, weight_scale, over_chosen);
 }
 
 __device__ __forceinline__ void ld4_any(const short* p, float* v) {
@@ -283,14 +298,15 @@ extern "C" hipError_t ks_router_topk(void* idx_out, void* w_out,
                                      int tokens, int E, int top, int softmax,
                                      int renorm, const void* correction,
                                      float renorm_eps, float weight_scale,
-                                     hipStream_t stream) {
+                                     int over_chosen, hipStream_t stream) {
   if (tokens == 0) return hipSuccess;
   if (E < 1 || E > 64 * MAX_PER_LANE || top < 1 || top > E || top > 64)
     return hipErrorInvalidValue;
   hipLaunchKernelGGL(router_topk_kernel, dim3(cdiv(tokens, NW)), dim3(NT), 0,
                      stream, (int*)idx_out, (float*)w_out, (float*)dense_out,
                      (const float*)logits, tokens, E, top, softmax, renorm,
-                     (const float*)correction, renorm_eps, weight_scale);
+                     (const float*)correction, renorm_eps, weight_scale,
+                     over_chosen);
   HIP_CHECK_KERNEL();
   return hipSuccess;
 }
@@ -301,6 +317,7 @@ extern "C" hipError_t ks_route_tokens(void* idx_out, void* w_out,
                                       const void* router, int tokens, int W,
                                       int E, int top, int softmax, int renorm,
                                       const void* correction, float renorm_eps, float weight_scale,
+                                      int over_chosen, const void* bias,
                                       int is_f32, hipStream_t stream) {
   if (tokens == 0) return hipSuccess;
   if (E < 1 || E > 64 * MAX_PER_LANE || top < 1 || top > E || top > 64 ||
@@ -318,7 +335,8 @@ extern "C" hipError_t ks_route_tokens(void* idx_out, void* w_out,
                        stream, (int*)idx_out, (float*)w_out, (float*)dense_out,
                        (float*)logits_out, (const float*)h, h_stride,
                        (const float*)router, W, E, top, softmax, renorm,
-                       (const float*)correction, renorm_eps, weight_scale);
+                       (const float*)correction, renorm_eps, weight_scale,
+                       over_chosen, (const float*)bias);
   } else {
     if (smem > 48 * 1024) {
       hipError_t e = hipFuncSetAttribute(
@@ -330,7 +348,8 @@ extern "C" hipError_t ks_route_tokens(void* idx_out, void* w_out,
                        stream, (int*)idx_out, (float*)w_out, (float*)dense_out,
                        (float*)logits_out, (const short*)h, h_stride,
                        (const float*)router, W, E, top, softmax, renorm,
-                       (const float*)correction, renorm_eps, weight_scale);
+                       (const float*)correction, renorm_eps, weight_scale,
+                       over_chosen, (const float*)bias);
   }
   HIP_CHECK_KERNEL();
   return hipSuccess;

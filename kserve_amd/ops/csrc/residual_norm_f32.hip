@@ -2,10 +2,14 @@
 //
 //  * embed_scale_sinpos: row = table[token] * scale + interleaved sinusoid
 //    (even entry sin, odd entry cos of position * inv_freq[i]); fp32 out.
-//  * add_rms_norm_f32res: residual += s0*d0 + s1*d1 (fp32, in place), then
-//    out = residual / sqrt(mean(residual^2) + eps) * (w_offset + w).
-//    The deltas are sublayer outputs in the activation dtype; either may be
-//    absent. One kernel covers "add the previous sublayer, norm for the next".
+//  * add_rms_norm_f32res: residual += s0*c0*d0 + s1*c1*d1 (fp32, in place;
+//    c0, c1: optional factors per channel), then
+//    out = residual / sqrt(mean(residual^2) + eps) * (w_offset + w), or without
+//    a weight out = residual. The deltas are sublayer outputs in the activation
+//    dtype or fp32; either may be absent. The second one may be given as rows
+//    to be summed, sum_k row_w[t*top + k] * d1[index[t*top + k]]: a mixture's
+//    expert rows go into the stream without a pass of their own. One kernel
+//    covers "add the previous sublayers, norm for the next".
 //  * post_norm_add_rms_norm: closes a sandwich-normed sublayer and opens the
 //    next one: residual += layer_scale * (delta / rms(delta) * post_gain),
 //    += an optional per-token row and an optional shared row, then
@@ -63,6 +67,8 @@ template <typename TD, typename TO>
 __global__ void add_rms_norm_f32res_kernel(
     float* __restrict__ residual, const TD* __restrict__ d0, long d0_stride,
     float s0, const TD* __restrict__ d1, long d1_stride, float s1,
+    const float* __restrict__ c0, const float* __restrict__ c1,
+    const int* __restrict__ index, const float* __restrict__ row_w, int top,
     const float* __restrict__ weight, float w_offset, float eps,
     TO* __restrict__ out, int width) {
   __shared__ float scratch[NW];
@@ -71,13 +77,24 @@ __global__ void add_rms_norm_f32res_kernel(
   float ss = 0.f;
   for (int i = threadIdx.x; i < width; i += NT) {
     float v = r[i];
-    if (d0) v += s0 * ld_f32(d0, row * d0_stride + i);
-    if (d1) v += s1 * ld_f32(d1, row * d1_stride + i);
+    if (d0) v += s0 * ld_f32(d0, row * d0_stride + i) * (c0 ? c0[i] : 1.f);
+    if (d1) {
+      float d = 0.f;
+      if (index) {
+        for (int k = 0; k < top; ++k)
+          d += (row_w ? row_w[row * top + k] : 1.f) *
+               ld_f32(d1, (long)index[row * top + k] * d1_stride + i);
+      } else {
+        d = ld_f32(d1, row * d1_stride + i);
+      }
+      v += s1 * d * (c1 ? c1[i] : 1.f);
+    }
     if (d0 || d1) r[i] = v;
+    if (out && !weight) st_f32(out, row * width + i, v);
     ss += v * v;
   }
+  if (!out || !weight) return;
   ss = block_sum_sync<NW>(ss, scratch);
-  if (!out) return;
   const float inv = 1.0f / sqrtf(ss / (float)width + eps);
   for (int i = threadIdx.x; i < width; i += NT) {
     // each thread re-reads only what it wrote itself
@@ -122,6 +139,8 @@ template <typename TD, typename TO>
 __global__ void add_rms_norm_f32res_vec4_kernel(
     float* __restrict__ residual, const TD* __restrict__ d0, long d0_stride,
     float s0, const TD* __restrict__ d1, long d1_stride, float s1,
+    const float* __restrict__ c0, const float* __restrict__ c1,
+    const int* __restrict__ index, const float* __restrict__ row_w, int top,
     const float* __restrict__ weight, float w_offset, float eps,
     TO* __restrict__ out, int width) {
   __shared__ float scratch[NW];
@@ -136,16 +155,33 @@ __global__ void add_rms_norm_f32res_vec4_kernel(
       float v[4], d[4];
       ld4<float>(r + i, v);
       if (d0) {
+        float c[4] = {1.f, 1.f, 1.f, 1.f};
         ld4<TD>(d0 + row * d0_stride + i, d);
+        if (c0) ld4<float>(c0 + i, c);
 #pragma unroll
-        for (int j = 0; j < 4; ++j) v[j] += s0 * d[j];
+        for (int j = 0; j < 4; ++j) v[j] += s0 * d[j] * c[j];
       }
       if (d1) {
-        ld4<TD>(d1 + row * d1_stride + i, d);
+        float c[4] = {1.f, 1.f, 1.f, 1.f};
+        if (index) {
+          float a[4] = {0.f, 0.f, 0.f, 0.f};
+          for (int q = 0; q < top; ++q) {
+            ld4<TD>(d1 + (long)index[row * top + q] * d1_stride + i, d);
+            const float w = row_w ? row_w[row * top + q] : 1.f;
 #pragma unroll
-        for (int j = 0; j < 4; ++j) v[j] += s1 * d[j];
+            for (int j = 0; j < 4; ++j) a[j] += w * d[j];
+          }
+#pragma unroll
+          for (int j = 0; j < 4; ++j) d[j] = a[j];
+        } else {
+          ld4<TD>(d1 + row * d1_stride + i, d);
+        }
+        if (c1) ld4<float>(c1 + i, c);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) v[j] += s1 * d[j] * c[j];
       }
       if (d0 || d1) st4<float>(r + i, v);
+      if (out && !weight) st4<TO>(out + row * width + i, v);
 #pragma unroll
       for (int j = 0; j < 4; ++j) {
         keep[k][j] = v[j];
@@ -153,8 +189,8 @@ __global__ void add_rms_norm_f32res_vec4_kernel(
       }
     }
   }
+  if (!out || !weight) return;
   ss = block_sum_sync<NW>(ss, scratch);
-  if (!out) return;
   const float inv = 1.0f / sqrtf(ss / (float)width + eps);
 #pragma unroll
   for (int k = 0; k < VEC_STEPS; ++k) {
@@ -721,23 +757,30 @@ extern "C" hipError_t ks_embed_scale_sinpos(void* out, const void* table,
 
 extern "C" hipError_t ks_add_rms_norm_f32res(
     void* residual, const void* d0, long d0_stride, float s0, const void* d1,
-    long d1_stride, float s1, const void* weight, float w_offset, float eps,
-    void* out, int rows, int width, int is_f32, int d_is_f32,
-    hipStream_t stream) {
+    long d1_stride, float s1, const void* c0, const void* c1,
+    const void* index, const void* row_w, int top, const void* weight,
+    float w_offset, float eps, void* out, int rows, int width, int is_f32,
+    int d_is_f32, hipStream_t stream) {
   if (rows == 0) return hipSuccess;
+  if (index && (!d1 || top < 1)) return hipErrorInvalidValue;
   const int esz = is_f32 ? 4 : 2;
   const int dsz = d_is_f32 ? 4 : 2;
   auto al = [](const void* p, int bytes) { return ((uintptr_t)p % bytes) == 0; };
   const bool vec = width % 4 == 0 && width <= NT * 4 * VEC_STEPS &&
                    d0_stride % 4 == 0 && d1_stride % 4 == 0 &&
-                   al(residual, 16) && al(weight, 16) && al(d0, 4 * dsz) &&
-                   al(d1, 4 * dsz) && al(out, 4 * esz);
+                   al(residual, 16) && al(weight, 16) && al(c0, 16) &&
+                   al(c1, 16) && al(d0, 4 * dsz) && al(d1, 4 * dsz) &&
+                   al(out, 4 * esz);
 #define NORM_ARGS(TT)                                                         \
   (float*)residual, (const TT*)d0, d0_stride, s0, (const TT*)d1, d1_stride,   \
-      s1, (const float*)weight, w_offset, eps, (TT*)out, width
+      s1, (const float*)c0, (const float*)c1, (const int*)index,              \
+      (const float*)row_w, top, (const float*)weight, w_offset, eps,          \
+      (TT*)out, width
 #define NORM_ARGS_MIXED                                                       \
   (float*)residual, (const float*)d0, d0_stride, s0, (const float*)d1,        \
-      d1_stride, s1, (const float*)weight, w_offset, eps, (short*)out, width
+      d1_stride, s1, (const float*)c0, (const float*)c1, (const int*)index,   \
+      (const float*)row_w, top, (const float*)weight, w_offset, eps,          \
+      (short*)out, width
   if (!is_f32 && d_is_f32) {
     // fp32 deltas (an fp32 sum of sublayer outputs) beside a bf16 output
     if (vec)

@@ -337,12 +337,22 @@ def embed_scale_sinpos(table, tokens, positions, inv_freq, scale: float):
 
 
 def add_rms_norm_f32res(
-    residual, weight, eps, w_offset, out_dtype, d0=None, s0=1.0, d1=None, s1=1.0
+    residual, weight, eps, w_offset, out_dtype, d0=None, s0=1.0, d1=None,
+    s1=1.0, c0=None, c1=None, d1_index=None, d1_weights=None, d1_top: int = 1,
+    want_out: bool = True,
 ):
     if d0 is not None:
-        residual += s0 * d0.float()
+        d = s0 * d0.float()
+        residual += d if c0 is None else d * c0
     if d1 is not None:
-        residual += s1 * d1.float()
+        if d1_index is not None:
+            d1 = combine_rows(d1, d1_index, d1_top, weights=d1_weights)
+        d = s1 * d1.float()
+        residual += d if c1 is None else d * c1
+    if not want_out:
+        return None
+    if weight is None:
+        return residual.to(out_dtype)
     inv = torch.rsqrt(residual.pow(2).mean(-1, keepdim=True) + eps)
     return (residual * inv * (w_offset + weight)).to(out_dtype)
 
@@ -454,6 +464,7 @@ def ctx_attention_f32(
     q, k_cache, v_cache, block_tables, cu_q, ctx_lens, scale: float,
     heads: int, gate=None, out_dtype=torch.float32, sink=None, chunk: int = 0,
     out_inv_freq=None, window: int = 0, maps: int = 1, softcap: float = 0.0,
+    keep_first: int = 0,
 ):
     _, G, bs, D = k_cache.shape
     D //= maps
@@ -484,7 +495,7 @@ def ctx_attention_f32(
         if chunk > 0:
             vis = vis & (kpos // chunk == qpos // chunk)
         if window > 0:
-            vis = vis & (qpos - kpos < window)
+            vis = vis & ((qpos - kpos < window) | (kpos < keep_first))
         sc = sc.masked_fill(~vis.unsqueeze(0), float("-inf"))
         if sink is None:
             w = torch.softmax(sc, dim=-1)
@@ -527,8 +538,10 @@ def qk_headnorm_rope_cache(
     q, k, v, qw, kw, positions, slot_mapping, k_cache, v_cache, eps,
     heads: int, qk_inv_freq, v_unit_norm: bool, v_inv_freq,
     pairs: bool = False, rot_mult: float = 1.0, maps: int = 1,
+    qk_norm: bool = True,
 ):
-    """Per-head RMS norm of q and k (weights [dim], shared by the heads),
+    """Per-head RMS norm of q and k (weights [dim], shared by the heads;
+    ``qk_norm`` off: none),
     rotary positions on their first 2*len(qk_inv_freq) coordinates (``pairs``:
     2i with 2i+1 instead of i with i + half; the turned coordinates times
     ``rot_mult``). ``maps`` heads of k share one cached row (and one value
@@ -543,8 +556,10 @@ def qk_headnorm_rope_cache(
     qf = q.float().reshape(T, heads, D)
     kf = k.float().reshape(T, G * maps, D)
     vf = v.float().reshape(T, G, DV)
-    qn = qf * torch.rsqrt(qf.pow(2).mean(-1, keepdim=True) + eps)
-    kn = kf * torch.rsqrt(kf.pow(2).mean(-1, keepdim=True) + eps)
+    qn, kn = qf, kf
+    if qk_norm:
+        qn = qf * torch.rsqrt(qf.pow(2).mean(-1, keepdim=True) + eps)
+        kn = kf * torch.rsqrt(kf.pow(2).mean(-1, keepdim=True) + eps)
     if qw is not None:
         qn = qn * qw
     if kw is not None:
@@ -595,17 +610,22 @@ def post_norm_add_rms_norm(
 def router_topk(
     logits, top: int, softmax: bool = False, renorm: bool = False,
     dense: bool = False, correction=None, renorm_eps: float = 0.0,
-    weight_scale: float = 1.0,
+    weight_scale: float = 1.0, over_chosen: bool = False,
 ):
     """Scores (sigmoid, or softmax over the experts) of fp32 router logits
     [T, E]; the ``top`` largest per token -> (indices int32 [T, top],
     weights fp32 [T, top], and with ``dense`` the same weights as a [T, E]
     matrix that is zero elsewhere), optionally renormalised to sum 1
     (divided by their sum + ``renorm_eps``). With ``correction`` [E] the
-    choice goes by score + correction while the weights stay the scores."""
+    choice goes by score + correction while the weights stay the scores.
+    ``over_chosen``: the largest logits are chosen and the weights are the
+    softmax over those logits only."""
     z = logits.float()
     s = torch.softmax(z, dim=-1) if softmax else torch.sigmoid(z)
-    if correction is None:
+    if over_chosen:
+        w, idx = z.topk(top, dim=-1)
+        w = torch.softmax(w, dim=-1)
+    elif correction is None:
         w, idx = s.topk(top, dim=-1)
     else:
         idx = (s + correction.float()).topk(top, dim=-1).indices
@@ -622,14 +642,15 @@ def route_tokens(
     h, router, top: int, softmax: bool = False, renorm: bool = False,
     dense: bool = False, want_logits: bool = False, correction=None,
     renorm_eps: float = 0.0, weight_scale: float = 1.0,
+    over_chosen: bool = False, bias=None,
 ):
-    """Router logits h @ router^T in fp32 (h in the activation dtype, router
-    fp32 [E, W]) followed by ``router_topk``; returns (indices, weights,
+    """Router logits h @ router^T (+ bias [E]) in fp32 (h in the activation
+    dtype, router fp32 [E, W]) followed by ``router_topk``; returns (indices, weights,
     dense weights or None, logits or None)."""
-    logits = torch.nn.functional.linear(h.float(), router.float())
+    logits = torch.nn.functional.linear(h.float(), router.float(), bias)
     idx, w, dw = router_topk(
         logits, top, softmax, renorm, dense, correction, renorm_eps,
-        weight_scale,
+        weight_scale, over_chosen,
     )
     return idx, w, dw, (logits if want_logits else None)
 
@@ -711,44 +732,66 @@ def rotate_pairs(x, positions, inv_freq):
     return out
 
 
+def rotate_by_layout(x, positions, inv_freq, pairs: bool, mult: float):
+    """``rotate_pairs`` or ``rotate_halves`` on x [T, heads, n] (or [T, n]),
+    the turned coordinates times ``mult``."""
+    if inv_freq is None:
+        return x
+    flat = x.dim() == 2
+    y = x.unsqueeze(1) if flat else x
+    n = 2 * inv_freq.numel()
+    y = (rotate_pairs if pairs else rotate_halves)(y, positions, inv_freq)
+    if mult != 1.0:
+        y = torch.cat([y[..., :n] * mult, y[..., n:]], dim=-1)
+    return y.squeeze(1) if flat else y
+
+
 def latent_norm_rope_cache(
     proj, q_rank: int, kv_rank: int, rot_dim: int, qw, kw, positions,
-    slot_mapping, cache, eps: float, inv_freq,
+    slot_mapping, cache, eps: float, inv_freq, pairs: bool = True,
+    rot_mult: float = 1.0,
 ):
     """proj [T, >= q_rank + kv_rank + rot_dim] = [query latent | kv latent |
     key part to rotate | ...]. Returns the RMS-normed query latent times
     ``qw`` in proj's dtype; writes [normed kv latent * kw | rotated key part]
     into ``cache`` [blocks, 1, block, kv_rank + rot_dim] at the tokens'
-    slots (negative slots are skipped). ``cache`` None: the query side only."""
-    x = proj[:, :q_rank].float()
-    cq = x * torch.rsqrt(x.pow(2).mean(-1, keepdim=True) + eps) * qw
+    slots (negative slots are skipped). ``cache`` None: the query side only;
+    ``q_rank`` 0: the cache side only (returns None). ``pairs`` off: the key
+    part turns in halves; turned coordinates times ``rot_mult``."""
+    cq = None
+    if q_rank:
+        x = proj[:, :q_rank].float()
+        cq = x * torch.rsqrt(x.pow(2).mean(-1, keepdim=True) + eps) * qw
     if cache is not None:
         c = proj[:, q_rank : q_rank + kv_rank].float()
         c = c * torch.rsqrt(c.pow(2).mean(-1, keepdim=True) + eps) * kw
         row = c
         if rot_dim:
             kr = proj[:, q_rank + kv_rank : q_rank + kv_rank + rot_dim].float()
-            row = torch.cat([c, rotate_pairs(kr, positions, inv_freq)], dim=-1)
+            kr = rotate_by_layout(kr, positions, inv_freq, pairs, rot_mult)
+            row = torch.cat([c, kr], dim=-1)
         bs = cache.shape[2]
         slots = slot_mapping[: proj.shape[0]].long()
         ok = slots >= 0
         cache[slots[ok] // bs, 0, slots[ok] % bs] = row[ok].to(cache.dtype)
-    return cq.to(proj.dtype)
+    return None if cq is None else cq.to(proj.dtype)
 
 
 def head_matmul_rope(
-    x, w, heads: int, tail: int, positions, inv_freq, out_dtype
+    x, w, heads: int, tail: int, positions, inv_freq, out_dtype,
+    pairs: bool = True, rot_mult: float = 1.0,
 ):
     """x [T, heads * (k + tail)], w [heads, n, k] -> [T, heads * (n + tail)]:
     per head the head's matrix times the first k coordinates (fp32 sums),
-    followed by the ``tail`` coordinates rotated in pairs by the token's
-    position (copied when ``inv_freq`` is None)."""
+    followed by the ``tail`` coordinates rotated in pairs (or halves) by the
+    token's position, times ``rot_mult`` (copied when ``inv_freq`` is None)."""
     T = x.shape[0]
     H, n, k = w.shape
     xh = x.reshape(T, heads, k + tail).float()
     y = torch.einsum("thk,hnk->thn", xh[..., :k], w.float())
     if tail:
-        y = torch.cat([y, rotate_pairs(xh[..., k:], positions, inv_freq)], dim=-1)
+        t = rotate_by_layout(xh[..., k:], positions, inv_freq, pairs, rot_mult)
+        y = torch.cat([y, t], dim=-1)
     return y.reshape(T, heads * (n + tail)).to(out_dtype)
 
 
@@ -804,6 +847,7 @@ def unit_norm_heads(x, heads_a, scale_a, heads_b, scale_b, dim, eps):
 def linear_scan(
     q, k, v, state, positions, cu_seqlens, slots, qk_heads, decay=None,
     a_raw=None, b_raw=None, a_log=None, dt_bias=None, channel_decay=None,
+    q_scale: float = 1.0,
 ):
     """Token-by-token form of the decay / gated-delta recurrences; state
     [slots, heads, V, K] fp32 is read (unless the portion starts at position
@@ -813,7 +857,10 @@ def linear_scan(
     rep = heads // qk_heads
     o = torch.empty(T, heads * V, dtype=torch.float32)
     cu = cu_seqlens.tolist()
-    if decay is None:
+    channel_only = channel_decay is not None and b_raw is None
+    if channel_only:
+        g_all = channel_decay.reshape(T, heads, 1, K)
+    elif decay is None:
         if channel_decay is not None:
             g_all = channel_decay.reshape(T, heads, 1, K)
         else:
@@ -830,9 +877,12 @@ def linear_scan(
             S.zero_()
         for t in range(a, b):
             qt = q[t].float().reshape(qk_heads, K).repeat_interleave(rep, dim=0)
+            qt = qt * q_scale
             kt = k[t].float().reshape(qk_heads, K).repeat_interleave(rep, dim=0)
             vt = v[t].float().reshape(heads, V)
-            if decay is not None:
+            if channel_only:
+                S = g_all[t] * S + vt[:, :, None] * kt[:, None, :]
+            elif decay is not None:
                 S = decay[:, None, None] * S + vt[:, :, None] * kt[:, None, :]
             else:
                 S = g_all[t] * S
@@ -882,6 +932,26 @@ def yarn_inv_freq(n_rot: int, base: float, scaling=None):
     ramp = ((i - lo) / max(hi - lo, 0.001)).clamp(0.0, 1.0)
     f = f / scaling["factor"] * ramp + f * (1.0 - ramp)
     return f.to(torch.float32), 0.1 * math.log(scaling["factor"]) + 1.0
+
+
+def scaled_inv_freq(n_rot: int, base: float, scaling=None):
+    """Frequencies and the factor on cos and sin for ``scaling`` None, linear
+    ({"factor"}: every frequency divided by it) or YaRN (has "original")."""
+    if scaling and "original" not in scaling:
+        i = torch.arange(n_rot // 2, dtype=torch.float64)
+        f = float(base) ** (-2.0 * i / n_rot) / scaling["factor"]
+        return f.to(torch.float32), 1.0
+    return yarn_inv_freq(n_rot, base, scaling)
+
+
+def lowrank_channel_decay(low, w2, bias, tau: float):
+    """sigmoid(z)^(1/tau) of z = low @ w2^T + bias, fp32 [T, n]."""
+    z = low.float() @ w2.t() + bias
+    return torch.exp(torch.nn.functional.logsigmoid(z) / tau)
+
+
+def linear_f32out(x, w):
+    return torch.nn.functional.linear(x.float(), w.float())
 
 
 def distance_buckets(count: int, buckets: int, bias_max: float) -> torch.Tensor:
