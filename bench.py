@@ -279,6 +279,58 @@ def _mededra_model_configs(size: dict):
     return mededra, laperax
 
 
+# layer shapes for --kebesun-compare: the widths, head counts, head sizes,
+# window and experts of LAPERAX_SIZES (an expert has three matrices instead of
+# two: two thirds of the columns), latent rows of 192 + 64 columns
+KEBESUN_SIZES = {
+    "2k": dict(laperax="2k", ff=2752, kv_rank=192, rot_dim=64, keep=64),
+    "4k": dict(laperax="4k", ff=4800, kv_rank=192, rot_dim=64, keep=64),
+}
+
+
+def _kebesun_model_configs(size: dict):
+    """A Kebesun model of four layer runs (gated linear attention run twice
+    over, windowed attention with kept first positions, latent attention;
+    experts beside every mixer) and the Laperax model that --laperax-compare
+    measures at the same width."""
+    from kserve_amd.engine.config import (
+        AttentionMixerSpec,
+        GatedLinearMixerSpec,
+        HybridLayerSpec,
+        HybridModelConfig,
+        LatentAttentionSpec,
+        LoopSpec,
+        SoftmaxMoESpec,
+    )
+
+    base = LAPERAX_SIZES[size["laperax"]]
+    H, D, R = base["heads"], base["head_dim"], size["rot_dim"]
+    moe = SoftmaxMoESpec(experts=base["experts"], top=base["top"], ff=size["ff"],
+                         over_chosen=True, router_bias=True)
+    gla = GatedLinearMixerSpec(heads=H, dim=D, vdim=D, tau=16.0, a_rank=16)
+    attn = AttentionMixerSpec(heads=H, kv_heads=base["kv_heads"], dim=D, vdim=D,
+                              scale=D ** -0.5, rot_dims=D, rot_base=1e4,
+                              window=base["window"], keep_first=size["keep"],
+                              rot_scaling={"factor": 2.0})
+    latent = LatentAttentionSpec(
+        heads=H, dim=D, vdim=D, kv_rank=size["kv_rank"], q_rank=0,
+        scale=(D + R) ** -0.5, rot_dim=R, rot_dims=R, rot_base=1e6,
+        rot_pairs=False,
+        rot_scaling={"factor": 4.0, "original": 2048, "fast": 32.0, "slow": 1.0},
+    )
+    kebesun = HybridModelConfig(
+        vocab_size=base["vocab"], hidden_size=base["width"],
+        layers=[
+            HybridLayerSpec("gla", gated_linear=gla, mlp=moe),
+            HybridLayerSpec("attention", attention=attn, mlp=moe),
+            HybridLayerSpec("latent_attention", latent=latent, mlp=moe),
+        ],
+        loop=LoopSpec(0, 1, 2), model_name="kebesun-bench", architecture="Kebesun",
+    )
+    laperax, _ = _laperax_model_configs(base)
+    return kebesun, laperax
+
+
 def _throughput(mcfg, prompt_len, n_prompts, concurrency, steps, warmup, eager):
     """(prefill tok/s, decode tok/s) through the engine's own step()."""
     import torch
@@ -578,6 +630,56 @@ def mededra_compare(args):
     return 0
 
 
+def kebesun_compare(args):
+    """Prefill and decode tok/s of the Kebesun design next to the Laperax
+    model of equal width and depth (the closest design the engine serves:
+    parallel layers of linear or windowed attention beside experts), both
+    through LLMEngine.step() on one GPU, bf16, random weights. One JSON line
+    per (size, model), each measured in a process of its own."""
+    import subprocess
+    import sys
+
+    if args.compare_only is None or "," in args.kebesun_compare:
+        rc = 0
+        for name in args.kebesun_compare.split(","):
+            for label in ("kebesun", "laperax"):
+                if args.compare_only and args.compare_only != label:
+                    continue
+                cmd = [sys.executable, "-u", os.path.abspath(__file__),
+                       "--kebesun-compare", name, "--compare-only", label,
+                       "--steps", str(args.steps), "--warmup", str(args.warmup),
+                       "--concurrency", str(args.concurrency),
+                       "--prompt-len", str(args.prompt_len)]
+                if args.eager:
+                    cmd.append("--eager")
+                rc = subprocess.call(cmd)
+                if rc != 0:
+                    return rc
+        return rc
+
+    import torch
+
+    assert torch.cuda.is_available(), "--kebesun-compare needs a GPU"
+    name, label = args.kebesun_compare, args.compare_only
+    kebesun, laperax = _kebesun_model_configs(KEBESUN_SIZES[name])
+    mcfg = kebesun if label == "kebesun" else laperax
+    prefill, decode = _throughput(
+        mcfg, prompt_len=args.prompt_len if args.prompt_len != 512 else 2048,
+        n_prompts=8, concurrency=min(args.concurrency, 256),
+        steps=args.steps, warmup=args.warmup, eager=args.eager,
+    )
+    print(json.dumps({
+        "bench": "kebesun-compare", "size": name, "model": mcfg.model_name,
+        "layer_runs": len(mcfg.layer_runs()), "width": mcfg.hidden_size,
+        "prefill_tok_s": round(prefill, 1),
+        "decode_tok_s": round(decode, 1),
+        "prefill_batch": "8 x prompt", "decode_concurrency":
+            min(args.concurrency, 256),
+        "dtype": "bfloat16", "data": "synthetic, random-init weights",
+    }), flush=True)
+    return 0
+
+
 def main():
     parser = argparse.ArgumentParser()
     parser.add_argument("--gpus", type=int, default=1)
@@ -642,11 +744,18 @@ def main():
                              "decode throughput of a Mededra-design model "
                              "beside the Laperax model of equal width and "
                              "depth (sizes: " + ", ".join(MEDEDRA_SIZES) + ")")
+    parser.add_argument("--kebesun-compare", type=str, default=None,
+                        metavar="SIZE[,SIZE...]",
+                        help="instead of the flagship workload: prefill and "
+                             "decode throughput of a Kebesun-design model "
+                             "beside the Laperax model of equal width and "
+                             "depth (sizes: " + ", ".join(KEBESUN_SIZES) + ")")
     parser.add_argument("--compare-only", type=str, default=None,
                         choices=["desalix", "llama", "voborax", "laperax",
-                                 "merulorn", "mededra"],
+                                 "merulorn", "mededra", "kebesun"],
                         help="with --desalix-compare / --voborax-compare / "
-                             "--laperax-compare / --mededra-compare: run one "
+                             "--laperax-compare / --mededra-compare / "
+                             "--kebesun-compare: run one "
                              "side only (e.g. under a profiler)")
     parser.add_argument("--profile-cpu", action="store_true",
                         help="cProfile the timed loop and print hot functions")
@@ -661,6 +770,8 @@ def main():
         return laperax_compare(args)
     if args.mededra_compare:
         return mededra_compare(args)
+    if args.kebesun_compare:
+        return kebesun_compare(args)
 
     import torch
 
