@@ -89,7 +89,7 @@ hipError_t ks_linear_scan(void*, const void*, long, const void*, long,
                           const void*, const void*, long, int, const void*,
                           const void*, const void*, void*, const void*,
                           const void*, const void*, int, int, int, int, int,
-                          hipStream_t);
+                          int, hipStream_t);
 hipError_t ks_lowrank_channel_decay(void*, const void*, long, const void*,
                                     const void*, float, int, int, int, int,
                                     hipStream_t);
@@ -1083,8 +1083,9 @@ void linear_scan(at::Tensor& o, at::Tensor& q, at::Tensor& k, at::Tensor& v,
                            v.stride(0), qkv_f32, (float)q_scale, dp, ap, bp,
                            ab_stride, ab_f32, alp, dtp, cdp,
                            state.data_ptr(), positions.data_ptr(),
-                           cu_seqlens.data_ptr(), slots.data_ptr(), num_seqs,
-                           heads, (int)qk_heads, V, K, current_stream()),
+                           cu_seqlens.data_ptr(), slots.data_ptr(), tokens,
+                           num_seqs, heads, (int)qk_heads, V, K,
+                           current_stream()),
             "linear_scan");
 }
 

@@ -35,6 +35,14 @@
 // flight. Grid = column tiles x heads x sequences: prefill portions and
 // single-token decode batches run the same kernel.
 //
+// The two decay forms have no correction by the old state, so a prompt portion
+// takes 16 tokens at a time on the fp32 matrix cores (decay_chunk_kernel).
+// With b_t the product of a chunk's decays up to token t (per key channel),
+//   O = (Q b) S + mask(Q b (K / b)^T) V,   S <- diag(b_16) (S + (K / b)^T V).
+// b_16 >= 2^-60 keeps every factor and product finite and each term's relative
+// error at a few roundings; a chunk with a channel below that walks its tokens
+// one by one on the same registers.
+//
 // Helpers for what precedes the recurrence:
 //  * rope_scale_heads: rotary positions on the first 2*half coordinates of
 //    every head (coordinate i pairs with i + half), times a constant, fp32
@@ -190,10 +198,13 @@ __global__ void __launch_bounds__(NT) lowrank_channel_decay_kernel(
 #pragma unroll
   for (int a = 0; a < DT; ++a) {
     if (a < cnt) {
-      // log sigmoid(z) = min(z, 0) - log(1 + exp(-|z|))
-      const float z = acc[a];
-      const float lg = fminf(z, 0.f) - log1pf(expf(-fabsf(z)));
-      out[(t0 + a) * n + c] = expf(lg * inv_tau);
+      // log2 sigmoid(z) = min(z, 0) log2(e) - log2(1 + exp(-|z|)). The
+      // logarithm's argument lies in [1, 2], so its absolute error is an ulp
+      // of 1, no more than what rounding the decay itself costs.
+      const float z2 = acc[a] * 1.44269504088896340736f;
+      const float lg = fminf(z2, 0.f) -
+                       __builtin_amdgcn_logf(1.0f + __builtin_amdgcn_exp2f(-fabsf(z2)));
+      out[(t0 + a) * n + c] = __builtin_amdgcn_exp2f(lg * inv_tau);
     }
   }
 }
@@ -384,6 +395,346 @@ linear_scan_kernel(
   }
 }
 
+typedef float f32x4 __attribute__((ext_vector_type(4)));
+
+// KT: 16-row tiles of the key dimension (K <= 16 KT). 256 threads; a block
+// takes 64 value columns of one head of one sequence, a wave 16 of them.
+//
+// State: s[kt], lane (li, lg) register r = S[k = 16 kt + 4 lg + r][v = li]. That
+// is the accumulator layout of v_mfma_f32_16x16x4_f32 (rows k, columns v) and
+// at the same time, with the contraction index of k-step r in lane group lg
+// standing for 4 lg + r, the A operand of O^T = S^T (Q b)^T. The products:
+//   O^T [v][t] += S^T (Q b)^T            A = s registers, B from LDS rows t
+//   P^T [s][t]  = (K / b) (Q b)^T        A, B from LDS rows; the waves share
+//                                        the key tiles and sum through LDS
+//   O^T [v][t] += V^T mask(P)^T          A = v registers, B = P^T registers
+//   S   [k][v] += (K / b)^T V            A from LDS (transposed), B = v registers
+// V never passes through LDS: lane (li, lg) register r is v[token 4 lg + r][li].
+//
+// Staging: thread (n, g) takes key channel n of tokens g KT .. g KT + KT - 1
+// (16 / KT threads per channel) and the decays of all 16 tokens. Tokens past
+// the end and channels past K count as decay 1, q = k = v = 0.
+// CHAN: per-channel decays, otherwise one constant per head.
+template <int KT, bool CHAN, typename TQ>
+__global__ void __launch_bounds__(NT)
+__attribute__((amdgpu_waves_per_eu(KT > 8 ? 1 : 2)))
+decay_chunk_kernel(
+    float* __restrict__ o, const TQ* __restrict__ q, long q_stride,
+    const TQ* __restrict__ k, long k_stride, const TQ* __restrict__ v,
+    long v_stride, float q_scale, const float* __restrict__ decay,
+    const float* __restrict__ channel_decay, float* __restrict__ state,
+    const long* __restrict__ positions, const int* __restrict__ cu_seqlens,
+    const int* __restrict__ slots, int heads, int qk_heads, int V, int K) {
+  constexpr int TC = 16;         // tokens per chunk
+  constexpr int KP = 16 * KT;
+  constexpr int KS = KP + 4;     // row strides that spread rows over the banks
+  constexpr int TS = TC + 4;
+  constexpr float MIN_PRODUCT = 8.67361737988403547e-19f;  // 2^-60
+  extern __shared__ float lds[];
+  float* Qb = lds;               // [TC][KS]  q b        (slow chunk: q)
+  float* Kb = Qb + TC * KS;      // [TC][KS]  k / b      (slow chunk: k)
+  float* Kt = Kb + TC * KS;      // [KP][TS]  (k / b)^T  (slow chunk: decays^T)
+  float* Bc = Kt + KP * TS;      // [KP]      b_16
+  float* Ps = Bc + KP;           // [NW][64][4] partial P^T
+  int* flag = reinterpret_cast<int*>(Ps + NW * WAVE_SIZE * 4);  // [NW]
+
+  const int s = blockIdx.z, h = blockIdx.y;
+  const int lane = threadIdx.x & 63;
+  // a scalar, so that what one wave skips is skipped by a scalar branch (the
+  // matrix instructions do not look at the execution mask)
+  const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+  const int li = lane & 15, lg = lane >> 4;
+  const int first = cu_seqlens[s];
+  const int len = cu_seqlens[s + 1] - first;
+  if (len <= 0) return;
+  const int hq = h / (heads / qk_heads);
+  const int inner = heads * V;
+  const int col = blockIdx.x * 64 + wave * 16;  // first value column of the wave
+  const bool vok = col + li < V;
+  const bool fresh = positions[first] == 0;
+  const float fixed = CHAN ? 1.f : decay[h];
+
+  // state rows are K floats; 4-element access where rows are aligned
+  float* sp = state + (((long)slots[s] * heads + h) * V + col + li) * K;
+  const bool kvec = K % 4 == 0;
+  f32x4 st[KT];
+#pragma unroll
+  for (int kt = 0; kt < KT; ++kt) {
+    const int m = 16 * kt + 4 * lg;
+    st[kt] = f32x4{0.f, 0.f, 0.f, 0.f};
+    if (vok && !fresh) {
+      if (kvec) {
+        if (m < K) st[kt] = *reinterpret_cast<const f32x4*>(sp + m);
+      } else {
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+          if (m + r < K) st[kt][r] = sp[m + r];
+      }
+    }
+  }
+
+  const int n = threadIdx.x % KP;
+  const int g = KP >= WAVE_SIZE ? wave * WAVE_SIZE / KP : threadIdx.x / KP;
+  const bool nok = n < K;
+  // A chunk's elements as they come from memory. The loads carry no condition
+  // (clamped indexes instead; what is out of range is replaced in convert())
+  // and nothing is computed from them in prefetch(), so all of them are in
+  // flight together; rows are addressed by scalars where the token is one.
+  float ra[TC];
+  TQ rq[KT], rk[KT], rv[4];
+  const unsigned nc = min(n, K - 1), vc = min(col + li, V - 1);
+  // rows of one chunk are less than 2^31 elements apart (the host checks)
+  const int a_row = heads * K, q_row = (int)q_stride, k_row = (int)k_stride,
+            v_row = (int)v_stride;
+  auto prefetch = [&](int t0) {
+    const int last = min(TC, len - t0) - 1;
+    const long t = first + t0;
+    if (CHAN) {
+      const float* ab = channel_decay + (t * heads + h) * K;
+#pragma unroll
+      for (int j = 0; j < TC; ++j) ra[j] = (ab + min(j, last) * a_row)[nc];
+    }
+    const TQ* qb = q + t * q_stride + (long)hq * K;
+    const TQ* kb = k + t * k_stride + (long)hq * K;
+#pragma unroll
+    for (int j = 0; j < KT; ++j) {
+      const int tk = min(g * KT + j, last);
+      rq[j] = (qb + tk * q_row)[nc];
+      rk[j] = (kb + tk * k_row)[nc];
+    }
+    const TQ* vb = v + t * v_stride + (long)h * V;
+#pragma unroll
+    for (int r = 0; r < 4; ++r)
+      rv[r] = vb[(unsigned)(min(4 * lg + r, last) * v_row) + vc];
+  };
+  // widened, q scaled, decay products up to this thread's tokens
+  float fq[KT], fk[KT], b[KT], prod;
+  f32x4 vv;
+  auto convert = [&](int t0) {
+    const int cnt = min(TC, len - t0);
+    // zero unless ok, without a branch
+    auto keep = [](float x, bool ok) {
+      return __builtin_bit_cast(float, __builtin_bit_cast(int, x) & (ok ? -1 : 0));
+    };
+#pragma unroll
+    for (int j = 0; j < TC; ++j) {
+      if (!CHAN) ra[j] = fixed;
+      ra[j] = nok && j < cnt ? ra[j] : 1.f;
+    }
+#pragma unroll
+    for (int j = 0; j < KT; ++j) {
+      const bool ok = nok && g * KT + j < cnt;
+      fq[j] = keep(ld_f32(rq, j) * q_scale, ok);
+      fk[j] = keep(ld_f32(rk, j), ok);
+    }
+#pragma unroll
+    for (int r = 0; r < 4; ++r)
+      vv[r] = keep(ld_f32(rv, r), vok && 4 * lg + r < cnt);
+    prod = 1.f;
+#pragma unroll
+    for (int j = 0; j < TC; ++j) {
+      prod *= ra[j];
+#pragma unroll
+      for (int i = 0; i < KT; ++i)
+        if (j % KT == i && j / KT == g) b[i] = prod;
+    }
+  };
+
+  prefetch(0);
+  convert(0);
+  for (int t0 = 0; t0 < len; t0 += TC) {
+    const int cnt = min(TC, len - t0);
+    // the last chunk fetches itself once more: no condition around the loads
+    const int tn = t0 + TC < len ? t0 + TC : t0;
+    const bool bad = !(prod >= MIN_PRODUCT);
+    __syncthreads();  // previous chunk consumed
+    float kb[KT];
+#pragma unroll
+    for (int i = 0; i < KT; ++i) {
+      kb[i] = fk[i] * __builtin_amdgcn_rcpf(b[i]);
+      Qb[(g * KT + i) * KS + n] = fq[i] * b[i];
+      Kb[(g * KT + i) * KS + n] = kb[i];
+    }
+    if constexpr (KT % 4 == 0) {
+#pragma unroll
+      for (int i = 0; i < KT; i += 4)
+        *reinterpret_cast<f32x4*>(Kt + n * TS + g * KT + i) =
+            f32x4{kb[i], kb[i + 1], kb[i + 2], kb[i + 3]};
+    } else {
+#pragma unroll
+      for (int i = 0; i < KT; ++i) Kt[n * TS + g * KT + i] = kb[i];
+    }
+    if (g == 0) Bc[n] = prod;
+    const bool wave_bad = __any(bad);
+    if (lane == 0) flag[wave] = wave_bad;
+    __syncthreads();
+    int slow = 0;
+#pragma unroll
+    for (int w = 0; w < NW; ++w) slow |= flag[w];
+    const f32x4 vcur = vv;
+
+    if (__builtin_amdgcn_readfirstlane(slow)) {
+      // every thread has read the flags before anything is overwritten
+      __syncthreads();
+#pragma unroll
+      for (int i = 0; i < KT; ++i) {
+        Qb[(g * KT + i) * KS + n] = fq[i];
+        Kb[(g * KT + i) * KS + n] = fk[i];
+      }
+      if (g == 0) {
+#pragma unroll
+        for (int j = 0; j < TC; ++j) Kt[n * TS + j] = ra[j];
+      }
+      __syncthreads();
+      for (int tk = 0; tk < cnt; ++tk) {
+        const int r4 = tk & 3;
+        const float vs = r4 == 0   ? vcur[0]
+                         : r4 == 1 ? vcur[1]
+                         : r4 == 2 ? vcur[2]
+                                   : vcur[3];
+        const float vt = __shfl(vs, (tk >> 2) * 16 + li, WAVE_SIZE);
+        float acc = 0.f;
+#pragma unroll
+        for (int kt = 0; kt < KT; ++kt) {
+          const int m = 16 * kt + 4 * lg;
+          const f32x4 qq = *reinterpret_cast<const f32x4*>(Qb + tk * KS + m);
+          const f32x4 kk = *reinterpret_cast<const f32x4*>(Kb + tk * KS + m);
+#pragma unroll
+          for (int r = 0; r < 4; ++r) {
+            st[kt][r] = st[kt][r] * Kt[(m + r) * TS + tk] + kk[r] * vt;
+            acc += qq[r] * st[kt][r];
+          }
+        }
+        acc += __shfl_xor(acc, 16, WAVE_SIZE);
+        acc += __shfl_xor(acc, 32, WAVE_SIZE);
+        if (lg == 0 && vok)
+          o[(long)(first + t0 + tk) * inner + (long)h * V + col + li] = acc;
+      }
+      prefetch(tn);
+      convert(tn);
+      continue;
+    }
+    prefetch(tn);
+
+    // Operands are read from LDS in groups ahead of their products (the
+    // scheduling barriers keep the compiler from moving each read back to its
+    // use, where every group of four products would wait for it).
+    constexpr int PN = (KT + NW - 1) / NW;  // key tiles of P^T per wave
+    const bool share = KT >= NW || wave < KT;
+    f32x4 pa[PN], pc[PN], cq[KT];
+#pragma unroll
+    for (int i = 0; i < PN; ++i) {
+      const int at = li * KS + 16 * (share ? wave + NW * i : 0) + 4 * lg;
+      pa[i] = *reinterpret_cast<const f32x4*>(Kb + at);
+      pc[i] = *reinterpret_cast<const f32x4*>(Qb + at);
+    }
+#pragma unroll
+    for (int kt = 0; kt < KT; ++kt)
+      cq[kt] = *reinterpret_cast<const f32x4*>(Qb + li * KS + 16 * kt + 4 * lg);
+    __builtin_amdgcn_sched_barrier(0);
+    // this wave's share of P^T and O^T from the old state: independent chains
+    f32x4 p = f32x4{0.f, 0.f, 0.f, 0.f}, oa = p, ob = p;
+    if (share) {
+#pragma unroll
+      for (int i = 0; i < PN; ++i)
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+          p = __builtin_amdgcn_mfma_f32_16x16x4f32(pa[i][r], pc[i][r], p, 0, 0, 0);
+    }
+#pragma unroll
+    for (int kt = 0; kt < KT; ++kt) {
+      oa = __builtin_amdgcn_mfma_f32_16x16x4f32(st[kt][0], cq[kt][0], oa, 0, 0, 0);
+      ob = __builtin_amdgcn_mfma_f32_16x16x4f32(st[kt][1], cq[kt][1], ob, 0, 0, 0);
+      oa = __builtin_amdgcn_mfma_f32_16x16x4f32(st[kt][2], cq[kt][2], oa, 0, 0, 0);
+      ob = __builtin_amdgcn_mfma_f32_16x16x4f32(st[kt][3], cq[kt][3], ob, 0, 0, 0);
+    }
+    *reinterpret_cast<f32x4*>(Ps + (wave * WAVE_SIZE + lane) * 4) = p;
+    f32x4 bc[KT];
+#pragma unroll
+    for (int kt = 0; kt < KT; ++kt) {
+      cq[kt] = *reinterpret_cast<const f32x4*>(Kt + (16 * kt + li) * TS + 4 * lg);
+      bc[kt] = *reinterpret_cast<const f32x4*>(Bc + 16 * kt + 4 * lg);
+    }
+    __builtin_amdgcn_sched_barrier(0);
+    // the state takes the chunk
+#pragma unroll
+    for (int r = 0; r < 4; ++r)
+#pragma unroll
+      for (int kt = 0; kt < KT; ++kt)
+        st[kt] = __builtin_amdgcn_mfma_f32_16x16x4f32(cq[kt][r], vcur[r], st[kt], 0, 0, 0);
+#pragma unroll
+    for (int kt = 0; kt < KT; ++kt) st[kt] *= bc[kt];
+    __syncthreads();
+    p = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int w = 0; w < NW; ++w)
+      p += *reinterpret_cast<const f32x4*>(Ps + (w * WAVE_SIZE + lane) * 4);
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const float m = 4 * lg + r <= li ? p[r] : 0.f;  // key token <= query token
+      if (r & 1) ob = __builtin_amdgcn_mfma_f32_16x16x4f32(vcur[r], m, ob, 0, 0, 0);
+      else oa = __builtin_amdgcn_mfma_f32_16x16x4f32(vcur[r], m, oa, 0, 0, 0);
+    }
+    oa += ob;
+    // the next chunk's loads are waited for ahead of this chunk's stores, so
+    // that no wait has to include the stores (the empty asm keeps the compiler
+    // from sinking the work behind them)
+    convert(tn);
+#pragma unroll
+    for (int i = 0; i < KT; ++i) asm volatile("" : "+v"(fq[i]), "+v"(fk[i]), "+v"(b[i]));
+#pragma unroll
+    for (int r = 0; r < 4; ++r) asm volatile("" : "+v"(vv[r]));
+    asm volatile("" : "+v"(prod));
+    if (li < cnt) {
+      float* orow = o + (long)(first + t0 + li) * inner + (long)h * V;
+      const int c0 = col + 4 * lg;
+      if (V % 4 == 0) {
+        if (c0 < V) *reinterpret_cast<f32x4*>(orow + c0) = oa;
+      } else {
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+          if (c0 + r < V) orow[c0 + r] = oa[r];
+      }
+    }
+  }
+#pragma unroll
+  for (int kt = 0; kt < KT; ++kt) {
+    const int m = 16 * kt + 4 * lg;
+    if (!vok) continue;
+    if (kvec) {
+      if (m < K) *reinterpret_cast<f32x4*>(sp + m) = st[kt];
+    } else {
+#pragma unroll
+      for (int r = 0; r < 4; ++r)
+        if (m + r < K) sp[m + r] = st[kt][r];
+    }
+  }
+}
+
+template <int KT, bool CHAN, typename TQ>
+hipError_t launch_decay_chunks(float* o, const TQ* q, long q_stride, const TQ* k,
+                               long k_stride, const TQ* v, long v_stride,
+                               float q_scale, const float* decay,
+                               const float* channel_decay, float* state,
+                               const long* positions, const int* cu_seqlens,
+                               const int* slots, int num_seqs, int heads,
+                               int qk_heads, int V, int K, hipStream_t stream) {
+  constexpr int KP = 16 * KT;
+  const size_t smem = sizeof(float) * (size_t)(2 * 16 * (KP + 4) + KP * 20 + KP +
+                                               NW * WAVE_SIZE * 4 + NW);
+  auto fn = decay_chunk_kernel<KT, CHAN, TQ>;
+  if (smem > 48 * 1024) {
+    hipError_t e = hipFuncSetAttribute(
+        (const void*)fn, hipFuncAttributeMaxDynamicSharedMemorySize, (int)smem);
+    if (e != hipSuccess) return e;
+  }
+  hipLaunchKernelGGL(fn, dim3(cdiv(V, 64), heads, num_seqs), dim3(NT), smem,
+                     stream, o, q, q_stride, k, k_stride, v, v_stride, q_scale,
+                     decay, channel_decay, state, positions, cu_seqlens, slots,
+                     heads, qk_heads, V, K);
+  return hipGetLastError();
+}
+
 }  // namespace
 
 extern "C" hipError_t ks_rope_scale_heads(void* out, const void* in,
@@ -508,7 +859,8 @@ extern "C" hipError_t ks_linear_scan(
     const void* b_raw, long ab_stride, int ab_is_f32, const void* a_log,
     const void* dt_bias, const void* channel_decay, void* state,
     const void* positions, const void* cu_seqlens, const void* slots,
-    int num_seqs, int heads, int qk_heads, int V, int K, hipStream_t stream) {
+    int tokens, int num_seqs, int heads, int qk_heads, int V, int K,
+    hipStream_t stream) {
   if (num_seqs == 0) return hipSuccess;
   if (qk_heads <= 0 || heads % qk_heads != 0 || K < 1 || K > 256 || V < 1)
     return hipErrorInvalidValue;
@@ -518,6 +870,28 @@ extern "C" hipError_t ks_linear_scan(
     return hipErrorInvalidValue;
   if (!qkv_is_f32 && !chan) return hipErrorInvalidValue;
   const int R = cdiv(K, 16);
+  // more tokens than sequences: prompt portions, in chunks on the matrix cores
+  if ((decay || chan) && tokens > num_seqs) {
+#define CHUNK_ARGS(TT)                                                        \
+  (float*)o, (const TT*)q, q_stride, (const TT*)k, k_stride, (const TT*)v,    \
+      v_stride, q_scale, (const float*)decay, (const float*)channel_decay,    \
+      (float*)state, (const long*)positions, (const int*)cu_seqlens,          \
+      (const int*)slots, num_seqs, heads, qk_heads, V, K, stream
+#define CHUNK_LAUNCH(CC, TT)                                                  \
+  do {                                                                        \
+    if (R <= 1) return launch_decay_chunks<1, CC, TT>(CHUNK_ARGS(TT));        \
+    if (R <= 2) return launch_decay_chunks<2, CC, TT>(CHUNK_ARGS(TT));        \
+    if (R <= 4) return launch_decay_chunks<4, CC, TT>(CHUNK_ARGS(TT));        \
+    if (R <= 8) return launch_decay_chunks<8, CC, TT>(CHUNK_ARGS(TT));        \
+    return launch_decay_chunks<16, CC, TT>(CHUNK_ARGS(TT));                   \
+  } while (0)
+    if (q_stride > (1 << 26) || k_stride > (1 << 26) || v_stride > (1 << 26) ||
+        (long)heads * K > (1 << 26))
+      return hipErrorInvalidValue;
+    if (!qkv_is_f32) CHUNK_LAUNCH(true, short);
+    if (chan) CHUNK_LAUNCH(true, float);
+    CHUNK_LAUNCH(false, float);
+  }
   int pc = V > 32 ? 4 : (V > 16 ? 2 : 1);
   if (R > 8 && pc > 2) pc = 2;
   // a block walks its tokens one after the other, so a launch with few

@@ -197,6 +197,28 @@ class TestGatedLinearScan:
                 at += n
             close(torch.cat(got), want, be, f32_tol=1e-5, bf16_tol=1e-5)
 
+    @pytest.mark.parametrize("H,K,V", [(2, 16, 20), (1, 100, 64), (2, 130, 66)])
+    def test_decays_of_any_size(self, be, H, K, V):
+        """Decays from 1 down to 0, changing from token to token: stretches in
+        which a channel's product falls below anything a quotient of products
+        could bear, next to ordinary ones."""
+        T = 100
+        q, k, v, a = self._inputs(T, H, K, V, be, seed=33)
+        z = rnd(T, H * K, seed=37, scale=4.0)
+        z[20:30] = 9.0            # no decay at all
+        z[40:44, ::3] = -60.0
+        z[70, 1] = -300.0         # one channel forgets everything at one token
+        a = torch.sigmoid(z.double()).float()
+        a[75, 0] = 0.0
+        want = self._oracle(q, k, v, a, H, K ** -0.5)
+        state = torch.full((2, H, V, K), 1e6).to(be[0])
+        for cuts in ([T], [1] * T, [3, 60, 2, 35]):
+            got, at = [], 0
+            for n in cuts:
+                got.append(self._run(be, [((q, k, v, a), at, n, 1)], state))
+                at += n
+            close(torch.cat(got), want, be, f32_tol=1e-5, bf16_tol=1e-5)
+
     def test_unequal_batch_and_slot_reuse(self, be):
         H, K, V = 2, 16, 8
         seqs = [self._inputs(n, H, K, V, be, seed=40 + 5 * i) for i, n in enumerate((30, 12, 21))]
