@@ -5,8 +5,8 @@ A layer is parallel: with h = norm1(x),
 
     x += ls1 * mixer(h) + ls2 * ff(h)
 
-— one RMS norm whose weight is stored around zero, both sublayers read its
-output, each result has a factor per channel. Mixers: ``GatedLinearMixer``
+— one RMS norm (gain 1 + w per channel) read by both sublayers, and a factor
+per channel on each result. Mixers: ``GatedLinearMixer``
 ("gla"), ``LatentAttention`` with directly projected queries and a half-split
 YaRN rotation ("latent_attention"), and sliding-window softmax attention that
 keeps the first positions visible (``RotaryChunkSinkAttention`` without norms
@@ -189,7 +189,7 @@ class KebesunForCausalLM(nn.Module):
                 p.fill_(0.5)
             elif leaf in ("kv_norm", "norm_w"):
                 p.fill_(1.0)
-            else:  # norms stored around zero, biases
+            else:  # norm gains (their distance from one), biases
                 p.normal_(0.0, 0.1, generator=gen)
         return self
 
@@ -216,8 +216,8 @@ class KebesunForCausalLM(nn.Module):
         return self._add(x, self.final_norm, pending)
 
     def _add(self, x, weight, pending, want_out: bool = True):
-        """The stream takes what is pending; returns its norm (``weight``
-        stored around zero), or the stream itself in the activation dtype."""
+        """The stream takes what is pending; returns its norm (gain
+        1 + ``weight``), or the stream itself in the activation dtype."""
         return ops.add_rms_norm_f32res(
             x, weight, self.eps, 1.0, self.dtype, want_out=want_out, **pending
         )
