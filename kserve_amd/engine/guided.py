@@ -32,7 +32,11 @@ AFTER_VALUE = 5        # value finished; container decides what's next
 EXPECT_KEY = 6         # inside object, before a key string
 EXPECT_COLON = 7
 DONE = 8               # top-level value complete
+NEXT_KEY = 9           # after a comma in an object: a key has to follow
+NEXT_VALUE = 10        # after a comma in an array: a value has to follow
+IN_UNICODE = 11        # hex digits of a \u escape (count in ``lit_pos``)
 
+HEX_DIGITS = frozenset(b"0123456789abcdefABCDEF")
 WS = frozenset(b" \t\n\r")
 DIGITS = frozenset(b"0123456789")
 NUMBER_BODY = frozenset(b"0123456789+-.eE")
@@ -106,10 +110,21 @@ class JsonMachine:
                 return True
             return b >= 0x20  # control bytes banned; UTF-8 bytes pass
         if s == IN_STRING_ESCAPE:
+            if b == 0x75:  # u: four hex digits follow
+                self.state = IN_UNICODE
+                self.lit_pos = 0
+                return True
             if b in STRING_ESCAPES:
                 self.state = IN_STRING
                 return True
             return False
+        if s == IN_UNICODE:
+            if b not in HEX_DIGITS:
+                return False
+            self.lit_pos += 1
+            if self.lit_pos == 4:
+                self.state = IN_STRING
+            return True
         if s == IN_NUMBER:
             ns = self.lit_pos
             if b in DIGITS:
@@ -152,7 +167,7 @@ class JsonMachine:
                     self._finish_value()
                 return True
             return False
-        if s == EXPECT_VALUE:
+        if s in (EXPECT_VALUE, NEXT_VALUE):
             if b in WS:
                 return True
             if self.object_only and not self.stack and b != 0x7B:
@@ -182,20 +197,26 @@ class JsonMachine:
                     self.lit = lit
                     self.lit_pos = 1
                     return True
-            if b == 0x5D and self.stack and self.stack[-1] == 0x5B:
+            if (
+                b == 0x5D and s == EXPECT_VALUE
+                and self.stack and self.stack[-1] == 0x5B
+            ):
                 # empty array "[]"
                 self.stack.pop()
                 self._finish_value()
                 return True
             return False
-        if s == EXPECT_KEY:
+        if s in (EXPECT_KEY, NEXT_KEY):
             if b in WS:
                 return True
             if b == 0x22:
                 self.state = IN_STRING
                 self.key_mode = True
                 return True
-            if b == 0x7D and self.stack and self.stack[-1] == 0x7B:
+            if (
+                b == 0x7D and s == EXPECT_KEY
+                and self.stack and self.stack[-1] == 0x7B
+            ):
                 # empty object "{}"
                 self.stack.pop()
                 self._finish_value()
@@ -213,7 +234,7 @@ class JsonMachine:
                 return True
             top = self.stack[-1] if self.stack else 0
             if b == 0x2C:  # ,
-                self.state = EXPECT_KEY if top == 0x7B else EXPECT_VALUE
+                self.state = NEXT_KEY if top == 0x7B else NEXT_VALUE
                 return True
             if b == 0x7D and top == 0x7B:
                 self.stack.pop()
@@ -376,7 +397,8 @@ class _FixedFrame:
 class _StringFrame:
     """'"' body '"' with escape handling; any UTF-8 content."""
 
-    __slots__ = ("state",)  # 0=open quote, 1=body, 2=escape
+    # 0=open quote, 1=body, 2=escape, 3..6=hex digits of a \u escape
+    __slots__ = ("state",)
 
     def __init__(self, state: int = 0):
         self.state = state
@@ -400,6 +422,14 @@ class _StringFrame:
                 self.state = 2
                 return _CONSUME
             return _CONSUME if b >= 0x20 else _ILLEGAL
+        if self.state >= 3:
+            if b not in HEX_DIGITS:
+                return _ILLEGAL
+            self.state = self.state + 1 if self.state < 6 else 1
+            return _CONSUME
+        if b == 0x75:  # u: four hex digits follow
+            self.state = 3
+            return _CONSUME
         if b in STRING_ESCAPES:
             self.state = 1
             return _CONSUME

@@ -51,6 +51,22 @@ def test_json_machine_walks_produce_valid_json(rng_bytes):
         assert check.advance(b)
 
 
+def test_comma_needs_a_successor_and_unicode_escapes_their_digits():
+    def accepts(text):
+        m = JsonMachine()
+        return m.accepts(text) and m.complete
+
+    for good in (b'{}', b'{"a":[]}', b'{"a":[1,2]}', b'{"a":1,"b":2}', b'{"a":"\\u00e9x"}'):
+        assert accepts(good), good
+        json.loads(good)
+    for bad in (b'{"a":1,}', b'{"a":[1,]}', b'{"a":[1, ]}', b'{"a":"\\u00g9"}', b'{"a":"\\u12"}'):
+        assert not accepts(bad), bad
+    m = SchemaMachine({"type": "object", "properties": {"s": {"type": "string"}}, "required": ["s"]})
+    assert all(m.advance(b) for b in b'{"s":"\\u00e9"}') and m.complete
+    m = SchemaMachine({"type": "object", "properties": {"s": {"type": "string"}}, "required": ["s"]})
+    assert not all(m.advance(b) for b in b'{"s":"\\u0"')
+
+
 SCHEMAS = [
     {"type": "object",
      "properties": {"name": {"type": "string"},
